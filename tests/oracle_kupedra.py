@@ -1,0 +1,296 @@
+"""A plain, slow float64 implementation of the Kupedra decoder, one function per mechanism, written from the
+model's equations and sharing no code with distributed_llms_amd: whole sequences only, Python loops, no
+cache, no batching.  The tests compare the engine against it.
+
+The model: several residual streams that all start as the scaled token embedding; a sublayer reads one
+weighted sum of them (normed by a scalar-weight RMS norm), its output is written back to every stream with a
+weight per stream while the streams are mixed by a small matrix; at the end the streams are summed.  Two kinds
+of layer: "attention" (rotated queries and keys that are normed AFTER the rotation, a temperature per head, a
+softmax with one added to its denominator) and "parallel" (attention with weighted query / key norms, a
+query temperature that grows with the position, a learned bias per distance bucket and a learned sink, beside
+a matrix memory with exponential gates; the two outputs are normed apart and averaged).  Feed-forward: a
+mixture of clipped-GLU experts weighted by a softmax over ALL experts that is not renormalised, and a shared
+expert with a gate of its own.  A span of the layers may run several times with the same weights.
+
+Checkpoint names: embed, final.norm, head, l<i>.norm1, l<i>.norm2, l<i>.hc1.*, l<i>.hc2.*, l<i>.mix.*,
+l<i>.mlp.*.  Linear weights are [out, in].
+"""
+import math
+
+import numpy as np
+
+
+def rms(x, eps):
+    """x / sqrt(mean(x^2) + eps) over the last axis."""
+    return x / np.sqrt((x * x).mean(-1, keepdims=True) + eps)
+
+
+def sigmoid(z):
+    return 1.0 / (1.0 + np.exp(-z))
+
+
+def log_sigmoid(z):
+    return -np.logaddexp(0.0, -z)
+
+
+def sub(w, prefix):
+    """The tensors under ``prefix`` with the prefix taken off."""
+    return {k[len(prefix):]: v for k, v in w.items() if k.startswith(prefix)}
+
+
+# ------------------------------------------------------------------------------ streams
+def hyper_connected(streams, hc, sublayer):
+    """streams [S, T, W]: the sublayer reads sum_s in_s x_s; stream t becomes sum_s mix[s, t] x_s + out_t y."""
+    u = np.zeros_like(streams[0])
+    for s in range(len(streams)):
+        u += hc["in"][s] * streams[s]
+    y = sublayer(u)
+    new = np.zeros_like(streams)
+    for t in range(len(streams)):
+        new[t] = hc["out"][t] * y
+        for s in range(len(streams)):
+            new[t] += hc["mix"][s, t] * streams[s]
+    return new
+
+
+# ------------------------------------------------------------------------------ attention
+def rotate_pairs(x, rot, first_pos=0):
+    """x [T, heads, D]: dimensions 2i and 2i + 1 (2i < dims) turn by p * base^(-2i / dims) / factor."""
+    out = x.copy()
+    factor = (rot.get("scaling") or {}).get("factor", 1.0)
+    p = (first_pos + np.arange(x.shape[0]))[:, None]
+    for i in range(rot["dims"] // 2):
+        a = p * (rot["base"] ** (-2.0 * i / rot["dims"]) / factor)
+        u, v = x[:, :, 2 * i], x[:, :, 2 * i + 1]
+        out[:, :, 2 * i] = u * np.cos(a) - v * np.sin(a)
+        out[:, :, 2 * i + 1] = v * np.cos(a) + u * np.sin(a)
+    return out
+
+
+def bucket(n, rows, far):
+    """Row of the distance-bias table for a key ``n`` positions back: one row per distance up to half the
+    table, then rows whose width grows geometrically until ``far``; everything beyond shares the last row."""
+    half = rows // 2
+    if n < half:
+        return n
+    return min(rows - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (rows - half)))
+
+
+def query_temperature(pos, qt):
+    """1 + coef ln(floor((p + 1) / every) + 1)."""
+    return 1.0 + qt["coef"] * np.log(np.floor((pos + 1) / qt["every"]) + 1.0)
+
+
+def softmax_attention(q, k, v, scale, sink, bias=None):
+    """q [T, H, D], k [T, G, D], v [T, G, Dv]; causal; the denominator also holds exp(sink[h]); ``bias`` [T, H]:
+    added to the score of a key ``n`` positions back."""
+    t, hh, _ = q.shape
+    rep = hh // k.shape[1]
+    out = np.zeros((t, hh, v.shape[2]))
+    for a in range(hh):
+        kv = a // rep
+        for i in range(t):
+            s = (k[:i + 1, kv] @ q[i, a]) * scale
+            if bias is not None:
+                s = s + bias[i - np.arange(i + 1), a]
+            top = max(s.max(), sink[a])
+            e = np.exp(s - top)
+            out[i, a] = (e @ v[:i + 1, kv]) / (e.sum() + math.exp(sink[a] - top))
+    return out
+
+
+def attention_mixer(h, w, m, eps):
+    """h [T, W]; w: q, k, v, temp, o; m: heads, kv_heads, dim, vdim, rot, scale."""
+    t = h.shape[0]
+    hh, g, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q = rms(rotate_pairs((h @ w["q"].T).reshape(t, hh, d), m["rot"]), eps)
+    k = rms(rotate_pairs((h @ w["k"].T).reshape(t, g, d), m["rot"]), eps)
+    v = (h @ w["v"].T).reshape(t, g, dv)
+    # exp(0) = 1 is the added term of the denominator
+    o = softmax_attention(q * w["temp"][None, :, None], k, v, m["scale"], np.zeros(hh))
+    return o.reshape(t, hh * dv) @ w["o"].T
+
+
+def biased_attention(h, w, m, eps):
+    """h [T, W]; w: q, k, v, q.norm, k.norm, rel, sink, o; m: heads, kv_heads, dim, vdim, scale, q_temp, bias_max."""
+    t = h.shape[0]
+    hh, g, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q = rms((h @ w["q"].T).reshape(t, hh, d), eps) * w["q.norm"]
+    k = rms((h @ w["k"].T).reshape(t, g, d), eps) * w["k.norm"]
+    v = (h @ w["v"].T).reshape(t, g, dv)
+    if m.get("q_temp"):
+        q = q * query_temperature(np.arange(t), m["q_temp"])[:, None, None]
+    bias = np.stack([w["rel"][bucket(n, w["rel"].shape[0], m["bias_max"])] for n in range(t)])
+    o = softmax_attention(q, k, v, m["scale"], w["sink"], bias)
+    return o.reshape(t, hh * dv) @ w["o"].T
+
+
+# ------------------------------------------------------------------------------ matrix memory
+def memory_scan(q, k, v, i_gate, f_gate):
+    """One head.  q, k [T, dim], v [T, vdim], i_gate / f_gate [T]: the log input and log forget gates.
+    S <- exp(f + m' - m) S + exp(i - m) k v^T with the running maximum m = max(f + m', i) (0 before the first
+    token), n the same with k alone; o = S^T q / (max(|n.q|, exp(-m)) + 1e-6).  Returns o [T, vdim]."""
+    s, n, m = np.zeros((q.shape[1], v.shape[1])), np.zeros(q.shape[1]), 0.0
+    o = np.zeros_like(v)
+    for t in range(q.shape[0]):
+        m_new = max(f_gate[t] + m, i_gate[t])
+        keep, put = math.exp(f_gate[t] + m - m_new), math.exp(i_gate[t] - m_new)
+        m = m_new
+        s = keep * s + put * np.outer(k[t], v[t])
+        n = keep * n + put * k[t]
+        o[t] = (s.T @ q[t]) / (max(abs(n @ q[t]), math.exp(-m)) + 1e-6)
+    return o
+
+
+def capped(z, cap):
+    return cap * np.tanh(z / cap)
+
+
+def memory_mixer(h, w, m, eps):
+    """h [T, W]; w: q, k, v, g, o, norm, i, i.b, f, f.b; m: heads, dim, vdim, gate_cap."""
+    t = h.shape[0]
+    hh, d, dv = m["heads"], m["dim"], m["vdim"]
+    q = (h @ w["q"].T).reshape(t, hh, d) * d ** -0.5
+    k = (h @ w["k"].T).reshape(t, hh, d)
+    v = (h @ w["v"].T).reshape(t, hh, dv)
+    ig = capped(h @ w["i"].T + w["i.b"], m["gate_cap"])
+    fg = log_sigmoid(capped(h @ w["f"].T + w["f.b"], m["gate_cap"]))
+    o = np.stack([memory_scan(q[:, a], k[:, a], v[:, a], ig[:, a], fg[:, a]) for a in range(hh)], 1)
+    y = rms(o, eps).reshape(t, hh * dv) * w["norm"] * sigmoid(h @ w["g"].T)
+    return y @ w["o"].T
+
+
+def parallel_mixer(h, w, m, eps):
+    left = biased_attention(h, sub(w, "left."), m["left"], eps)
+    right = memory_mixer(h, sub(w, "right."), m["right"], eps)
+    return 0.5 * (rms(left, eps) * w["left.out"] + rms(right, eps) * w["right.out"])
+
+
+# ------------------------------------------------------------------------------ feed-forward
+def clipped_expert(h, w, limit):
+    g = np.minimum(h @ w["gate"].T, limit)
+    u = np.clip(h @ w["up"].T, -limit, limit)
+    return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w["down"].T
+
+
+def route(z, top):
+    """z [E] router logits -> (indices of the ``top`` largest, their softmax over ALL E)."""
+    e = np.exp(z - z.max())
+    p = e / e.sum()
+    idx = np.argsort(-z, kind="stable")[:top]
+    return idx, p[idx]
+
+
+def moe_ff(h, w, mlp, margins=None):
+    """``margins``: a list that receives, per token, the gap between the last chosen logit and the best one
+    left out (how far the choice is from turning over)."""
+    out = np.zeros_like(h)
+    z = h @ w["router"].T
+    top, limit = mlp["router"]["top"], mlp["expert"]["limit"]
+    if margins is not None:
+        zs = -np.sort(-z, axis=-1)
+        margins.append(zs[:, top - 1] - zs[:, top] if top < z.shape[1] else np.full(h.shape[0], np.inf))
+    weight = np.zeros_like(z)
+    for i in range(h.shape[0]):
+        idx, p = route(z[i], top)
+        weight[i, idx] = p
+    for j in range(z.shape[1]):
+        rows = np.nonzero(weight[:, j])[0]
+        if len(rows):
+            out[rows] += weight[rows, j, None] * clipped_expert(h[rows], sub(w, f"e{j}."), limit)
+    if mlp.get("shared"):
+        gate = sigmoid(h @ w["shared.sg"].T)
+        out += gate * clipped_expert(h, sub(w, "shared."), mlp["shared"]["limit"])
+    return out
+
+
+# ------------------------------------------------------------------------------ the model
+def layer_runs(cfg):
+    """Layer indices in the order in which they run."""
+    n, loop = len(cfg["layers"]), cfg.get("loop")
+    if not loop:
+        return list(range(n))
+    return list(range(loop["start"])) + list(range(loop["start"], loop["stop"])) * loop["times"] + list(range(loop["stop"], n))
+
+
+def forward(cfg, sd, tokens, taps=None, margins=None):
+    """Logits [T, vocab] of one whole sequence.  ``sd``: checkpoint name -> float64 array.  ``taps``: a list that
+    receives the sum of the streams after every layer run; ``margins``: one that receives every router's."""
+    eps = cfg["norm"]["eps"]
+    e = sd["embed"][np.asarray(tokens)] * cfg["embedding"]["scale"]
+    x = np.stack([e] * cfg["streams"])
+    for i in layer_runs(cfg):
+        layer, w = cfg["layers"][i], sub(sd, f"l{i}.")
+        mixer = attention_mixer if layer["type"] == "attention" else parallel_mixer
+        x = hyper_connected(x, sub(w, "hc1."), lambda u: mixer(rms(u, eps) * w["norm1"], sub(w, "mix."), layer["mixer"], eps))
+        if layer.get("mlp"):
+            x = hyper_connected(x, sub(w, "hc2."),
+                                lambda u: moe_ff(rms(u, eps) * w["norm2"], sub(w, "mlp."), layer["mlp"], margins))
+        if taps is not None:
+            taps.append(x.sum(0))
+    return (rms(x.sum(0), eps) * sd["final.norm"]) @ sd["head"].T * cfg["logit_scale"]
+
+
+def shapes(cfg):
+    """Checkpoint name -> shape.  ``mixer.left.rows`` (default 8) is the row count of the distance-bias table."""
+    w, ns = cfg["width"], cfg["streams"]
+    s = {"embed": (cfg["vocab"], w), "final.norm": (), "head": (cfg["vocab"], w)}
+    for i, layer in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        m = layer["mixer"]
+        mlp = layer.get("mlp")
+        for q in (1, 2) if mlp else (1,):
+            s.update({p + f"norm{q}": (), p + f"hc{q}.in": (ns,), p + f"hc{q}.out": (ns,), p + f"hc{q}.mix": (ns, ns)})
+        a, pa = (m, p + "mix.") if layer["type"] == "attention" else (m["left"], p + "mix.left.")
+        s.update({pa + "q": (a["heads"] * a["dim"], w), pa + "k": (a["kv_heads"] * a["dim"], w),
+                  pa + "v": (a["kv_heads"] * a["vdim"], w), pa + "o": (w, a["heads"] * a["vdim"])})
+        if layer["type"] == "attention":
+            s[pa + "temp"] = (a["heads"],)
+        else:
+            s.update({pa + "q.norm": (a["dim"],), pa + "k.norm": (a["dim"],), pa + "sink": (a["heads"],),
+                      pa + "rel": (a.get("rows", 8), a["heads"]), p + "mix.left.out": (w,), p + "mix.right.out": (w,)})
+            r, pr = m["right"], p + "mix.right."
+            qk, vv = r["heads"] * r["dim"], r["heads"] * r["vdim"]
+            s.update({pr + "q": (qk, w), pr + "k": (qk, w), pr + "v": (vv, w), pr + "g": (vv, w), pr + "o": (w, vv),
+                      pr + "norm": (vv,), pr + "i": (r["heads"], w), pr + "i.b": (r["heads"],), pr + "f": (r["heads"], w),
+                      pr + "f.b": (r["heads"],)})
+        if mlp:
+            e, f = mlp["router"]["experts"], mlp["expert"]["ff"]
+            s[p + "mlp.router"] = (e, w)
+            for j in range(e):
+                s.update({p + f"mlp.e{j}.gate": (f, w), p + f"mlp.e{j}.up": (f, w), p + f"mlp.e{j}.down": (w, f)})
+            if mlp.get("shared"):
+                fs = mlp["shared"]["ff"]
+                s.update({p + "mlp.shared.gate": (fs, w), p + "mlp.shared.up": (fs, w), p + "mlp.shared.down": (w, fs),
+                          p + "mlp.shared.sg": (1, w)})
+    return s
+
+
+def make_weights(cfg, seed=0):
+    """Random float64 weights under the checkpoint names: projections ~ N(0, 1 / fan_in), norm weights and
+    temperatures around one, distance biases and sinks of moderate size, gates that keep a memory for a while,
+    stream mixes near the identity, a router wide enough that few choices are close calls."""
+    rng = np.random.default_rng(seed)
+    sd = {}
+    for name, shape in shapes(cfg).items():
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf in ("norm1", "norm2", "norm", "temp") or leaf == "out" and ".mix." in name:
+            t = 1.0 + 0.2 * rng.standard_normal(shape)
+        elif leaf in ("in", "out") and ".hc" in name:
+            t = (1.0 if leaf == "out" else 1.0 / shape[0]) + 0.3 * rng.standard_normal(shape)
+        elif leaf == "mix":
+            t = np.eye(shape[0]) * 0.8 + 0.15 * rng.standard_normal(shape)
+        elif leaf in ("rel", "sink"):
+            t = rng.standard_normal(shape)
+        elif name.endswith("i.b"):
+            t = 0.5 * rng.standard_normal(shape)
+        elif name.endswith("f.b"):
+            t = 3.0 + rng.standard_normal(shape)
+        elif leaf == "router":
+            t = 4.0 * rng.standard_normal(shape) / shape[-1] ** 0.5
+        elif name == "embed":
+            t = rng.standard_normal(shape) / cfg["embedding"]["scale"]
+        else:
+            t = rng.standard_normal(shape) / shape[-1] ** 0.5
+        sd[name] = np.asarray(t, dtype=np.float64)
+    return sd
