@@ -22,7 +22,7 @@ from typing import Any, Dict, List, Optional
 @dataclass
 class ModelConfig:
     name: str
-    arch: str                      # "llama" (Llama-2/3), "mixtral", "gpt2"; layer-list models: "tudilix", "gikovik", "zebutar", "fekizen"
+    arch: str                      # "llama" (Llama-2/3), "mixtral", "gpt2"; layer-list models: "tudilix", "gikovik", "zebutar", "fekizen", "kupedra"
     vocab_size: int
     hidden_size: int
     intermediate_size: int
@@ -49,7 +49,9 @@ class ModelConfig:
     # their weights (every repetition gets separate caches); and the width of the per-layer token input
     loop: Optional[Dict[str, int]] = None
     token_side_dim: int = 0
-    embed_scale: float = 1.0       # arch "fekizen": token embeddings enter times this; ``max_position`` rows of learned positions
+    embed_scale: float = 1.0       # arch "fekizen" (with ``max_position`` rows of learned positions), "kupedra": token embeddings enter times this
+    streams: int = 1               # arch "kupedra": residual streams per token (hyper-connections)
+    logit_scale: float = 1.0       # arch "kupedra": the head's product times this
 
     # ------------------------------------------------------------------ sizes
     @property
@@ -59,7 +61,7 @@ class ModelConfig:
     @property
     def needs_state_slots(self) -> bool:
         """Sequences carry per-layer state besides paged K/V (recurrent state, convolution tails)."""
-        return self.layers is not None and self.arch in ("tudilix", "zebutar", "fekizen")
+        return self.layers is not None and self.arch in ("tudilix", "zebutar", "fekizen", "kupedra")
 
     @property
     def needs_seq_index(self) -> bool:
@@ -141,6 +143,13 @@ class ModelConfig:
             if self.loop:
                 d["loop"] = dict(self.loop)
             return d
+        if self.arch == "kupedra":
+            d = {"architecture": "Kupedra", "layers": [dict(l) for l in self.layers], "norm": {"eps": self.norm_eps},
+                 "vocab": self.vocab_size, "width": self.hidden_size, "embedding": {"scale": self.embed_scale},
+                 "streams": self.streams, "logit_scale": self.logit_scale, "_dllm_name": self.name}
+            if self.loop:
+                d["loop"] = dict(self.loop)
+            return d
         if self.arch == "zebutar":
             return {"architecture": "Zebutar", "layers": [dict(l) for l in self.layers], "norm": {"eps": self.norm_eps},
                     "vocab": self.vocab_size, "width": self.hidden_size, "_dllm_name": self.name}
@@ -188,6 +197,8 @@ class ModelConfig:
             return _from_zebutar(cfg, name)
         if cfg.get("architecture") == "Fekizen":
             return _from_fekizen(cfg, name)
+        if cfg.get("architecture") == "Kupedra":
+            return _from_kupedra(cfg, name)
         mt = cfg.get("model_type", "llama")
         name = name or cfg.get("_dllm_name") or cfg.get("_name_or_path") or mt
         eos = cfg.get("eos_token_id", 2)
@@ -334,6 +345,38 @@ def _from_fekizen(cfg: Dict[str, Any], name: Optional[str] = None) -> ModelConfi
         embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)))
 
 
+def _from_kupedra(cfg: Dict[str, Any], name: Optional[str] = None) -> ModelConfig:
+    """A ``config.json`` with "architecture": "Kupedra": ``width``, ``vocab``, ``norm.eps``, ``embedding.scale``,
+    ``streams``, ``logit_scale``, ``layers`` (per layer ``type`` "attention" | "parallel", ``mixer`` sizes, ``mlp`` None | moe)
+    and optionally ``loop`` (start, stop, times)."""
+    layers = [dict(l) for l in cfg["layers"]]
+    if not layers:
+        raise ValueError("layer-list config without layers")
+    for l in layers:
+        if l["type"] not in ("attention", "parallel"):
+            raise ValueError(f"unsupported layer type {l['type']!r} (attention, parallel)")
+        if l.get("mlp") is not None and l["mlp"].get("kind", "moe") != "moe":
+            raise ValueError(f"unsupported mlp kind {l['mlp'].get('kind')!r} (moe)")
+    extra = set(cfg.get("norm", {})) - {"eps"}
+    if extra:
+        raise ValueError(f"unsupported norm options {sorted(extra)}")
+    loop = cfg.get("loop")
+    if loop:
+        loop = {k: int(loop[k]) for k in ("start", "stop", "times")}
+        if not (0 <= loop["start"] < loop["stop"] <= len(layers)) or loop["times"] < 1:
+            raise ValueError(f"loop {loop} does not fit {len(layers)} layers")
+    attn = [l["mixer"] if l["type"] == "attention" else l["mixer"]["left"] for l in layers]
+    ff = [l["mlp"]["expert"]["ff"] for l in layers if l.get("mlp")]
+    return ModelConfig(
+        name=name or cfg.get("_dllm_name") or "kupedra", arch="kupedra", vocab_size=int(cfg["vocab"]),
+        hidden_size=int(cfg["width"]), intermediate_size=int(max(ff or [0])), num_layers=len(layers),
+        num_heads=max(m["heads"] for m in attn), num_kv_heads=max(m["kv_heads"] for m in attn),
+        head_dim=max(max(m["dim"], m["vdim"]) for m in attn), max_position=1 << 30,
+        norm_eps=float(cfg["norm"]["eps"]), bos_token_id=-1, eos_token_id=-1, layers=layers, loop=loop or None,
+        embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), streams=int(cfg.get("streams") or 1),
+        logit_scale=float(1.0 if cfg.get("logit_scale") is None else cfg["logit_scale"]))
+
+
 _LLAMA3_ROPE = {"rope_type": "llama3", "factor": 8.0, "low_freq_factor": 1.0,
                 "high_freq_factor": 4.0, "original_max_position_embeddings": 8192}
 
@@ -448,6 +491,22 @@ PRESETS: Dict[str, ModelConfig] = {
                 "right": {"dim": 24, "vdim": 16, "heads": 3, "tau": 4.0}},
              "mlp": {"kind": "moe", "expert": {"ff": 32}, "shared": {"ff": 32}, "router": {"experts": 4, "top": 1}}},
         ]}, name="tiny-fekizen"),
+    "tiny-kupedra": _from_kupedra({
+        "architecture": "Kupedra", "vocab": 304, "width": 96, "norm": {"eps": 1e-6}, "embedding": {"scale": 2.0},
+        "streams": 2, "logit_scale": 0.5, "loop": {"start": 1, "stop": 2, "times": 2},
+        "layers": [
+            {"type": "attention", "mixer": {"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 16, "scale": 0.3,
+                                            "rot": {"base": 10000.0, "dims": 16, "scaling": {"factor": 2.0}}},
+             "mlp": {"kind": "moe", "expert": {"ff": 48, "limit": 3.0}, "shared": {"ff": 64, "limit": 2.5},
+                     "router": {"experts": 6, "top": 2}}},
+            {"type": "parallel", "mixer": {
+                "left": {"heads": 3, "kv_heads": 1, "dim": 32, "vdim": 24, "scale": 0.2, "bias_max": 40,
+                         "q_temp": {"coef": 0.2, "every": 32}},
+                "right": {"heads": 2, "dim": 16, "vdim": 40, "gate_cap": 12.0}},
+             "mlp": {"kind": "moe", "expert": {"ff": 32, "limit": 2.0}, "shared": None, "router": {"experts": 4, "top": 1}}},
+            {"type": "attention", "mixer": {"heads": 2, "kv_heads": 2, "dim": 16, "vdim": 16, "scale": 0.25,
+                                            "rot": {"base": 500.0, "dims": 8}}, "mlp": None},
+        ]}, name="tiny-kupedra"),
     "tiny-gpt2": ModelConfig(
         name="tiny-gpt2", arch="gpt2", vocab_size=512, hidden_size=128,
         intermediate_size=512, num_layers=4, num_heads=2, num_kv_heads=2, head_dim=64,

@@ -10,6 +10,9 @@
 // window a query at position p also sees entries b < npool(p) = floor(max(p - window + 1, 0) / pool) -- one
 // mean key and value per block of `pool` positions that lies wholly before the window -- in the same softmax;
 // every kernel visits those entries first (32-entry tiles from entry 0), then the window's tokens.
+// `bias` (float32 [H, nbias], or null) is added to head h's scaled score of a key n positions before the query:
+// bias[h][min(n, nbias - 1)] (a learned distance bias, expanded from its buckets by the caller; a tile all of
+// whose keys are nbias - 1 or more back adds one constant).
 // Scores, softmax weights and the weighted sum are float32; T is the storage
 // type (bf16 or float).  Head sizes, window and block size are runtime values.
 //
@@ -106,7 +109,8 @@ __global__ void __launch_bounds__(kWinTile) window_attn_row_kernel(
     const void* __restrict__ v_cache_, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ positions, const int32_t* __restrict__ tok_seq, int t0, int H, int G, int D, int Dv,
     int bs, int window, int chunk, float scale, const float* __restrict__ sinks, float softcap,
-    const void* __restrict__ kp_, const void* __restrict__ vp_, int pool, int pbs) {
+    const void* __restrict__ kp_, const void* __restrict__ vp_, int pool, int pbs, const float* __restrict__ bias,
+    int nbias) {
   extern __shared__ float lds[];
   float* qs = lds;                       // [D]
   float* p = qs + D;                     // [kWinTile]
@@ -140,6 +144,7 @@ __global__ void __launch_bounds__(kWinTile) window_attn_row_kernel(
         rows[tid] = row;                                    // K row; V element (e) at ((row / cbs) * Dv + e) * cbs + row % cbs
         s = dot_row<T>(qs, kc + (size_t)row * D, D) * scale;
         if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+        if (bias) s += bias[(size_t)h * nbias + min(pos - j, nbias - 1)];      // never beside averaged entries
       }
       const float m_new = fmaxf(m, block_max(s, red));
       const float pj = j <= last ? expf(s - m_new) : 0.f;
@@ -197,7 +202,8 @@ static size_t win_row_lds(int D, int Dv) {
 static void launch_rows(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                         int max_blocks, uintptr_t positions, uintptr_t tok_seq, int t0, int rows, int H, int G, int D,
                         int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, float softcap, uintptr_t kp,
-                        uintptr_t vp, int pool, int pbs, int f32, uintptr_t stream) {
+                        uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int f32, uintptr_t stream) {
+  DLLM_HOST_CHECK(!bias || (nbias >= 1 && pool == 0), "window attention distance bias");
   DLLM_HOST_CHECK(H > 0 && G > 0 && H % G == 0 && D > 0 && Dv > 0 && Dv <= kWinTile * kWinMaxAcc, "window attention heads");
   DLLM_HOST_CHECK(pool == 0 || (pool > 0 && kp && vp && pbs > 0 && chunk == 0), "window attention averaged caches");
   DLLM_HOST_CHECK(bs > 0 && window >= 1 && chunk >= 0 && max_blocks > 0 && H <= 65535, "window attention sizes");
@@ -208,13 +214,13 @@ static void launch_rows(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t
                        (hipStream_t)stream, (void*)out, (const void*)q, (const void*)k_cache, (const void*)v_cache,
                        (const int32_t*)block_tables, max_blocks, (const int32_t*)positions, (const int32_t*)tok_seq, t0,
                        H, G, D, Dv, bs, window, chunk, scale, (const float*)sinks, softcap, (const void*)kp, (const void*)vp,
-                       pool, pbs);
+                       pool, pbs, (const float*)bias, nbias);
   else
     hipLaunchKernelGGL(HIP_KERNEL_NAME(window_attn_row_kernel<bf16>), dim3(rows, H), dim3(kWinTile), lds,
                        (hipStream_t)stream, (void*)out, (const void*)q, (const void*)k_cache, (const void*)v_cache,
                        (const int32_t*)block_tables, max_blocks, (const int32_t*)positions, (const int32_t*)tok_seq, t0,
                        H, G, D, Dv, bs, window, chunk, scale, (const float*)sinks, softcap, (const void*)kp, (const void*)vp,
-                       pool, pbs);
+                       pool, pbs, (const float*)bias, nbias);
   DLLM_HIP_CHECK(hipGetLastError());
 }
 
@@ -243,17 +249,20 @@ __device__ __forceinline__ void split_pack(const float (&e)[8], bf16x8& ph, bf16
 constexpr int kTK = 32;          // keys per tile
 constexpr int kPad = 8;          // bf16 elements of row padding in LDS (16 bytes: rows start on different banks)
 constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kBiasLds = 2048;   // distance biases per head kept in LDS (8 KiB); longer tables are read through the caches
 
 // NQK: 32-wide K-dim steps of q.k (D <= 32 NQK); NDV: 16-wide tiles of value channels (Dv <= 16 NDV).
 // Every K / V^T fragment a wave reads from LDS feeds both of its query column tiles; the next key tile's
 // global loads are issued before the current tile's MFMAs and land in LDS after them.
-template <int NQK, int NDV, int QT>
+// BIAS: a distance bias is given (a build of its own: the others keep their registers).
+template <int NQK, int NDV, int QT, bool BIAS>
 __global__ void __launch_bounds__(256) window_attn_tile_kernel(
     bf16* __restrict__ out, const bf16* __restrict__ q, const bf16* __restrict__ k_cache,
     const bf16* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ cu, const int32_t* __restrict__ positions, int seq0, int nseq, int nqt, int H, int G,
     int D, int Dv, int bs, int window, int chunk, float scale, const float* __restrict__ sinks, int sub, float softcap,
-    const bf16* __restrict__ kp_cache, const bf16* __restrict__ vp_cache, int pool, int pbs) {
+    const bf16* __restrict__ kp_cache, const bf16* __restrict__ vp_cache, int pool, int pbs,
+    const float* __restrict__ bias, int nbias) {
   constexpr int kQT = QT, kTQ = 64 * QT;
   constexpr int DP = 32 * NQK, KROW = DP + kPad, VROW = kTK + kPad;
   constexpr int KPT = (kTK * (DP / 8) + 255) / 256, VPT = (16 * NDV * (kTK / 8) + 255) / 256;   // 16-byte pieces per thread
@@ -313,6 +322,18 @@ __global__ void __launch_bounds__(256) window_attn_tile_kernel(
   float m[kQT], l[kQT];
 #pragma unroll
   for (int c2 = 0; c2 < kQT; ++c2) m[c2] = -INFINITY, l[c2] = 0.f;
+  // the head's distance biases in log2 units, in LDS when they fit (the first tile's barriers order the writes)
+  extern __shared__ float bs_lds[];
+  const float* brow = nullptr;
+  float bfar = 0.f;
+  bool b_lds = false;
+  if constexpr (BIAS) {
+    brow = bias + (size_t)h * nbias;
+    bfar = brow[nbias - 1] * kLog2e;
+    b_lds = nbias <= kBiasLds;
+    if (b_lds)
+      for (int i = tid; i < nbias; i += 256) bs_lds[i] = brow[i] * kLog2e;
+  }
   const int d8 = D >> 3;
   const float sc2 = scale * kLog2e;
   const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap * kLog2e;   // capped scores in log2 units
@@ -402,6 +423,18 @@ __global__ void __launch_bounds__(256) window_attn_tile_kernel(
         for (int i = 0; i < 8; ++i) {
           const float raw = i < 4 ? s0[c2][i] : s1[c2][i - 4];
           p[i] = softcap > 0.f ? fast_tanh(raw * cap_in) * cap_out : raw * sc2;      // wave-uniform choice
+        }
+        if constexpr (BIAS) {
+          if (start + wq0 - (k0 + kTK - 1) >= nbias - 1) {   // wave-uniform: every key is in the last bucket
+#pragma unroll
+            for (int i = 0; i < 8; ++i) p[i] += bfar;
+          } else {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+              const int n2 = min(max(qpos[c2] - (k0 + 8 * grp + i), 0), nbias - 1);     // keys ahead are masked below
+              p[i] += b_lds ? bs_lds[n2] : brow[n2] * kLog2e;
+            }
+          }
         }
         if (nomask) {                                      // wave-uniform: no per-element mask work
 #pragma unroll
@@ -495,22 +528,22 @@ __global__ void __launch_bounds__(256) window_attn_tile_kernel(
   }
 }
 
-template <int NQK, int NDV, int QT>
+template <int NQK, int NDV, int QT, bool BIAS>
 static void launch_tile(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                         int max_blocks, uintptr_t cu, uintptr_t positions, int seq0, int nseq, int max_q_len, int H,
                         int G, int D, int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, float softcap,
-                        uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t stream) {
+                        uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, uintptr_t stream) {
   constexpr int kTQ = 64 * QT;
   const int nqt = (max_q_len + kTQ - 1) / kTQ;
   const int pairs = nseq * G, per_pair = nqt * (H / G);
   const int sub = pairs < 8 ? 8 : 1;                                    // XCDs that share a pair's tiles
   const long per_xcd = (long)(((long)pairs * sub + 7) / 8) * ((per_pair + sub - 1) / sub);   // workgroups of one XCD
   DLLM_HOST_CHECK(per_xcd * 8 < (1L << 31), "window attention grid");
-  hipLaunchKernelGGL(HIP_KERNEL_NAME(window_attn_tile_kernel<NQK, NDV, QT>), dim3((unsigned)(per_xcd * 8)),
-                     dim3(256), 0, (hipStream_t)stream, (bf16*)out, (const bf16*)q, (const bf16*)k_cache,
+  hipLaunchKernelGGL(HIP_KERNEL_NAME(window_attn_tile_kernel<NQK, NDV, QT, BIAS>), dim3((unsigned)(per_xcd * 8)),
+                     dim3(256), BIAS && nbias <= kBiasLds ? sizeof(float) * nbias : 0, (hipStream_t)stream, (bf16*)out, (const bf16*)q, (const bf16*)k_cache,
                      (const bf16*)v_cache, (const int32_t*)block_tables, max_blocks, (const int32_t*)cu,
                      (const int32_t*)positions, seq0, nseq, nqt, H, G, D, Dv, bs, window, chunk, scale, (const float*)sinks, sub,
-                     softcap, (const bf16*)kp, (const bf16*)vp, pool, pbs);
+                     softcap, (const bf16*)kp, (const bf16*)vp, pool, pbs, (const float*)bias, nbias);
   DLLM_HIP_CHECK(hipGetLastError());
 }
 
@@ -523,13 +556,14 @@ static void launch_tile(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t
 // O^T = V^T P^T.  Each wave keeps an online softmax; the waves' partial results meet in LDS.
 constexpr int kDW = 4;
 
-template <int NQK, int NDV>
+template <int NQK, int NDV, bool BIAS>
 __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
     bf16* __restrict__ out, const bf16* __restrict__ q, const bf16* __restrict__ k_cache,
     const bf16* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ positions, const int32_t* __restrict__ tok_seq, int H, int G, int D, int Dv, int bs,
     int window, int chunk, float scale, const float* __restrict__ sinks, int hpw, int splits, float* __restrict__ ws,
-    float softcap, const bf16* __restrict__ kp_cache, const bf16* __restrict__ vp_cache, int pool, int pbs) {
+    float softcap, const bf16* __restrict__ kp_cache, const bf16* __restrict__ vp_cache, int pool, int pbs,
+    const float* __restrict__ bias, int nbias) {
   constexpr int DVP = 16 * NDV;
   __shared__ float so[kDW][16][DVP + 1];
   __shared__ float sml[kDW][2][16];
@@ -594,6 +628,9 @@ __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
   const int tstop = min(ntile, ((int)blockIdx.z + 1) * tps);
   const int tbeg = (int)blockIdx.z * tps + wave;
   const float cap_in = softcap > 0.f ? scale / softcap : 0.f;
+  const float* brow = nullptr;                       // distance biases of this lane's head
+  float bfar = 0.f;
+  if constexpr (BIAS) brow = bias + (size_t)(hb + min(col, nh - 1)) * nbias, bfar = brow[nbias - 1];
   if (tbeg < tstop) load_k(tbeg);
   for (int ti = tbeg; ti < tstop; ti += kDW) {
     const bool pooled = ti < ptile;
@@ -624,11 +661,13 @@ __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
     if (ti + kDW < tstop) load_k(ti + kDW);
     float p[8];
     float cm = -INFINITY;
+    const bool near = BIAS && pos - (k0 + 31) < nbias - 1;       // some key of the tile is not in the last bucket
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int kp = k0 + 8 * grp + i;
       const float raw = i < 4 ? s0[i] : s1[i - 4];
-      const float sv = softcap > 0.f ? softcap * fast_tanh(raw * cap_in) : raw * scale;
+      float sv = softcap > 0.f ? softcap * fast_tanh(raw * cap_in) : raw * scale;
+      if constexpr (BIAS) sv += near ? brow[min(max(pos - kp, 0), nbias - 1)] : bfar;
       p[i] = (kp >= rlo && kp <= rhi) ? sv : -INFINITY;
       cm = fmaxf(cm, p[i]);
     }
@@ -719,11 +758,11 @@ __global__ void __launch_bounds__(64) window_attn_merge_kernel(bf16* __restrict_
   }
 }
 
-template <int NQK, int NDV>
+template <int NQK, int NDV, bool BIAS>
 static void launch_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                           int max_blocks, uintptr_t positions, uintptr_t tok_seq, int rows, int H, int G, int D,
                           int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, int splits, uintptr_t ws,
-                          float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t stream) {
+                          float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, uintptr_t stream) {
   // heads per workgroup: 16 (all MFMA columns) when rows x K/V heads x key runs fill the chip, else halved
   // until about half the CUs have a workgroup -- the keys are re-read from L2, the columns left idle cost
   // nothing.  Key runs come first: a workgroup holds a CU's registers alone, so the call takes
@@ -732,12 +771,12 @@ static void launch_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr
   splits = ws ? std::max(1, std::min(splits, 64)) : 1;
   int hpw = std::min(16, R);
   while (hpw > 2 && (long)rows * G * ((R + hpw - 1) / hpw) * splits < 128) hpw = (hpw + 1) / 2;
-  hipLaunchKernelGGL(HIP_KERNEL_NAME(window_attn_decode_kernel<NQK, NDV>),
+  hipLaunchKernelGGL(HIP_KERNEL_NAME(window_attn_decode_kernel<NQK, NDV, BIAS>),
                      dim3(rows, G * ((R + hpw - 1) / hpw), splits), dim3(64 * kDW), 0,
                      (hipStream_t)stream, (bf16*)out, (const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache,
                      (const int32_t*)block_tables, max_blocks, (const int32_t*)positions, (const int32_t*)tok_seq, H, G,
                      D, Dv, bs, window, chunk, scale, (const float*)sinks, hpw, splits, (float*)ws, softcap, (const bf16*)kp,
-                     (const bf16*)vp, pool, pbs);
+                     (const bf16*)vp, pool, pbs, (const float*)bias, nbias);
   DLLM_HIP_CHECK(hipGetLastError());
   if (splits > 1) {
     hipLaunchKernelGGL(window_attn_merge_kernel, dim3(rows, H), dim3(64), 0, (hipStream_t)stream, (bf16*)out,
@@ -759,14 +798,24 @@ static bool win_mfma_ok(int f32, int H, int G, int D, int Dv, int bs, int pool, 
 void sm_window_attn_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                            int max_blocks, uintptr_t positions, uintptr_t tok_seq, int rows, int H, int G, int D,
                            int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, int splits, uintptr_t ws,
-                           float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, int f32, uintptr_t stream) {
+                           float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int f32,
+                           uintptr_t stream) {
   if (rows <= 0) return;
   if (win_mfma_ok(f32, H, G, D, Dv, bs, pool, pbs) && (long)G * ((H / G + 1) / 2) <= 65535) {
     DLLM_HOST_CHECK(window >= 1 && chunk >= 0 && max_blocks > 0, "window attention sizes");
     DLLM_HOST_CHECK(pool == 0 || (pool > 0 && kp && vp && chunk == 0), "window attention averaged caches");
-#define WIN_DEC(NQK, NDV)                                                                                       \
-  launch_decode<NQK, NDV>(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, rows, H, G, D, Dv, \
-                          bs, window, chunk, scale, sinks, splits, ws, softcap, kp, vp, pool, pbs, stream)
+    DLLM_HOST_CHECK(!bias || (nbias >= 1 && pool == 0), "window attention distance bias");
+#define WIN_DEC(NQK, NDV)                                                                                          \
+  do {                                                                                                             \
+    if (bias)                                                                                                      \
+      launch_decode<NQK, NDV, true>(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, rows, H, G, \
+                                    D, Dv, bs, window, chunk, scale, sinks, splits, ws, softcap, kp, vp, pool, pbs, \
+                                    bias, nbias, stream);                                                          \
+    else                                                                                                           \
+      launch_decode<NQK, NDV, false>(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, rows, H, G, \
+                                     D, Dv, bs, window, chunk, scale, sinks, splits, ws, softcap, kp, vp, pool, pbs, \
+                                     0, 0, stream);                                                                \
+  } while (0)
     if (D <= 64 && Dv <= 64) WIN_DEC(2, 4);
     else if (D <= 128 && Dv <= 128) WIN_DEC(4, 8);
     else WIN_DEC(8, 16);
@@ -774,7 +823,7 @@ void sm_window_attn_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintpt
     return;
   }
   launch_rows(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, 0, rows, H, G, D, Dv, bs, window,
-              chunk, scale, sinks, softcap, kp, vp, pool, pbs, f32, stream);
+              chunk, scale, sinks, softcap, kp, vp, pool, pbs, bias, nbias, f32, stream);
 }
 
 // Prompt chunks: tokens [t0 .. tokens) of sequences [seq0, seqs).
@@ -782,7 +831,7 @@ void sm_window_attn_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintp
                             int max_blocks, uintptr_t cu, uintptr_t positions, uintptr_t tok_seq, int seq0, int seqs,
                             int tokens, int max_q_len, int H, int G, int D, int Dv, int bs, int window, int chunk,
                             float scale, uintptr_t sinks, float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs,
-                            int f32, uintptr_t stream) {
+                            uintptr_t bias, int nbias, int f32, uintptr_t stream) {
   // tokens of the decode rows come first: one per sequence before seq0
   const int t0 = seq0;
   if (tokens <= t0) return;
@@ -790,9 +839,18 @@ void sm_window_attn_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintp
     DLLM_HOST_CHECK(H > 0 && G > 0 && H % G == 0 && H <= 65535 && seqs - seq0 <= 65535, "window attention heads");
     DLLM_HOST_CHECK(bs > 0 && window >= 1 && chunk >= 0 && max_blocks > 0, "window attention sizes");
     DLLM_HOST_CHECK(pool == 0 || (pool > 0 && kp && vp && chunk == 0), "window attention averaged caches");
-#define WIN_TILE(NQK, NDV, QT)                                                                                  \
-  launch_tile<NQK, NDV, QT>(out, q, k_cache, v_cache, block_tables, max_blocks, cu, positions, seq0, seqs - seq0, \
-                            max_q_len, H, G, D, Dv, bs, window, chunk, scale, sinks, softcap, kp, vp, pool, pbs, stream)
+    DLLM_HOST_CHECK(!bias || (nbias >= 1 && pool == 0), "window attention distance bias");
+#define WIN_TILE(NQK, NDV, QT)                                                                                     \
+  do {                                                                                                             \
+    if (bias)                                                                                                      \
+      launch_tile<NQK, NDV, QT, true>(out, q, k_cache, v_cache, block_tables, max_blocks, cu, positions, seq0,     \
+                                      seqs - seq0, max_q_len, H, G, D, Dv, bs, window, chunk, scale, sinks, softcap, kp, \
+                                      vp, pool, pbs, bias, nbias, stream);                                         \
+    else                                                                                                           \
+      launch_tile<NQK, NDV, QT, false>(out, q, k_cache, v_cache, block_tables, max_blocks, cu, positions, seq0,    \
+                                       seqs - seq0, max_q_len, H, G, D, Dv, bs, window, chunk, scale, sinks, softcap, kp, \
+                                       vp, pool, pbs, 0, 0, stream);                                               \
+  } while (0)
     if (D <= 64 && Dv <= 64) WIN_TILE(2, 4, 1);
     else if (D <= 128 && Dv <= 128) WIN_TILE(4, 8, 1);
     else WIN_TILE(8, 16, 2);     // wide heads: 2b-size latent attention prompts 32 x 1024 +7 %, 4 x 4096 +29 % over QT = 1
@@ -800,7 +858,7 @@ void sm_window_attn_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintp
     return;
   }
   launch_rows(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, t0, tokens - t0, H, G, D, Dv, bs,
-              window, chunk, scale, sinks, softcap, kp, vp, pool, pbs, f32, stream);
+              window, chunk, scale, sinks, softcap, kp, vp, pool, pbs, bias, nbias, f32, stream);
 }
 
 }  // namespace dllm

@@ -69,6 +69,10 @@ PYBIND11_MODULE(_C_kernels, m) {
   m.def("sm_token_shift", &dllm::sm_token_shift);
   m.def("sm_pool_blocks", &dllm::sm_pool_blocks);
   m.def("la_scan", &dllm::la_scan);
+  m.def("ml_gates", &dllm::ml_gates);
+  m.def("sm_head_norm_rope", &dllm::sm_head_norm_rope);
+  m.def("hc_embed", &dllm::hc_embed);
+  m.def("hc_step", &dllm::hc_step);
   m.def("dr_prep", &dllm::dr_prep);
   m.def("dr_conv_prep", &dllm::dr_conv_prep);
   m.def("sm_conv_tail", &dllm::sm_conv_tail);

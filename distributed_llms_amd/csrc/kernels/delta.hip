@@ -327,11 +327,11 @@ template <typename T>
 __global__ void __launch_bounds__(64) dr_out_norm_kernel(void* __restrict__ y_, long ldy, const float* __restrict__ o,
                                                          const void* __restrict__ gate_, long ldg, int gcol,
                                                          const void* __restrict__ w_, int H, int vdim, float eps,
-                                                         float out_scale, int gate_sig) {
+                                                         float out_scale, int gate_sig, int w_stride) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const float* row = o + ((size_t)t * H + h) * vdim;
   const T* gate = (const T*)gate_ + (size_t)t * ldg + gcol + (size_t)h * vdim;
-  const T* w = (const T*)w_;
+  const T* w = (const T*)w_ + (size_t)h * w_stride;
   T* y = (T*)y_ + (size_t)t * ldy + (size_t)h * vdim;
   float ss = 0.f;
   for (int e = lane; e < vdim; e += 64) ss += row[e] * row[e];
@@ -348,7 +348,7 @@ template <typename T>
 __global__ void __launch_bounds__(256) dr_out_norm_vec_kernel(void* __restrict__ y_, long ldy, const float* __restrict__ o,
                                                              const void* __restrict__ gate_, long ldg, int gcol,
                                                              const void* __restrict__ w_, long heads_total, int H,
-                                                             int vdim, float eps, float out_scale, int gate_sig) {
+                                                             int vdim, float eps, float out_scale, int gate_sig, int w_stride) {
   const int lph = vdim >> 3;
   const long idx = (long)blockIdx.x * 256 + threadIdx.x;
   const long th = idx / lph;
@@ -365,7 +365,7 @@ __global__ void __launch_bounds__(256) dr_out_norm_vec_kernel(void* __restrict__
   for (int m = lph >> 1; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
   const float inv = out_scale / sqrtf(ss / (float)vdim + eps);
   ldv<8>((const T*)gate_ + (size_t)t * ldg + gcol + (size_t)h * vdim + c, gv);
-  ldv<8>((const T*)w_ + c, wv);
+  ldv<8>((const T*)w_ + (size_t)h * w_stride + c, wv);
 #pragma unroll
   for (int e = 0; e < 8; ++e) xv[e] = xv[e] * inv * wv[e] * (gate_sig ? dr_sigmoid(gv[e]) : gv[e] * dr_sigmoid(gv[e]));
   if (ok) stv<8>((T*)y_ + (size_t)t * ldy + (size_t)h * vdim + c, xv);
@@ -377,12 +377,12 @@ template <typename T>
 __global__ void __launch_bounds__(256) dr_out_norm_wide_kernel(void* __restrict__ y_, long ldy, const float* __restrict__ o,
                                                               const void* __restrict__ gate_, long ldg, int gcol,
                                                               const void* __restrict__ w_, int H, int vdim, float eps,
-                                                              float out_scale, int gate_sig) {
+                                                              float out_scale, int gate_sig, int w_stride) {
   __shared__ float red[16];
   const int t = blockIdx.x, h = blockIdx.y;
   const float* row = o + ((size_t)t * H + h) * vdim;
   const T* gate = (const T*)gate_ + (size_t)t * ldg + gcol + (size_t)h * vdim;
-  const T* w = (const T*)w_;
+  const T* w = (const T*)w_ + (size_t)h * w_stride;
   T* y = (T*)y_ + (size_t)t * ldy + (size_t)h * vdim;
   float ss = 0.f;
   for (int e = threadIdx.x * 8; e < vdim; e += 2048) {
@@ -404,28 +404,28 @@ __global__ void __launch_bounds__(256) dr_out_norm_wide_kernel(void* __restrict_
   }
 }
 
-void dr_out_norm(uintptr_t y, long ldy, uintptr_t o, uintptr_t gate, long ldg, int gcol, uintptr_t w, int tokens, int H,
-                 int vdim, float eps, float out_scale, int gate_sig, int f32, uintptr_t stream) {
+void dr_out_norm(uintptr_t y, long ldy, uintptr_t o, uintptr_t gate, long ldg, int gcol, uintptr_t w, int w_stride,
+                 int tokens, int H, int vdim, float eps, float out_scale, int gate_sig, int f32, uintptr_t stream) {
   if (tokens <= 0) return;
-  DLLM_HOST_CHECK(H > 0 && H <= 65535 && vdim > 0 && ldy >= (long)H * vdim && ldg >= gcol + (long)H * vdim && gcol >= 0,
+  DLLM_HOST_CHECK(H > 0 && H <= 65535 && vdim > 0 && ldy >= (long)H * vdim && ldg >= gcol + (long)H * vdim && gcol >= 0 && w_stride >= 0,
                   "delta rule output norm sizes");
   const int esz = f32 ? 4 : 2, lph = vdim >> 3;
   if (vdim % 8 == 0 && vdim > 512 && ldy % 8 == 0 && ldg % 8 == 0 && gcol % 8 == 0 && y % (8 * esz) == 0 &&
-      gate % (8 * esz) == 0 && w % (8 * esz) == 0 && o % 32 == 0) {
+      gate % (8 * esz) == 0 && w % (8 * esz) == 0 && w_stride % 8 == 0 && o % 32 == 0) {
     SM_DISPATCH(f32, dr_out_norm_wide_kernel, dim3(tokens, H), dim3(256), 0, stream, (void*)y, ldy, (const float*)o,
-                (const void*)gate, ldg, gcol, (const void*)w, H, vdim, eps, out_scale, gate_sig);
+                (const void*)gate, ldg, gcol, (const void*)w, H, vdim, eps, out_scale, gate_sig, w_stride);
     return;
   }
   if (vdim % 8 == 0 && lph <= 64 && (lph & (lph - 1)) == 0 && ldy % 8 == 0 && ldg % 8 == 0 && gcol % 8 == 0 &&
-      y % (8 * esz) == 0 && gate % (8 * esz) == 0 && w % (8 * esz) == 0 && o % 32 == 0) {
+      y % (8 * esz) == 0 && gate % (8 * esz) == 0 && w % (8 * esz) == 0 && w_stride % 8 == 0 && o % 32 == 0) {
     const long heads_total = (long)tokens * H, lanes = heads_total * lph;
     DLLM_HOST_CHECK((lanes + 255) / 256 < (1L << 31), "delta rule output norm grid");
     SM_DISPATCH(f32, dr_out_norm_vec_kernel, dim3((unsigned)((lanes + 255) / 256)), dim3(256), 0, stream, (void*)y, ldy,
-                (const float*)o, (const void*)gate, ldg, gcol, (const void*)w, heads_total, H, vdim, eps, out_scale, gate_sig);
+                (const float*)o, (const void*)gate, ldg, gcol, (const void*)w, heads_total, H, vdim, eps, out_scale, gate_sig, w_stride);
     return;
   }
   SM_DISPATCH(f32, dr_out_norm_kernel, dim3(tokens, H), dim3(64), 0, stream, (void*)y, ldy, (const float*)o,
-              (const void*)gate, ldg, gcol, (const void*)w, H, vdim, eps, out_scale, gate_sig);
+              (const void*)gate, ldg, gcol, (const void*)w, H, vdim, eps, out_scale, gate_sig, w_stride);
 }
 
 }  // namespace dllm

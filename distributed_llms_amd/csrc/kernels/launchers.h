@@ -83,8 +83,17 @@ void sm_pool_blocks(uintptr_t k_cache, uintptr_t v_cache, uintptr_t kp_cache, ui
                     int max_blocks, uintptr_t cu, uintptr_t positions, int seqs, int max_q_len, int G, int D, int Dv,
                     int bs, int pb, int pool, int f32, uintptr_t stream);
 void la_scan(uintptr_t o, uintptr_t proj, long ld, int qcol, int kcol, int vcol, uintptr_t decay, uintptr_t z,
-             uintptr_t z_bias, float inv_tau, float q_scale, int silu, uintptr_t state, uintptr_t cu, uintptr_t positions,
-             uintptr_t slots, int seqs, int max_q_len, int H, int D, int Dv, int f32, uintptr_t stream);
+             uintptr_t z_bias, float inv_tau, float q_scale, int silu, uintptr_t gates, uintptr_t state, uintptr_t cu,
+             uintptr_t positions, uintptr_t slots, int seqs, int max_q_len, int H, int D, int Dv, int f32, uintptr_t stream);
+void ml_gates(uintptr_t gates, uintptr_t proj, long ld, int qcol, int kcol, int icol, int fcol, uintptr_t i_bias,
+              uintptr_t f_bias, float cap, float q_scale, float den_eps, uintptr_t n_state, uintptr_t m_state, uintptr_t cu,
+              uintptr_t positions, uintptr_t slots, int seqs, int max_q_len, int H, int D, int f32, uintptr_t stream);
+// hyper-connections: several residual streams (hyper.hip)
+void hc_embed(uintptr_t x, uintptr_t ids, uintptr_t table, int tokens, int streams, int width, int vocab, float scale,
+              int f32, uintptr_t stream);
+void hc_step(uintptr_t x, uintptr_t mix, uintptr_t out_w, uintptr_t o, uintptr_t w1, uintptr_t o2, uintptr_t w2, float coef,
+             uintptr_t in_w, float gain, uintptr_t h, int rows, int streams, int width, float eps, int f32,
+             uintptr_t stream);
 void sm_rms_norm(uintptr_t y, uintptr_t x, uintptr_t w, int rows, int width, float eps, float offset, int f32,
                  uintptr_t stream);
 void sm_post_norm_add(uintptr_t x, uintptr_t o, uintptr_t bias, uintptr_t w_post, uintptr_t w_next, uintptr_t h,
@@ -103,7 +112,11 @@ void sm_rglru_scan(uintptr_t out, uintptr_t a, uintptr_t g, uintptr_t y_raw, lon
                    uintptr_t ab, int f32, uintptr_t stream);
 void sm_clipped_glu(uintptr_t out, uintptr_t gu, uintptr_t bias, int tokens, int F, float limit, float alpha, int f32,
                     uintptr_t stream);
-void sm_softcap(uintptr_t out, uintptr_t x, long n, float cap, int f32, uintptr_t stream);
+void sm_softcap(uintptr_t out, uintptr_t x, long n, float cap, float scale, int f32, uintptr_t stream);
+void sm_head_norm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_t q_norm, uintptr_t k_norm,
+                       uintptr_t freqs, int nrot, int norm_last, float eps, uintptr_t q_mul, float temp_coef, int temp_every,
+                       uintptr_t k_cache, uintptr_t v_cache, uintptr_t slot_mapping, uintptr_t positions, int tokens, int H,
+                       int G, int D, int Dv, int bs, int f32, uintptr_t stream);
 void sm_attn_prep(uintptr_t q_out, uintptr_t qkv, uintptr_t conv_w, uintptr_t state, uintptr_t q_norm,
                   uintptr_t k_norm, uintptr_t freqs, int nrot, float mag, float eps, uintptr_t k_cache,
                   uintptr_t v_cache, uintptr_t slot_mapping, uintptr_t cu, uintptr_t positions, uintptr_t tok_seq,
@@ -116,12 +129,13 @@ void sm_rownorm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_
 void sm_window_attn_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                            int max_blocks, uintptr_t positions, uintptr_t tok_seq, int rows, int H, int G, int D,
                            int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, int splits, uintptr_t ws,
-                           float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, int f32, uintptr_t stream);
+                           float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int f32,
+                           uintptr_t stream);
 void sm_window_attn_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                             int max_blocks, uintptr_t cu, uintptr_t positions, uintptr_t tok_seq, int seq0, int seqs,
                             int tokens, int max_q_len, int H, int G, int D, int Dv, int bs, int window, int chunk,
                             float scale, uintptr_t sinks, float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs,
-                            int f32, uintptr_t stream);
+                            uintptr_t bias, int nbias, int f32, uintptr_t stream);
 // latent attention input stage and parallel layers on a float32 stream (latent.hip)
 void lat_prep(uintptr_t cq, uintptr_t down, long ld, int q_off, int q_rank, uintptr_t qn_w, int c_off, int rank,
               uintptr_t cn_w, int r_off, int rot_dim, uintptr_t freqs, int nfreq, uintptr_t positions,
@@ -159,8 +173,8 @@ void dr_conv_prep(uintptr_t u, uintptr_t bd, uintptr_t x, long ld, int col0, int
                   uintptr_t stream);
 void dr_scan(uintptr_t o, uintptr_t u, long ld, uintptr_t bd, uintptr_t state, uintptr_t cu, uintptr_t positions,
              uintptr_t slots, int seqs, int max_q_len, int H, int G, int dim, int vdim, uintptr_t stream);
-void dr_out_norm(uintptr_t y, long ldy, uintptr_t o, uintptr_t gate, long ldg, int gcol, uintptr_t w, int tokens, int H,
-                 int vdim, float eps, float out_scale, int gate_sig, int f32, uintptr_t stream);
+void dr_out_norm(uintptr_t y, long ldy, uintptr_t o, uintptr_t gate, long ldg, int gcol, uintptr_t w, int w_stride,
+                 int tokens, int H, int vdim, float eps, float out_scale, int gate_sig, int f32, uintptr_t stream);
 void moe_combine_gated(uintptr_t out, uintptr_t ysorted, uintptr_t topk_w, uintptr_t inv, uintptr_t shared,
                        uintptr_t gate_logits, long gate_ld, int T, int H, int k, int f32, uintptr_t stream);
 

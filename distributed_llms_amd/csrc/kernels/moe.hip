@@ -376,7 +376,8 @@ void moe_combine(uintptr_t out, uintptr_t ysorted, uintptr_t topk_w, uintptr_t i
 // expert-sorted slot lists that the grouped GEMMs and the combine read.
 // `softmax_top` != 0 is the other router form: selection ranks the logits plus `correction` (here a bias
 // that is part of the logit), and the mixing weights are the softmax over the selected logits only,
-// times `scale`; groups do not apply.
+// times `scale`; groups do not apply.  `softmax_top` = 2: the weights are the softmax over ALL E logits at the
+// selected experts, not renormalised, times `scale`.
 constexpr int kMaxGroups = 64;
 constexpr int kMaxChoiceExperts = 256;
 
@@ -429,6 +430,10 @@ __device__ __forceinline__ void choose_groups(const float* __restrict__ lg, cons
     }
     ids[j] = best;
     tot += softmax_top ? expf(sc[best] - sc[ids[0]]) : sc[best];      // ids[0] holds the largest logit
+  }
+  if (softmax_top == 2) {
+    tot = 0.f;
+    for (int e = 0; e < E; ++e) tot += expf(sc[e] - sc[ids[0]]);
   }
   for (int j = 0; j < k; ++j) {
     ti[j] = ids[j];

@@ -946,18 +946,18 @@ void sm_clipped_glu(uintptr_t out, uintptr_t gu, uintptr_t bias, int tokens, int
 // --------------------------------------------------------------------------- logit soft cap
 template <typename T>
 __global__ void __launch_bounds__(256) sm_softcap_kernel(float* __restrict__ out, const void* __restrict__ x_, long n,
-                                                         float cap) {
+                                                         float cap, float scale) {
   const T* x = (const T*)x_;
   for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256) {
-    const float v = ldf(x + i);
+    const float v = ldf(x + i) * scale;
     out[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
   }
 }
 
-void sm_softcap(uintptr_t out, uintptr_t x, long n, float cap, int f32, uintptr_t stream) {
+void sm_softcap(uintptr_t out, uintptr_t x, long n, float cap, float scale, int f32, uintptr_t stream) {
   if (n <= 0) return;
   const int grid = (int)std::min<long>((n + 255) / 256, 65535);
-  SM_DISPATCH(f32, sm_softcap_kernel, dim3(grid), dim3(256), 0, stream, (float*)out, (const void*)x, n, cap);
+  SM_DISPATCH(f32, sm_softcap_kernel, dim3(grid), dim3(256), 0, stream, (float*)out, (const void*)x, n, cap, scale);
 }
 
 // --------------------------------------------------------------------------- attention input stage
@@ -1319,6 +1319,176 @@ void sm_rownorm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_
   SM_DISPATCH(f32, sm_rownorm_rope_kernel, dim3(tokens), dim3(256), 2 * (size_t)nrot * sizeof(float), stream, (void*)q_out, (const void*)qkv, ld, col0,
               (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot, eps, (void*)k_cache, (void*)v_cache,
               (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, mag, v_from_k);
+}
+
+// --------------------------------------------------------------------------- attention input: per-head norm, paired rotation, append
+// From a fused projection row [.. | q (H D) | k (G D) | v (G Dv) | ..] (row stride ld, q at column `col0`): every q and
+// k head is divided by its root mean square over D (times the plain weight qw / kw [D] shared by the heads, when
+// given) before or -- `norm_last` -- after the rotation of its first 2 nrot dimensions, pairs (2i, 2i + 1) turning by
+// float(pos) * freqs[i].  q is then multiplied by q_mul[h] (when given) and, with temp_every > 0, by
+// 1 + temp_coef ln(floor((pos + 1) / temp_every) + 1).  q goes to q_out [T, H, D]; k and v (unchanged) are appended at
+// slot_mapping to caches k [NB, G, BS, D] / v [NB, G, Dv, BS].  Norms, angles and factors are float32.
+//
+// One workgroup per token; 8 consecutive dimensions per lane, a head on an aligned group of `lph` lanes (a power of
+// two, 8 lph >= D): the mean square is a butterfly inside the group, the rotation stays inside a lane.
+__device__ __forceinline__ float query_temp(int pos, float coef, int every) {
+  return every > 0 ? 1.0f + coef * logf((float)((pos + 1) / every) + 1.0f) : 1.0f;
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256) sm_head_norm_rope_vec_kernel(
+    void* __restrict__ q_out_, const void* __restrict__ qkv_, long ld, int col0, const void* __restrict__ qw_,
+    const void* __restrict__ kw_, const float* __restrict__ freqs, int nrot, int norm_last, float eps,
+    const float* __restrict__ q_mul, float temp_coef, int temp_every, void* __restrict__ k_cache_,
+    void* __restrict__ v_cache_, const int32_t* __restrict__ slot_mapping, const int32_t* __restrict__ positions, int H,
+    int G, int D, int Dv, int bs, int lph) {
+  extern __shared__ float csn[];                   // cos | sin of the token's nrot angles
+  const int t = blockIdx.x, tid = threadIdx.x, pos = positions[t];
+  const float fpos = (float)pos;
+  for (int i = tid; i < nrot; i += 256) {
+    const float ang = fpos * freqs[i];
+    csn[i] = cosf(ang);
+    csn[nrot + i] = sinf(ang);
+  }
+  const T* q = (const T*)qkv_ + (size_t)t * ld + col0;
+  const int nq = H * D, nk = G * D, nv = G * Dv;
+  const T* v = q + nq + nk;
+  const int slot = slot_mapping[t], blk = slot / bs, off = slot - blk * bs;
+  T* q_out = (T*)q_out_ + (size_t)t * nq;
+  T* kc = (T*)k_cache_;
+  T* vc = (T*)v_cache_;
+  const float qt = query_temp(pos, temp_coef, temp_every);
+  const int sub = tid & (lph - 1), d = sub * 8;
+  if (nrot > 0) __syncthreads();                   // uniform: csn is complete
+  // every lane of a wave runs the same number of passes: the butterfly below needs whole groups
+  for (int h0 = 0; h0 < H + G; h0 += 256 / lph) {
+    const int head = h0 + tid / lph;
+    const bool ok = head < H + G && d < D;
+    const bool isq = head < H;
+    float x[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] = 0.f;
+    if (ok) ldv<8>(q + (size_t)head * D + d, x);
+    float ss = 0.f;
+    auto turn = [&]() {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int pr = (d >> 1) + i;
+        if (pr < nrot) {
+          const float cs = csn[pr], sn = csn[nrot + pr], a = x[2 * i], b = x[2 * i + 1];
+          x[2 * i] = a * cs - b * sn;
+          x[2 * i + 1] = b * cs + a * sn;
+        }
+      }
+    };
+    if (norm_last) turn();
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+    for (int m = lph >> 1; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+    const float inv = 1.0f / sqrtf(ss / (float)D + eps);
+    const T* w = (const T*)(isq ? qw_ : kw_);
+    if (w && ok) {
+      float g[8];
+      ldv<8>(w + d, g);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) x[i] *= inv * g[i];
+    } else {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) x[i] *= inv;
+    }
+    if (!norm_last) turn();
+    if (!ok) continue;
+    if (isq) {
+      const float f = q_mul ? qt * q_mul[head] : qt;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) x[i] *= f;
+      stv<8>(q_out + (size_t)head * D + d, x);
+    } else {
+      stv<8>(kc + (((size_t)blk * G + (head - H)) * bs + off) * D + d, x);
+    }
+  }
+  for (int e = tid; e < nv; e += 256) {
+    const int g = e / Dv, c = e - g * Dv;
+    vc[(((size_t)blk * G + g) * Dv + c) * bs + off] = v[e];
+  }
+}
+
+// The same for any head size: a wave per (token, head), the head's values in LDS.
+template <typename T>
+__global__ void __launch_bounds__(64) sm_head_norm_rope_kernel(
+    void* __restrict__ q_out_, const void* __restrict__ qkv_, long ld, int col0, const void* __restrict__ qw_,
+    const void* __restrict__ kw_, const float* __restrict__ freqs, int nrot, int norm_last, float eps,
+    const float* __restrict__ q_mul, float temp_coef, int temp_every, void* __restrict__ k_cache_,
+    void* __restrict__ v_cache_, const int32_t* __restrict__ slot_mapping, const int32_t* __restrict__ positions, int H,
+    int G, int D, int Dv, int bs, int) {
+  extern __shared__ float hv[];                    // the head's values [D]
+  const int t = blockIdx.x, head = blockIdx.y, lane = threadIdx.x, pos = positions[t];
+  const T* q = (const T*)qkv_ + (size_t)t * ld + col0;
+  const int slot = slot_mapping[t], blk = slot / bs, off = slot - blk * bs;
+  if (head >= H + G) {                             // a value head
+    const int g = head - H - G;
+    const T* v = q + (size_t)(H + G) * D + (size_t)g * Dv;
+    T* dst = (T*)v_cache_ + ((size_t)blk * G + g) * Dv * bs + off;
+    for (int c = lane; c < Dv; c += 64) dst[(size_t)c * bs] = v[c];
+    return;
+  }
+  const bool isq = head < H;
+  const T* src = q + (size_t)head * D;
+  const T* w = (const T*)(isq ? qw_ : kw_);
+  T* dst = isq ? (T*)q_out_ + ((size_t)t * H + head) * D
+               : (T*)k_cache_ + (((size_t)blk * G + (head - H)) * bs + off) * D;
+  const float fpos = (float)pos;
+  auto turn = [&]() {                              // a lane turns its own pairs
+    for (int i = lane; i < nrot; i += 64) {
+      const float ang = fpos * freqs[i], cs = cosf(ang), sn = sinf(ang), a = hv[2 * i], b = hv[2 * i + 1];
+      hv[2 * i] = a * cs - b * sn;
+      hv[2 * i + 1] = b * cs + a * sn;
+    }
+    __syncthreads();
+  };
+  for (int e = lane; e < D; e += 64) hv[e] = ldf(src + e);
+  __syncthreads();
+  if (norm_last) turn();
+  float ss = 0.f;
+  for (int e = lane; e < D; e += 64) ss += hv[e] * hv[e];
+  const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
+  for (int e = lane; e < D; e += 64) hv[e] *= w ? inv * ldf(w + e) : inv;
+  __syncthreads();
+  if (!norm_last) turn();
+  float f = 1.f;
+  if (isq) {
+    f = query_temp(pos, temp_coef, temp_every);
+    if (q_mul) f *= q_mul[head];
+  }
+  for (int e = lane; e < D; e += 64) stf(dst + e, hv[e] * f);
+}
+
+void sm_head_norm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_t q_norm, uintptr_t k_norm,
+                       uintptr_t freqs, int nrot, int norm_last, float eps, uintptr_t q_mul, float temp_coef, int temp_every,
+                       uintptr_t k_cache, uintptr_t v_cache, uintptr_t slot_mapping, uintptr_t positions, int tokens, int H,
+                       int G, int D, int Dv, int bs, int f32, uintptr_t stream) {
+  if (tokens <= 0) return;
+  DLLM_HOST_CHECK(H > 0 && G > 0 && D > 0 && Dv > 0 && bs > 0 && nrot >= 0 && 2 * nrot <= D && col0 >= 0 && temp_every >= 0 &&
+                      H + 2 * G <= 65535 && D <= 8192 && ld >= col0 + (long)H * D + (long)G * (D + Dv),
+                  "head_norm_rope sizes");
+  DLLM_HOST_CHECK(q_out && qkv && k_cache && v_cache && slot_mapping && positions && (nrot == 0 || freqs) &&
+                      (!q_norm == !k_norm),
+                  "head_norm_rope arguments");
+  const int esz = f32 ? 4 : 2;
+  if (D % 8 == 0 && D <= 512 && ld % 8 == 0 && col0 % 8 == 0 && qkv % (8 * esz) == 0 && q_norm % (8 * esz) == 0 &&
+      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0) {
+    int lph = 1;
+    while (8 * lph < D) lph *= 2;
+    SM_DISPATCH(f32, sm_head_norm_rope_vec_kernel, dim3(tokens), dim3(256), 2 * (size_t)nrot * sizeof(float), stream,
+                (void*)q_out, (const void*)qkv, ld, col0, (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot,
+                norm_last, eps, (const float*)q_mul, temp_coef, temp_every, (void*)k_cache, (void*)v_cache,
+                (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, lph);
+    return;
+  }
+  SM_DISPATCH(f32, sm_head_norm_rope_kernel, dim3(tokens, H + 2 * G), dim3(64), (size_t)D * sizeof(float), stream,
+              (void*)q_out, (const void*)qkv, ld, col0, (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot,
+              norm_last, eps, (const float*)q_mul, temp_coef, temp_every, (void*)k_cache, (void*)v_cache,
+              (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, 0);
 }
 
 // --------------------------------------------------------------------------- averaged blocks of old keys

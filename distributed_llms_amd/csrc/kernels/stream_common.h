@@ -18,6 +18,10 @@ template <int V> __device__ __forceinline__ void ldv(const bf16* p, float (&o)[V
   if constexpr (V == 2) {
     const bf16x2 v = *reinterpret_cast<const bf16x2*>(p);
     o[0] = bf2f(v[0]), o[1] = bf2f(v[1]);
+  } else if constexpr (V == 4) {
+    const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = bf2f(v[j]);
   } else if constexpr (V == 8) {
     const bf16x8 v = *reinterpret_cast<const bf16x8*>(p);
 #pragma unroll
@@ -31,6 +35,10 @@ template <int V> __device__ __forceinline__ void ldv(const float* p, float (&o)[
   if constexpr (V == 2) {
     const f32x2 v = *reinterpret_cast<const f32x2*>(p);
     o[0] = v[0], o[1] = v[1];
+  } else if constexpr (V == 4) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = v[j];
   } else if constexpr (V == 8) {
     const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
 #pragma unroll
@@ -45,6 +53,11 @@ template <int V> __device__ __forceinline__ void stv(bf16* p, const float (&o)[V
     bf16x2 v;
     v[0] = f2bf(o[0]), v[1] = f2bf(o[1]);
     *reinterpret_cast<bf16x2*>(p) = v;
+  } else if constexpr (V == 4) {
+    bf16x4 v;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = f2bf(o[j]);
+    *reinterpret_cast<bf16x4*>(p) = v;
   } else if constexpr (V == 8) {
     bf16x8 v;
 #pragma unroll
@@ -58,6 +71,8 @@ template <int V> __device__ __forceinline__ void stv(bf16* p, const float (&o)[V
 template <int V> __device__ __forceinline__ void stv(float* p, const float (&o)[V]) {
   if constexpr (V == 2) {
     *reinterpret_cast<f32x2*>(p) = f32x2{o[0], o[1]};
+  } else if constexpr (V == 4) {
+    *reinterpret_cast<f32x4*>(p) = f32x4{o[0], o[1], o[2], o[3]};
   } else if constexpr (V == 8) {
     *reinterpret_cast<f32x4*>(p) = f32x4{o[0], o[1], o[2], o[3]};
     *reinterpret_cast<f32x4*>(p + 4) = f32x4{o[4], o[5], o[6], o[7]};

@@ -14,6 +14,9 @@ def stage_class(arch: str):
     if arch == "fekizen":
         from .fekizen import FekizenStage
         return FekizenStage
+    if arch == "kupedra":
+        from .kupedra import KupedraStage
+        return KupedraStage
     if arch in ("llama", "mixtral", "gpt2"):
         from .stage import ModelStage
         return ModelStage

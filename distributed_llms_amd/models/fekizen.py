@@ -41,7 +41,7 @@ decays and states are float32 also when activations are bfloat16.
 """
 from __future__ import annotations
 
-from typing import Any, Dict, List, Optional, Tuple
+from typing import Any, Dict, Optional
 
 import torch
 
@@ -50,22 +50,11 @@ from ..config import ModelConfig
 from ..ops import linattn as la
 from ..ops import moe
 from ..ops import seqmix as sm
-from .hybrid import LayerListStage
+from .hybrid import LayerListStage, layer_runs
 from .stage import BatchMeta
 from .weights import tensor_seed
 
 DEFAULT_DECAY_RANK = 8       # synthetic weights only: a checkpoint's tensors give the rank
-
-
-def layer_runs(cfg: ModelConfig) -> List[Tuple[int, Optional[int]]]:
-    """[(layer index, number of the loop pass this run opens, or None)] in execution order."""
-    n, lp = len(cfg.layers), cfg.loop
-    if not lp:
-        return [(i, None) for i in range(n)]
-    runs: List[Tuple[int, Optional[int]]] = [(i, None) for i in range(lp["start"])]
-    for t in range(lp["times"]):
-        runs += [(i, t if i == lp["start"] else None) for i in range(lp["start"], lp["stop"])]
-    return runs + [(i, None) for i in range(lp["stop"], n)]
 
 
 def lin_spec(layer: Dict[str, Any]) -> la.LinAttnSpec:

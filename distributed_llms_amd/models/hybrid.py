@@ -28,7 +28,7 @@ unchanged; it owns every layer (no pipeline cuts, no tensor parallelism).
 """
 from __future__ import annotations
 
-from typing import Any, Dict, List, Optional
+from typing import Any, Dict, List, Optional, Tuple
 
 import torch
 
@@ -104,6 +104,18 @@ def synth_state_dict(cfg: ModelConfig, seed: int = 0, dtype=torch.float32) -> Di
             t = torch.randn(shape, generator=g) / shape[-1] ** 0.5
         sd[name] = t.to(dtype)
     return sd
+
+
+def layer_runs(cfg: ModelConfig) -> List[Tuple[int, Optional[int]]]:
+    """[(layer index, number of the loop pass this run opens, or None)] in execution order: layers
+    [loop.start, loop.stop) run ``loop.times`` times in a row."""
+    n, lp = len(cfg.layers), cfg.loop
+    if not lp:
+        return [(i, None) for i in range(n)]
+    runs: List[Tuple[int, Optional[int]]] = [(i, None) for i in range(lp["start"])]
+    for t in range(lp["times"]):
+        runs += [(i, t if i == lp["start"] else None) for i in range(lp["start"], lp["stop"])]
+    return runs + [(i, None) for i in range(lp["stop"], n)]
 
 
 class LayerListStage:

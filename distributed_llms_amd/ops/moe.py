@@ -292,37 +292,62 @@ def route_softmax_top(logits: torch.Tensor, top: int, scale: float = 1.0):
     return torch.softmax(v[:, :top], -1) * scale, ids[:, :top]
 
 
+def route_softmax_all(logits: torch.Tensor, top: int, scale: float = 1.0):
+    """Reference (PyTorch, any device): the ``top`` largest logits per row (ties: the lower index), weighted by the
+    softmax over ALL logits, not renormalised.  Returns (weights [T, top] float32, ids [T, top] int64)."""
+    _, ids = torch.sort(logits.float(), dim=-1, descending=True, stable=True)
+    return torch.softmax(logits.float(), -1).gather(1, ids[:, :top]) * scale, ids[:, :top]
+
+
+def linear_clipped_glu(x: torch.Tensor, w_gate_up: torch.Tensor, limit: float, alpha: float = 1.702) -> torch.Tensor:
+    """g sigmoid(alpha g) (u + 1) with g = min(x Wg^T, limit), u = clamp(x Wu^T, -limit, limit), W = [Wg; Wu]."""
+    from . import linear
+    from .seqmix import clipped_glu
+    return clipped_glu(linear(x, w_gate_up), None, limit, alpha)
+
+
 def softmax_top_ffn(x: torch.Tensor, w_router: torch.Tensor, b_router: Optional[torch.Tensor],
                     w_gate_up: torch.Tensor, w_down: torch.Tensor, top: int,
                     shared_gate_up: Optional[torch.Tensor] = None, shared_down: Optional[torch.Tensor] = None,
-                    scale: float = 1.0) -> torch.Tensor:
+                    scale: float = 1.0, over_all: bool = False, limit: Optional[float] = None,
+                    shared_limit: Optional[float] = None) -> torch.Tensor:
     """Mixture of GLU experts down_e(silu(gate_e x) * (up_e x)): router logits ``w_router x + b_router``
     are a float32 product (``w_router`` [E, W] and ``b_router`` [E] float32), every token uses the ``top``
     experts with the largest logits, weighted by the softmax over those logits only.  ``w_gate_up``
     [E, 2 F, W] (gate rows, then up rows), ``w_down`` [E, W, F].  ``shared_gate_up`` [2 Fs, W] /
-    ``shared_down`` [W, Fs]: an expert of the same form that every token uses, added unweighted."""
+    ``shared_down`` [W, Fs]: an expert of the same form that every token uses, added unweighted -- or, when
+    ``w_router`` has one more row [E + 1, W], times the sigmoid of that row's product, one gate per token.
+    ``over_all``: the weights are the softmax over all E logits, not renormalised over the chosen.  ``limit``
+    (``shared_limit`` for the shared expert): the experts are clipped GLUs (:func:`linear_clipped_glu`)."""
     e, two_f, width = w_gate_up.shape
     f = two_f // 2
     t = x.shape[0]
-    if w_router.shape != (e, width) or w_router.dtype != torch.float32 or (
+    rows = w_router.shape[0]
+    gated = shared_gate_up is not None and rows == e + 1
+    if w_router.shape != (e + (1 if gated else 0), width) or w_router.dtype != torch.float32 or (
             b_router is not None and (b_router.dtype != torch.float32 or b_router.numel() != e)):
-        raise ValueError("softmax_top_ffn: router [E, W] and bias [E] in float32")
+        raise ValueError("softmax_top_ffn: router [E (+ 1 with a gated shared expert), W] and bias [E] in float32")
     if not 1 <= top <= min(e, 16):
         raise ValueError("softmax_top_ffn: 1 <= top <= min(experts, 16)")
     if not x.is_cuda:
         xf = x.float()
-        tw, ids = route_softmax_top(F.linear(xf, w_router, b_router), top, scale)
+        logits = F.linear(xf, w_router)
+        choice = logits[:, :e] if b_router is None else logits[:, :e] + b_router
+        tw, ids = (route_softmax_all if over_all else route_softmax_top)(choice, top, scale)
         out = torch.zeros(t, width, dtype=torch.float32)
 
-        def glu(h, wgu, wd):
+        def glu(h, wgu, wd, lim=None):
+            if lim is not None:
+                return F.linear(linear_clipped_glu(h, wgu.float(), lim), wd.float())
             gu = F.linear(h, wgu.float())
             return F.linear(F.silu(gu[:, :wgu.shape[0] // 2]) * gu[:, wgu.shape[0] // 2:], wd.float())
         for j in range(e):
-            rows, col = (ids == j).nonzero(as_tuple=True)
-            if rows.numel():
-                out.index_add_(0, rows, glu(xf[rows], w_gate_up[j], w_down[j]) * tw[rows, col, None])
+            rw, col = (ids == j).nonzero(as_tuple=True)
+            if rw.numel():
+                out.index_add_(0, rw, glu(xf[rw], w_gate_up[j], w_down[j], limit) * tw[rw, col, None])
         if shared_gate_up is not None:
-            out += glu(xf, shared_gate_up, shared_down)
+            y = glu(xf, shared_gate_up, shared_down, shared_limit)
+            out += y * torch.sigmoid(logits[:, e:]) if gated else y
         return out.to(x.dtype)
     from . import linear
     from .latent import linear_swiglu
@@ -338,22 +363,24 @@ def softmax_top_ffn(x: torch.Tensor, w_router: torch.Tensor, b_router: Optional[
     offsets = torch.empty(e + 1, dtype=torch.int32, device=dev)
     sorted_tok = torch.empty(t * top, dtype=torch.int32, device=dev)
     inv = torch.empty(t * top, dtype=torch.int32, device=dev)
+    mode = 2 if over_all else 1
     bp = 0 if b_router is None else b_router.data_ptr()
     if t <= ROUTER_FUSED_MAX_TOKENS:
         # few tokens: the float32 router product and the selection in one launch (+ the scatter)
-        logits = torch.empty(t, e, dtype=torch.float32, device=dev)
-        k.moe_router_groups(x.data_ptr(), w_router.data_ptr(), width, e, logits.data_ptr(), bp, t, e, top, 1, 1,
-                            float(scale), 1, topk_w.data_ptr(), topk_ids.data_ptr(), counts.data_ptr(),
+        logits = torch.empty(t, rows, dtype=torch.float32, device=dev)
+        k.moe_router_groups(x.data_ptr(), w_router.data_ptr(), width, rows, logits.data_ptr(), bp, t, e, top, 1, 1,
+                            float(scale), mode, topk_w.data_ptr(), topk_ids.data_ptr(), counts.data_ptr(),
                             offsets.data_ptr(), sorted_tok.data_ptr(), inv.data_ptr(), f32, st)
     else:
         logits = F.linear(x.float(), w_router)                   # float32 also for bf16 activations
-        k.moe_route_groups(logits.data_ptr(), e, bp, t, e, top, 1, 1, float(scale), 1, topk_w.data_ptr(),
+        k.moe_route_groups(logits.data_ptr(), rows, bp, t, e, top, 1, 1, float(scale), mode, topk_w.data_ptr(),
                            topk_ids.data_ptr(), counts.data_ptr(), offsets.data_ptr(), sorted_tok.data_ptr(),
                            inv.data_ptr(), st)
     slots = t * top
     ys = torch.empty(slots, width, dtype=x.dtype, device=dev)
     bf = x.dtype == torch.bfloat16
     cp, op = counts.data_ptr(), offsets.data_ptr()
+    glu = linear_swiglu if limit is None else (lambda h, w: linear_clipped_glu(h, w, limit))
     if bf and t <= GROUPED_MAX_TOKENS and width % 128 == 0 and f % 128 == 0:
         # decode-sized: grouped GEMMs on the expert-sorted slots with the SwiGLU in the first one's
         # epilogue, no host sync (the MFMA-tiled kernel from several rows per expert on)
@@ -364,10 +391,10 @@ def softmax_top_ffn(x: torch.Tensor, w_router: torch.Tensor, b_router: Optional[
                             width, 1 | ring, st)
             k.moe_wide_gemm(ys.data_ptr(), act.data_ptr(), 0, w_down.data_ptr(), cp, op, e, width, f, ring, st)
         else:
-            rows = -(-slots // e)
+            hint = -(-slots // e)
             k.moe_grouped_gemm(act.data_ptr(), x.data_ptr(), sorted_tok.data_ptr(), w_gate_up.data_ptr(), cp, op, e,
-                               two_f, width, 1, rows, knobs.K.moe_variant, st)
-            k.moe_grouped_gemm(ys.data_ptr(), act.data_ptr(), 0, w_down.data_ptr(), cp, op, e, width, f, 0, rows,
+                               two_f, width, 1, hint, knobs.K.moe_variant, st)
+            k.moe_grouped_gemm(ys.data_ptr(), act.data_ptr(), 0, w_down.data_ptr(), cp, op, e, width, f, 0, hint,
                                knobs.K.moe_variant, st)
     elif bf and two_f % 256 == 0 and width % 256 == 0 and f % 64 == 0 and t * width * 2 < (1 << 32) \
             and slots * f * 2 < (1 << 32):
@@ -383,11 +410,12 @@ def softmax_top_ffn(x: torch.Tensor, w_router: torch.Tensor, b_router: Optional[
         for j in range(e):
             a, b = off[j], off[j + 1]
             if b > a:
-                ys[a:b] = F.linear(linear_swiglu(xs[a:b], w_gate_up[j]), w_down[j])
+                ys[a:b] = F.linear(glu(xs[a:b], w_gate_up[j]), w_down[j])
     sh = None
     if shared_gate_up is not None:
-        sh = linear(linear_swiglu(x, shared_gate_up), shared_down)
+        sg = linear_swiglu(x, shared_gate_up) if shared_limit is None else linear_clipped_glu(x, shared_gate_up, shared_limit)
+        sh = linear(sg, shared_down)
     out = torch.empty_like(x)
     k.moe_combine_gated(out.data_ptr(), ys.data_ptr(), topk_w.data_ptr(), inv.data_ptr(), 0 if sh is None else sh.data_ptr(),
-                        0, 0, t, width, top, f32, st)
+                        logits.data_ptr() + 4 * e if gated else 0, rows, t, width, top, f32, st)
     return out

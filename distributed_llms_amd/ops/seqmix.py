@@ -5,7 +5,8 @@ recurrent unit (RG-LRU), sliding-window and chunked attention over a paged K/V c
 widths differ (optionally with capped scores, per-head sinks and one averaged key / value per block of
 positions older than the window), two attention input stages (convolution + per-head norm + interleaved
 rotation; whole-projection norm + half-split rotation, also without norms and with the values taken from
-the keys), the close of pre-norm sublayers whose outputs are normed apart, a token shift, the entry of a
+the keys; per-head norm before or after a paired rotation with query temperatures), a learned bias per distance
+bucket, the close of pre-norm sublayers whose outputs are normed apart, a token shift, the entry of a
 looped span of layers, a clipped GLU and the logit soft cap.
 
 Same dispatch as :mod:`distributed_llms_amd.ops`: a CUDA tensor goes to the in-tree HIP kernels
@@ -23,6 +24,7 @@ from __future__ import annotations
 
 import math
 from dataclasses import dataclass
+from fractions import Fraction
 from typing import Optional, Tuple
 
 import torch
@@ -392,14 +394,14 @@ def clipped_glu(gu: torch.Tensor, bias_gu: Optional[torch.Tensor], limit: float,
     return out
 
 
-def softcap_f32(logits: torch.Tensor, cap: float) -> torch.Tensor:
-    """float32 cap * tanh(logits / cap) (cap <= 0: a plain float32 copy)."""
+def softcap_f32(logits: torch.Tensor, cap: float, scale: float = 1.0) -> torch.Tensor:
+    """float32 cap * tanh(z / cap) with z = logits * scale (cap <= 0: z itself)."""
     if not logits.is_cuda:
-        x = logits.float()
+        x = logits.float() * scale
         return cap * torch.tanh(x / cap) if cap > 0 else x
     _ck(logits, "logits")
     out = torch.empty(logits.shape, dtype=torch.float32, device=logits.device)
-    _k().sm_softcap(out.data_ptr(), logits.data_ptr(), logits.numel(), float(cap), _f32flag(logits), _stream())
+    _k().sm_softcap(out.data_ptr(), logits.data_ptr(), logits.numel(), float(cap), float(scale), _f32flag(logits), _stream())
     return out
 
 
@@ -496,9 +498,10 @@ def attn_prep(qkv: torch.Tensor, conv_w: torch.Tensor, state: torch.Tensor, q_no
 
 
 # ------------------------------------------------------------------ attention input: row norm + half-split rotation + append
-def rotary_frequencies(dims: int, base: float) -> torch.Tensor:
-    """f_i = base^(-2i / dims), i < dims / 2, computed in float64 and rounded once to float32."""
-    return yarn_frequencies(dims, base, None)[0]
+def rotary_frequencies(dims: int, base: float, factor: float = 1.0) -> torch.Tensor:
+    """f_i = base^(-2i / dims) / factor, i < dims / 2, computed in float64 and rounded once to float32."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    return (torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims) / factor).float()
 
 
 def _ref_rope_half(x: torch.Tensor, pos: torch.Tensor, freqs: torch.Tensor, mag: float = 1.0) -> torch.Tensor:
@@ -563,6 +566,99 @@ def rownorm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor], k
     return q
 
 
+# ------------------------------------------------------------------ attention input: per-head norm + paired rotation + append
+def head_norm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor],
+                   freqs: Optional[torch.Tensor], eps: float, k_cache: torch.Tensor, v_cache: torch.Tensor,
+                   slot_mapping: torch.Tensor, positions: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int,
+                   norm_last: bool = False, q_mul: Optional[torch.Tensor] = None,
+                   q_temp: Optional[Tuple[float, int]] = None) -> torch.Tensor:
+    """From columns ``col0 ..`` of a fused projection [T, .. | q (heads dim) | k (kv_heads dim) | v (kv_heads
+    vdim) | ..]: an RMS norm of every q and k head over its ``dim`` (plain weights ``q_norm`` / ``k_norm`` [dim] shared
+    by the heads; both None: no weight), before or -- ``norm_last`` -- after the rotation of its first 2 len(freqs)
+    dimensions, pairs (2i, 2i + 1) turning by position * freqs[i] (None: no rotation).  q is then multiplied by
+    ``q_mul`` [heads] float32 and by 1 + coef ln(floor((position + 1) / every) + 1) with ``q_temp`` = (coef, every); k and
+    v (unchanged) are appended at ``slot_mapping`` to caches k [NB, kv_heads, BS, dim] / v [NB, kv_heads, vdim, BS].
+    Returns q [T, heads, dim]."""
+    t = qkv.shape[0]
+    nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
+    nrot = 0 if freqs is None else freqs.numel()
+    if (q_norm is None) != (k_norm is None) or 2 * nrot > dim or (q_norm is not None and (q_norm.numel() != dim or
+                                                                                          k_norm.numel() != dim)):
+        raise ValueError("head_norm_rope: norm weights [dim] for both or neither; rotated dims fit the head")
+    bs = k_cache.shape[2]
+    if qkv.shape[1] < col0 + nq + nk + nv or k_cache.shape[1:] != (kv_heads, bs, dim) or v_cache.shape[1:] != (kv_heads, vdim, bs):
+        raise ValueError("head_norm_rope: shape mismatch")
+    if q_mul is not None and (q_mul.dtype != torch.float32 or q_mul.numel() != heads):
+        raise ValueError("head_norm_rope: q_mul [heads] float32")
+    coef, every = (0.0, 0) if q_temp is None else (float(q_temp[0]), int(q_temp[1]))
+    if q_temp is not None and every < 1:
+        raise ValueError("head_norm_rope: q_temp period")
+    if not qkv.is_cuda:
+        def prep(x, w):
+            turn = (lambda a: a) if nrot == 0 else (lambda a: _ref_rope_interleaved(a, positions, freqs, 1.0))
+            x = turn(x) if norm_last else x
+            x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+            x = x if w is None else x * w.float()
+            return x if norm_last else turn(x)
+        q = prep(qkv[:, col0:col0 + nq].float().reshape(t, heads, dim), q_norm)
+        k = prep(qkv[:, col0 + nq:col0 + nq + nk].float().reshape(t, kv_heads, dim), k_norm)
+        if q_mul is not None:
+            q = q * q_mul[None, :, None]
+        if every:
+            q = q * (1.0 + coef * torch.log(((positions + 1) // every).float() + 1.0))[:, None, None]
+        slot = slot_mapping.long()
+        k_cache[slot // bs, :, slot % bs] = k.to(k_cache.dtype)
+        v_cache[slot // bs, :, :, slot % bs] = qkv[:, col0 + nq + nk:col0 + nq + nk + nv].reshape(t, kv_heads, vdim).to(v_cache.dtype)
+        return q.to(qkv.dtype)
+    _ck(qkv, "qkv")
+    if q_norm is not None:
+        _ck(q_norm, "q_norm", qkv.dtype)
+        _ck(k_norm, "k_norm", qkv.dtype)
+    if nrot:
+        _ck(freqs, "freqs", torch.float32)
+    if q_mul is not None:
+        _ck(q_mul, "q_mul", torch.float32)
+    _ck(k_cache, "k_cache", qkv.dtype)
+    _ck(v_cache, "v_cache", qkv.dtype)
+    _ck(positions, "positions", torch.int32)
+    _ck(slot_mapping, "slot_mapping", torch.int32)
+    q = torch.empty(t, heads, dim, dtype=qkv.dtype, device=qkv.device)
+    _k().sm_head_norm_rope(q.data_ptr(), qkv.data_ptr(), qkv.shape[1], int(col0), _ptr(q_norm), _ptr(k_norm),
+                           _ptr(freqs) if nrot else 0, nrot, 1 if norm_last else 0, float(eps), _ptr(q_mul), coef, every,
+                           k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), positions.data_ptr(), t, heads,
+                           kv_heads, dim, vdim, bs, _f32flag(qkv), _stream())
+    return q
+
+
+# ------------------------------------------------------------------ distance bias
+def bucket_thresholds(rows: int, far: float) -> list:
+    """First distance of every row of a distance-bias table with ``rows`` rows: row r < rows // 2 is distance r
+    alone; above, row half + k starts where half (far / half)^(k / (rows - half)) is reached, and everything from
+    the last row's start on shares it.  Exact (integer powers), so that a distance that lies ON a border -- far /
+    half a perfect power -- falls on the same side everywhere."""
+    half = rows // 2
+    if half < 1 or far <= half:
+        raise ValueError("distance bias: needs rows >= 2 and a far distance beyond half the rows")
+    m, far = rows - half, Fraction(far)
+    out = list(range(half))
+    n = half
+    for k in range(m):
+        # smallest n with (n / half)^m >= (far / half)^k
+        while n ** m * half ** k < half ** m * far ** k:
+            n += 1
+        out.append(n)
+    return out
+
+
+def distance_bias_table(rel: torch.Tensor, far: float) -> torch.Tensor:
+    """The bias per head and distance [H, L] float32 from a bucketed table ``rel`` [rows, H]: entry n is the row of
+    :func:`bucket_thresholds` that distance n falls into, the last entry stands for every distance >= L - 1."""
+    th = bucket_thresholds(rel.shape[0], far)
+    n = torch.arange(th[-1] + 1)
+    row = torch.searchsorted(torch.tensor(th), n, right=True) - 1
+    return rel.float()[row.to(rel.device)].t().contiguous()
+
+
 # ------------------------------------------------------------------ averaged blocks of old keys
 def pooled_block_size(block_size: int, pool: int) -> int:
     """Entries per cache block of the averaged-key cache: a power of two >= 8 that holds at least
@@ -622,7 +718,8 @@ def decode_splits(rows: int, heads: int, kv_heads: int, ctx: int) -> int:
 def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
                      sb: SeqBatch, window: int, scale: float, num_decode: Optional[int] = None,
                      sinks: Optional[torch.Tensor] = None, max_ctx: Optional[int] = None, chunk: int = 0,
-                     softcap: float = 0.0, pooled: Optional[tuple] = None) -> torch.Tensor:
+                     softcap: float = 0.0, pooled: Optional[tuple] = None,
+                     bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Softmax attention of every query token over the keys j of its own sequence with
     0 <= p - j < window (p the query's position) and, with ``chunk`` > 0, floor(j / chunk) =
     floor(p / chunk) (attention inside fixed chunks of positions counted from position 0, wherever a
@@ -639,7 +736,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     averaged key and value for every block of ``pool`` positions that lies wholly before the window -- entries
     b < floor((p - window + 1) / pool) of the averaged caches (:func:`pool_blocks`), scored, capped and
     normalised in the same softmax; tokens that left the window inside a block not yet complete are not
-    seen at all.  Returns [T, H, vdim]."""
+    seen at all.  ``bias`` [H, L] float32 (:func:`distance_bias_table`): bias[h][min(n, L - 1)] is added to the scaled
+    score of a key n positions back (not beside averaged caches).  Returns [T, H, vdim]."""
     t, h, d = q.shape
     g, bs, dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[2]
     kp = vp = None
@@ -649,6 +747,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         pb = kp.shape[2]
         if pool < 1 or chunk or kp.shape[1:] != (g, pb, d) or vp.shape[1:] != (g, dv, pb) or pb * pool < bs:
             raise ValueError("window_attention: averaged caches do not fit (and exclude a chunk mask)")
+    if bias is not None and (pool or bias.dtype != torch.float32 or bias.dim() != 2 or bias.shape[0] != h):
+        raise ValueError("window_attention: bias [H, L] float32 (and no averaged caches)")
     if not q.is_cuda:
         out = torch.empty(t, h, dv, dtype=torch.float32)
         pos, seq = sb.positions.tolist(), sb.tok_seq.tolist()
@@ -668,6 +768,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             s = torch.einsum("hd,nhd->hn", q[i].float(), kk) * scale
             if softcap > 0:
                 s = softcap * torch.tanh(s / softcap)
+            if bias is not None:
+                s = s + bias[:, torch.clamp(p - idx, max=bias.shape[1] - 1)]
             if sinks is not None:      # one more column in the softmax whose weight is dropped
                 pr = torch.softmax(torch.cat([s, sinks.float()[:, None]], -1), -1)[:, :-1]
             else:
@@ -687,6 +789,10 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     if pool:
         _ck(kp, "kp_cache", q.dtype)
         _ck(vp, "vp_cache", q.dtype)
+    nbias = 0
+    if bias is not None:
+        _ck(bias, "bias", torch.float32)
+        nbias = bias.shape[1]
     out = torch.empty(t, h, dv, dtype=q.dtype, device=q.device)
     nd = sb.num_seqs if num_decode is None else int(num_decode)
     f = _f32flag(q)
@@ -701,12 +807,12 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                                    block_tables.data_ptr(), block_tables.shape[1], sb.positions.data_ptr(),
                                    sb.tok_seq.data_ptr(), nd, h, g, d, dv, bs, int(window), int(chunk), float(scale), _ptr(sinks),
                                    splits if ws is not None else 1, _ptr(ws), float(softcap), _ptr(kp), _ptr(vp), int(pool),
-                                   int(pb), f, _stream())
+                                   int(pb), _ptr(bias), nbias, f, _stream())
     if t > nd:
         _k().sm_window_attn_prefill(out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                                     block_tables.data_ptr(), block_tables.shape[1], sb.cu.data_ptr(),
                                     sb.positions.data_ptr(), sb.tok_seq.data_ptr(), nd, sb.num_seqs, t, sb.max_q_len,
                                     h, g, d, dv, bs,
                                     int(window), int(chunk), float(scale), _ptr(sinks), float(softcap), _ptr(kp), _ptr(vp),
-                                    int(pool), int(pb), f, _stream())
+                                    int(pool), int(pb), _ptr(bias), nbias, f, _stream())
     return out
