@@ -93,7 +93,9 @@ def parse(argv=None):
                          "or gikovik,mixtral (latent attention + grouped-choice experts beside Mixtral), or "
                          "zebutar,mixtral (chunked attention beside a gated delta rule + SwiGLU experts beside "
                          "Mixtral), or fekizen,zebutar,mixtral (window attention with averaged blocks beside gated "
-                         "linear attention, lightning layers + SwiGLU experts, beside both), or one of them")
+                         "linear attention, lightning layers + SwiGLU experts, beside both), or "
+                         "kupedra,fekizen,mixtral (hyper-connected streams, distance-biased attention beside a gated "
+                         "matrix memory + clipped-GLU experts, beside both), or one of them")
     return ap.parse_args(argv)
 
 

@@ -19,7 +19,8 @@ PYBIND11_MODULE(_C_kernels, m) {
   m.def("argmax", &dllm::argmax);
   m.def("add_inplace", &dllm::add_inplace);
   m.def("moe_route", &dllm::moe_route);
-  m.def("moe_grouped_gemm", &dllm::moe_grouped_gemm);
+  m.def("moe_grouped_gemm", &dllm::moe_grouped_gemm, py::arg("y"), py::arg("x"), py::arg("gather"), py::arg("w"), py::arg("counts"), py::arg("offsets"), py::arg("experts"), py::arg("n"), py::arg("k"), py::arg("mode"), py::arg("rows_hint"), py::arg("variant"), py::arg("stream"),
+        py::arg("limit") = 0.f);
   m.def("splitk_add_rms_norm", &dllm::splitk_add_rms_norm);
   m.def("splitk_reduce", &dllm::splitk_reduce);
   m.def("gemm_wide", &dllm::gemm_wide);
@@ -29,11 +30,13 @@ PYBIND11_MODULE(_C_kernels, m) {
   m.def("moe_wide_gemm_fp8", &dllm::moe_wide_gemm_fp8);
   m.def("splitk_add_rms_norm_q8", &dllm::splitk_add_rms_norm_q8);
   m.def("gemm_sq", &dllm::gemm_sq);
-  m.def("gemm_pp_moe", &dllm::gemm_pp_moe);
+  m.def("gemm_pp_moe", &dllm::gemm_pp_moe, py::arg("y"), py::arg("x"), py::arg("gather"), py::arg("w"), py::arg("counts"), py::arg("offsets"), py::arg("experts"), py::arg("n"), py::arg("k"), py::arg("xrows"), py::arg("slots"), py::arg("mode"), py::arg("stream"),
+        py::arg("limit") = 0.f);
   m.def("gemm_pp", &dllm::gemm_pp);
   m.def("gemm_pf", &dllm::gemm_pf);
   m.def("moe_combine", &dllm::moe_combine);
-  m.def("moe_wide_gemm", &dllm::moe_wide_gemm);
+  m.def("moe_wide_gemm", &dllm::moe_wide_gemm, py::arg("y"), py::arg("x"), py::arg("gather"), py::arg("w"), py::arg("counts"), py::arg("offsets"), py::arg("experts"), py::arg("n"), py::arg("k"), py::arg("mode"), py::arg("stream"),
+        py::arg("limit") = 0.f);
   m.def("moe_router_route", &dllm::moe_router_route);
   m.def("paged_attention_decode", &dllm::paged_attention_decode);
   m.def("paged_attention_decode_rope", &dllm::paged_attention_decode_rope);

@@ -80,6 +80,15 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 // result to bf16
 __device__ __forceinline__ float silu_f(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 
+// Clipped GLU g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit): the expert
+// activation of the grouped GEMMs' epilogues (rounded to bf16 by every caller, hence the hardware reciprocal)
+constexpr float kGluAlpha = 1.702f;
+__device__ __forceinline__ float clipped_glu_f(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * __builtin_amdgcn_rcpf(1.f + __expf(-kGluAlpha * g)) * (u + 1.0f);
+}
+
 // f32 -> bf16 via the compiler cast: gfx950 emits v_cvt_pk_bf16_f32 (RNE, NaN-preserving).
 __device__ __forceinline__ bf16 f2bf(float x) { return (bf16)x; }
 __device__ __forceinline__ float bf2f(bf16 x) { return (float)x; }

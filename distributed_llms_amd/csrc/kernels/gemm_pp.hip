@@ -156,7 +156,7 @@ __global__ void __launch_bounds__(256, 1) gemm_pp_kernel(const bf16* __restrict_
                                                          bf16* __restrict__ C, float* __restrict__ P, int M, int N,
                                                          int K, int ks_per_split, int nsplit, float* __restrict__ D,
                                                          const int* __restrict__ gather, const int* __restrict__ counts,
-                                                         const int* __restrict__ offsets, int E) {
+                                                         const int* __restrict__ offsets, int E, float limit = 0.f) {
   constexpr int NW = 4, NWN = 2;
   constexpr int BM = 256, TM = 128, TN = BN / NWN;     // waves as 2 (M) x NWN (N)
   constexpr int RT = TM / 16, CT = TN / 16;            // 16 x 16 fragments per wave: 8 x 8 or 8 x 4
@@ -173,6 +173,8 @@ __global__ void __launch_bounds__(256, 1) gemm_pp_kernel(const bf16* __restrict_
   // of bunched into half of K-half 1 (see the loop)
   constexpr bool SCHED2 = (VAR & 32) != 0;
   constexpr bool SWIGLU = MODE == 2;
+  // VAR bit 9, with SwiGLU on schedule 2: the clipped GLU of `limit` (common.h) instead of silu(g) * u
+  constexpr bool CLIPPED = (VAR & 512) != 0;
   constexpr int OUTW = SWIGLU ? BN / 2 : BN;           // output tile width (elements)
   // schedule 2 + SwiGLU: the epilogue stages gate and up as bf16 (the image is the full BN wide)
   // and applies silu(g) * u while storing -- the fused fp32 form kept the accumulators live
@@ -607,7 +609,8 @@ __global__ void __launch_bounds__(256, 1) gemm_pp_kernel(const bf16* __restrict_
       const bf16x8 u = *reinterpret_cast<const bf16x8*>(smem + r * OPITCH + icol + 16);
       bf16x8 h;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) h[e] = f2bf(silu_f(bf2f(g[e])) * bf2f(u[e]));
+      for (int e = 0; e < 8; ++e)
+        h[e] = f2bf(CLIPPED ? clipped_glu_f(bf2f(g[e]), bf2f(u[e]), limit) : silu_f(bf2f(g[e])) * bf2f(u[e]));
       v = *reinterpret_cast<const int4*>(&h);
     }
     if constexpr (MODE == 1) {
@@ -655,7 +658,7 @@ int gemm_pp(uintptr_t c, uintptr_t a, uintptr_t b, uintptr_t ws, long ws_floats,
 #define DLLM_PP_GO(BN_, MODE_, VAR_)                                                                     \
   hipLaunchKernelGGL((gemm_pp_kernel<BN_, MODE_, VAR_>), dim3((unsigned)grid), dim3(256), 0, s, (const bf16*)a, \
                      (const bf16*)b, (bf16*)c, (float*)ws, M, N, K, kps, S, dbg, (const int*)nullptr,       \
-                     (const int*)nullptr, (const int*)nullptr, 0)
+                     (const int*)nullptr, (const int*)nullptr, 0, 0.f)
   // variant bit 6: schedule 2 (the K-tile's fragments read early, staging spread; weights
   // nontemporal with bit 1 only in the natural tile order).  Bit 3: diagnostic build -- per-wave cycle stamps (loop, B_t waits) into the LAST
   // grid x 512 floats of ws (after the slabs); output as usual.  With it (schedule 1 only), bit 4:
@@ -708,11 +711,11 @@ int gemm_pp(uintptr_t c, uintptr_t a, uintptr_t b, uintptr_t ws, long ws_floats,
 // y [slots, N] (SwiGLU: [slots, N / 2]).  Schedule 2, 256 x 256 tiles, grouped row-tile order.
 // xrows: rows of x (buffer range), slots: total slot count (grid bound: slots / 256 + E row tiles).
 void gemm_pp_moe(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintptr_t counts, uintptr_t offsets, int E,
-                 int N, int K, int xrows, int slots, int mode, uintptr_t stream) {
+                 int N, int K, int xrows, int slots, int mode, uintptr_t stream, float limit) {
   DLLM_HOST_CHECK(E >= 1 && E <= 256, "1 <= experts <= 256");
   DLLM_HOST_CHECK(K % PBK == 0 && K >= PBK, "K must be a positive multiple of 64");
   DLLM_HOST_CHECK(N % 256 == 0, "N must be a multiple of 256");
-  DLLM_HOST_CHECK(mode == 0 || mode == 1 || mode == 2, "mode 0 (plain), 1 (SwiGLU) or 2 (squared ReLU)");
+  DLLM_HOST_CHECK(mode >= 0 && mode <= 3, "mode 0 (plain), 1 (SwiGLU), 2 (squared ReLU) or 3 (clipped GLU)");
   DLLM_HOST_CHECK(xrows >= 1 && slots >= 1, "rows");
   DLLM_HOST_CHECK((long)xrows * K * 2 < (1L << 32) && (long)N * K * 2 < (1L << 32), "operands must be < 4 GiB");
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
@@ -721,15 +724,19 @@ void gemm_pp_moe(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintpt
   if (mode == 1)
     hipLaunchKernelGGL((gemm_pp_kernel<256, 2, 128 | 32 | 2>), dim3((unsigned)grid), dim3(256), 0, s, (const bf16*)x,
                        (const bf16*)w, (bf16*)y, (float*)nullptr, xrows, N, K, K / PBK, 1, (float*)nullptr,
-                       (const int*)gather, (const int*)counts, (const int*)offsets, E);
+                       (const int*)gather, (const int*)counts, (const int*)offsets, E, limit);
+  else if (mode == 3)
+    hipLaunchKernelGGL((gemm_pp_kernel<256, 2, 512 | 128 | 32 | 2>), dim3((unsigned)grid), dim3(256), 0, s, (const bf16*)x,
+                       (const bf16*)w, (bf16*)y, (float*)nullptr, xrows, N, K, K / PBK, 1, (float*)nullptr,
+                       (const int*)gather, (const int*)counts, (const int*)offsets, E, limit);
   else if (mode == 2)
     hipLaunchKernelGGL((gemm_pp_kernel<256, 3, 128 | 32 | 2>), dim3((unsigned)grid), dim3(256), 0, s, (const bf16*)x,
                        (const bf16*)w, (bf16*)y, (float*)nullptr, xrows, N, K, K / PBK, 1, (float*)nullptr,
-                       (const int*)gather, (const int*)counts, (const int*)offsets, E);
+                       (const int*)gather, (const int*)counts, (const int*)offsets, E, limit);
   else
     hipLaunchKernelGGL((gemm_pp_kernel<256, 0, 128 | 32 | 2>), dim3((unsigned)grid), dim3(256), 0, s, (const bf16*)x,
                        (const bf16*)w, (bf16*)y, (float*)nullptr, xrows, N, K, K / PBK, 1, (float*)nullptr,
-                       (const int*)gather, (const int*)counts, (const int*)offsets, E);
+                       (const int*)gather, (const int*)counts, (const int*)offsets, E, limit);
   DLLM_HIP_CHECK(hipGetLastError());
 }
 

@@ -129,11 +129,12 @@ __device__ __forceinline__ void grouped_tile(int b, int mtiles, int ntiles, int&
 // SCALED (fp8 operands): the accumulator is in quantized units; output = acc * sa[m] * sb[n]
 // (per-token activation scale x per-output-channel weight scale), applied before the SwiGLU and
 // before a split-K slab store (the cross-slice sum is linear in it).
-template <int BM, bool SPLIT, bool SWIGLU, bool SCALED = false>
+// CLIPPED (with SWIGLU's row layout): the clipped GLU of `limit` instead of silu(g) * u
+template <int BM, bool SPLIT, bool SWIGLU, bool SCALED = false, bool CLIPPED = false>
 __device__ __forceinline__ void wide_epilogue(const f32x4 (&acc)[BM / 64][4], bf16* __restrict__ C,
                                               float* __restrict__ P, int M, int N, int m0, int n_t, int split, int wm,
                                               int wn, int lane, const float* __restrict__ sa = nullptr,
-                                              const float* __restrict__ sb = nullptr) {
+                                              const float* __restrict__ sb = nullptr, float limit = 0.f) {
   constexpr int RT = BM / 64;
   const int fr = lane & 15, fq = lane >> 4;
   float sbn[4];
@@ -166,7 +167,7 @@ __device__ __forceinline__ void wide_epilogue(const f32x4 (&acc)[BM / 64][4], bf
         for (int p = 0; p < 2; ++p) {
           const int c = n_t * 64 + (wn * 2 + p) * 16 + fr;
           const float g = v[2 * p], u = v[2 * p + 1];
-          C[(size_t)m * half + c] = f2bf(silu_f(g) * u);
+          C[(size_t)m * half + c] = f2bf(CLIPPED ? clipped_glu_f(g, u, limit) : silu_f(g) * u);
         }
       } else {
 #pragma unroll
@@ -547,12 +548,12 @@ __global__ void __launch_bounds__(512, 1) gemm_wide_fp8_kernel(const uint8_t* __
 // the decode regime of Mixtral at B >= 128 (32-128 rows per expert), where the weight-streaming
 // grouped kernel (moe.hip) runs its MFMAs at a fraction of the rate.
 // ---------------------------------------------------------------------------------------------
-template <int BM, bool SWIGLU, int VAR, bool FP8 = false, int NBUF = 3>
+template <int BM, bool SWIGLU, int VAR, bool FP8 = false, int NBUF = 3, bool CLIPPED = false>
 __device__ __forceinline__ void moe_wide_rows(bf16* smem, bf16* __restrict__ Y, const bf16* __restrict__ X,
                                               const int* __restrict__ gather, const bf16* __restrict__ We, int cnt,
                                               int off, int N, int K, int n_t, int wv, int lane,
                                               const float* __restrict__ sa = nullptr,
-                                              const float* __restrict__ sb = nullptr) {
+                                              const float* __restrict__ sb = nullptr, float limit = 0.f) {
   // FP8: X / We hold e4m3 bytes addressed in 2-byte units (K / 2 per row); sa: per-slot activation
   // scales (slot order), sb: this expert's per-channel weight scales
   constexpr int AI = BM / 64, BI = 2, RT = BM / 64;
@@ -577,8 +578,8 @@ __device__ __forceinline__ void moe_wide_rows(bf16* smem, bf16* __restrict__ Y, 
     }
     f32x4 acc[RT][4];
     wide_mainloop<BM, NBUF, VAR, FP8>(smem, srcA, srcB, KU / WBK, acc, wv, lane);
-    wide_epilogue<BM, false, SWIGLU, FP8>(acc, Y + (size_t)(off + r0) * ldy, nullptr, rows, N, 0, n_t, 0, wm, wn,
-                                          lane, FP8 ? sa + off + r0 : nullptr, sb);
+    wide_epilogue<BM, false, SWIGLU, FP8, CLIPPED>(acc, Y + (size_t)(off + r0) * ldy, nullptr, rows, N, 0, n_t, 0, wm, wn,
+                                          lane, FP8 ? sa + off + r0 : nullptr, sb, limit);
     __syncthreads();   // the next chunk's prologue refills buffers other waves may still read
   }
 }
@@ -593,13 +594,13 @@ constexpr int moe_nbuf() {
   return NBUF_SEL == 0 ? 3 : (BM == 64 ? 6 : 5);
 }
 
-template <bool SWIGLU, bool FP8 = false, int NBUF_SEL = 1>
+template <bool SWIGLU, bool FP8 = false, int NBUF_SEL = 1, bool CLIPPED = false>
 __global__ void __launch_bounds__(512, 1) moe_wide_kernel(bf16* __restrict__ Y, const bf16* __restrict__ X,
                                                           const int* __restrict__ gather, const bf16* __restrict__ W,
                                                           const int* __restrict__ counts,
                                                           const int* __restrict__ offsets, int N, int K, int nt,
                                                           const float* __restrict__ sa = nullptr,
-                                                          const float* __restrict__ wscale = nullptr) {
+                                                          const float* __restrict__ wscale = nullptr, float limit = 0.f) {
   static_assert(moe_nbuf<64, NBUF_SEL>() * (64 + WBN) * WBK <= MOE_LDS &&
                 moe_nbuf<128, NBUF_SEL>() * (128 + WBN) * WBK <= MOE_LDS, "LDS");
   __shared__ __attribute__((aligned(16))) bf16 smem[MOE_LDS];
@@ -614,34 +615,40 @@ __global__ void __launch_bounds__(512, 1) moe_wide_kernel(bf16* __restrict__ Y, 
   // an expert's weight tile is read once when its rows fit one row tile: stream it nt (variant 2);
   // with several row chunks the re-reads should hit the caches (default policy)
   if (cnt <= 64) {
-    if (nt) moe_wide_rows<64, SWIGLU, 2, FP8, NB64>(smem, Y, X, gather, We, cnt, off, N, K, blockIdx.x, wv, lane, sa, sb);
-    else moe_wide_rows<64, SWIGLU, 1, FP8, NB64>(smem, Y, X, gather, We, cnt, off, N, K, blockIdx.x, wv, lane, sa, sb);
+    if (nt) moe_wide_rows<64, SWIGLU, 2, FP8, NB64, CLIPPED>(smem, Y, X, gather, We, cnt, off, N, K, blockIdx.x, wv, lane, sa, sb,
+        limit);
+    else moe_wide_rows<64, SWIGLU, 1, FP8, NB64, CLIPPED>(smem, Y, X, gather, We, cnt, off, N, K, blockIdx.x, wv, lane, sa, sb,
+        limit);
   } else if (cnt <= 128 && nt) {
-    moe_wide_rows<128, SWIGLU, 2, FP8, NB128>(smem, Y, X, gather, We, cnt, off, N, K, blockIdx.x, wv, lane, sa, sb);
+    moe_wide_rows<128, SWIGLU, 2, FP8, NB128, CLIPPED>(smem, Y, X, gather, We, cnt, off, N, K, blockIdx.x, wv, lane, sa, sb,
+        limit);
   } else {
-    moe_wide_rows<128, SWIGLU, 1, FP8, NB128>(smem, Y, X, gather, We, cnt, off, N, K, blockIdx.x, wv, lane, sa, sb);
+    moe_wide_rows<128, SWIGLU, 1, FP8, NB128, CLIPPED>(smem, Y, X, gather, We, cnt, off, N, K, blockIdx.x, wv, lane, sa, sb,
+        limit);
   }
 }
 
-// mode 1 (SwiGLU): W [E, 2I, K] -> Y [slots, I]; mode 0: W [E, N, K] -> Y [slots, N]
+// mode 1 (SwiGLU): W [E, 2I, K] -> Y [slots, I]; mode 0: W [E, N, K] -> Y [slots, N]; mode 3: as 1 with the clipped GLU
+// of `limit`
 void moe_wide_gemm(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintptr_t counts, uintptr_t offsets,
-                   int E, int N, int K, int mode, uintptr_t stream) {
+                   int E, int N, int K, int mode, uintptr_t stream, float limit) {
   DLLM_HOST_CHECK(E >= 1, "experts >= 1");
   DLLM_HOST_CHECK(K % WBK == 0, "K must be a multiple of 64");
   DLLM_HOST_CHECK(N % 128 == 0, "N must be a multiple of 128");
   // mode bit 2: the 3-slot ring instead of the deep one (A/B runs)
   const bool shallow = (mode & 4) != 0;
   mode &= 3;
-  DLLM_HOST_CHECK(mode == 0 || mode == 1, "mode");
+  DLLM_HOST_CHECK(mode == 0 || mode == 1 || mode == 3, "mode");
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-  const int ntiles = mode == 1 ? (N / 2) / 64 : N / WBN;
+  const int ntiles = mode != 0 ? (N / 2) / 64 : N / WBN;
   constexpr int nt = 1;   // expert weights are read once per step: nontemporal
-#define DLLM_MOE_GO(SW_, SEL_)                                                                                   \
-  hipLaunchKernelGGL((moe_wide_kernel<SW_, false, SEL_>), dim3(ntiles, E), dim3(512), 0, s, (bf16*)y,            \
+#define DLLM_MOE_GO(SW_, SEL_, CL_)                                                                                   \
+  hipLaunchKernelGGL((moe_wide_kernel<SW_, false, SEL_, CL_>), dim3(ntiles, E), dim3(512), 0, s, (bf16*)y,            \
                      (const bf16*)x, (const int*)gather, (const bf16*)w, (const int*)counts, (const int*)offsets, N, \
-                     K, nt, (const float*)nullptr, (const float*)nullptr)
-  if (mode == 1) { if (shallow) DLLM_MOE_GO(true, 0); else DLLM_MOE_GO(true, 1); }
-  else { if (shallow) DLLM_MOE_GO(false, 0); else DLLM_MOE_GO(false, 1); }
+                     K, nt, (const float*)nullptr, (const float*)nullptr, limit)
+  if (mode == 3) DLLM_MOE_GO(true, 1, true);
+  else if (mode == 1) { if (shallow) DLLM_MOE_GO(true, 0, false); else DLLM_MOE_GO(true, 1, false); }
+  else { if (shallow) DLLM_MOE_GO(false, 0, false); else DLLM_MOE_GO(false, 1, false); }
 #undef DLLM_MOE_GO
   DLLM_HIP_CHECK(hipGetLastError());
 }
@@ -661,11 +668,11 @@ void moe_wide_gemm_fp8(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, 
   if (mode == 1)
     hipLaunchKernelGGL((moe_wide_kernel<true, true>), dim3(ntiles, E), dim3(512), 0, s, (bf16*)y, (const bf16*)x,
                        (const int*)gather, (const bf16*)w, (const int*)counts, (const int*)offsets, N, K, nt,
-                       (const float*)sa, (const float*)wscale);
+                       (const float*)sa, (const float*)wscale, 0.f);
   else
     hipLaunchKernelGGL((moe_wide_kernel<false, true>), dim3(ntiles, E), dim3(512), 0, s, (bf16*)y, (const bf16*)x,
                        (const int*)gather, (const bf16*)w, (const int*)counts, (const int*)offsets, N, K, nt,
-                       (const float*)sa, (const float*)wscale);
+                       (const float*)sa, (const float*)wscale, 0.f);
   DLLM_HIP_CHECK(hipGetLastError());
 }
 

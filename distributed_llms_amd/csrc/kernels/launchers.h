@@ -35,7 +35,7 @@ void quant_fp8_rows(uintptr_t q, uintptr_t scale, uintptr_t x, int M, int K, uin
 int gemm_pp(uintptr_t c, uintptr_t a, uintptr_t b, uintptr_t ws, long ws_floats, int M, int N, int K, int splits,
             int mode, int variant, uintptr_t stream);
 void gemm_pp_moe(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintptr_t counts, uintptr_t offsets, int E,
-                 int N, int K, int xrows, int slots, int mode, uintptr_t stream);
+                 int N, int K, int xrows, int slots, int mode, uintptr_t stream, float limit);
 void gemm_pf(uintptr_t c, uintptr_t a, uintptr_t b, int M, int N, int K, int mode, int variant, uintptr_t stream);
 int gemm_sq(uintptr_t c, uintptr_t a, uintptr_t b, uintptr_t ws, long ws_floats, int M, int N, int K, int splits,
             int mode, int variant, uintptr_t stream);
@@ -43,11 +43,11 @@ int gemm_sq(uintptr_t c, uintptr_t a, uintptr_t b, uintptr_t ws, long ws_floats,
 void moe_route(uintptr_t logits, int T, int E, int k, uintptr_t topk_w, uintptr_t topk_ids, uintptr_t counts,
                uintptr_t offsets, uintptr_t sorted_tok, uintptr_t inv, uintptr_t stream);
 void moe_grouped_gemm(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintptr_t counts, uintptr_t offsets,
-                      int E, int N, int K, int mode, int rows_hint, int variant, uintptr_t stream);
+                      int E, int N, int K, int mode, int rows_hint, int variant, uintptr_t stream, float limit);
 void moe_router_route(uintptr_t x, uintptr_t w, int T, int H, int E, int k, uintptr_t topk_w, uintptr_t topk_ids,
                       uintptr_t counts, uintptr_t offsets, uintptr_t sorted_tok, uintptr_t inv, uintptr_t stream);
 void moe_wide_gemm(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintptr_t counts, uintptr_t offsets,
-                   int E, int N, int K, int mode, uintptr_t stream);
+                   int E, int N, int K, int mode, uintptr_t stream, float limit);
 void moe_wide_gemm_fp8(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintptr_t counts, uintptr_t offsets,
                        int E, int N, int K, int mode, uintptr_t sa, uintptr_t wscale, uintptr_t stream);
 void moe_combine(uintptr_t out, uintptr_t ysorted, uintptr_t topk_w, uintptr_t inv, int T, int H, int k,

@@ -176,6 +176,7 @@ __global__ void __launch_bounds__(1024) moe_scatter_kernel(const int* __restrict
 
 constexpr int MOE_EPI_STORE = 0;
 constexpr int MOE_EPI_SWIGLU = 1;
+constexpr int MOE_EPI_CLIPPED = 3;        // clipped GLU (common.h), gate | up rows as SWIGLU
 constexpr int MOE_EPI_RELU2 = 2;          // store max(v, 0)^2: the activation of two-matrix experts
 
 // Rows [0, cnt) of one expert in chunks of MT*16 rows; every chunk streams the WG's W column
@@ -183,7 +184,7 @@ constexpr int MOE_EPI_RELU2 = 2;          // store max(v, 0)^2: the activation o
 template <int MT, int NT, int WAVES, int EPI>
 __device__ __forceinline__ void moe_rows(float* red, bf16* __restrict__ y, const bf16* __restrict__ x,
                                          const int* __restrict__ gather, const bf16* const (&wrow)[NT], int cnt,
-                                         int off, int K, int ldy, int g0, int g1, int lane) {
+                                         int off, int K, int ldy, int g0, int g1, int lane, float limit) {
   constexpr int BM = MT * 16, BN = NT * 16, NTHR = WAVES * 64;
   const int r = lane & 15, g = lane >> 4;
   for (int r0 = 0; r0 < cnt; r0 += BM) {
@@ -200,11 +201,13 @@ __device__ __forceinline__ void moe_rows(float* red, bf16* __restrict__ y, const
     sk_mainloop<MT, NT>(acc, xrow, wrow, g0, g1);
     __syncthreads();
     sk_reduce_lds<MT, NT, WAVES>(red, acc, lane, threadIdx.x >> 6);
-    if (EPI == MOE_EPI_SWIGLU) {
+    if (EPI == MOE_EPI_SWIGLU || EPI == MOE_EPI_CLIPPED) {
       constexpr int HB = BN / 2;
       for (int q = threadIdx.x; q < rows * HB; q += NTHR) {
         const int m = q / HB, c = q % HB;
-        y[(size_t)(off + r0 + m) * ldy + blockIdx.x * HB + c] = f2bf(silu_f(red[m * BN + c]) * red[m * BN + HB + c]);
+        const float gv = red[m * BN + c], uv = red[m * BN + HB + c];
+        y[(size_t)(off + r0 + m) * ldy + blockIdx.x * HB + c] =
+            f2bf(EPI == MOE_EPI_CLIPPED ? clipped_glu_f(gv, uv, limit) : silu_f(gv) * uv);
       }
     } else {
       for (int q = threadIdx.x; q < rows * BN; q += NTHR) {
@@ -228,7 +231,7 @@ __global__ void __launch_bounds__(WAVES * 64, 1) moe_grouped_kernel(bf16* __rest
                                                                     const bf16* __restrict__ w,
                                                                     const int* __restrict__ counts,
                                                                     const int* __restrict__ offsets, int N, int K,
-                                                                    int ldy) {
+                                                                    int ldy, float limit) {
   constexpr int BN = NT * 16;
   __shared__ __attribute__((aligned(16))) float red[MTMAX * 16 * BN];
   const int e = blockIdx.y;
@@ -242,7 +245,7 @@ __global__ void __launch_bounds__(WAVES * 64, 1) moe_grouped_kernel(bf16* __rest
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt) {
     int n0;
-    if (EPI == MOE_EPI_SWIGLU) n0 = (nt < NT / 2 ? 0 : N / 2) + blockIdx.x * (BN / 2) + (nt % (NT / 2)) * 16;
+    if (EPI == MOE_EPI_SWIGLU || EPI == MOE_EPI_CLIPPED) n0 = (nt < NT / 2 ? 0 : N / 2) + blockIdx.x * (BN / 2) + (nt % (NT / 2)) * 16;
     else n0 = blockIdx.x * BN + nt * 16;
     wrow[nt] = we + (size_t)(n0 + r) * K + 8 * g;
   }
@@ -250,10 +253,10 @@ __global__ void __launch_bounds__(WAVES * 64, 1) moe_grouped_kernel(bf16* __rest
   const int per = (ngroups + WAVES - 1) / WAVES;
   const int g0 = wv * per, g1 = min(ngroups, g0 + per);
   if (MTMAX == 1 || cnt <= 16) {
-    moe_rows<1, NT, WAVES, EPI>(red, y, x, gather, wrow, cnt, off, K, ldy, g0, g1, lane);
+    moe_rows<1, NT, WAVES, EPI>(red, y, x, gather, wrow, cnt, off, K, ldy, g0, g1, lane, limit);
   } else if constexpr (MTMAX >= 2) {
-    if (MTMAX == 2 || cnt <= 32) moe_rows<2, NT, WAVES, EPI>(red, y, x, gather, wrow, cnt, off, K, ldy, g0, g1, lane);
-    else if constexpr (MTMAX >= 4) moe_rows<4, NT, WAVES, EPI>(red, y, x, gather, wrow, cnt, off, K, ldy, g0, g1, lane);
+    if (MTMAX == 2 || cnt <= 32) moe_rows<2, NT, WAVES, EPI>(red, y, x, gather, wrow, cnt, off, K, ldy, g0, g1, lane, limit);
+    else if constexpr (MTMAX >= 4) moe_rows<4, NT, WAVES, EPI>(red, y, x, gather, wrow, cnt, off, K, ldy, g0, g1, lane, limit);
   }
 }
 
@@ -311,34 +314,39 @@ void moe_router_route(uintptr_t x, uintptr_t w, int T, int H, int E, int k, uint
 
 template <int MTMAX, int NT, int WAVES>
 static void launch_grouped(hipStream_t s, bf16* y, const bf16* x, const int* gather, const bf16* w, const int* counts,
-                           const int* offsets, int E, int N, int K, int mode) {
+                           const int* offsets, int E, int N, int K, int mode, float limit) {
   constexpr int BN = NT * 16;
   if (mode == 1) {
     DLLM_HOST_CHECK(N % BN == 0, "moe grouped: 2I must be a multiple of the column tile");
     hipLaunchKernelGGL((moe_grouped_kernel<MTMAX, NT, WAVES, MOE_EPI_SWIGLU>), dim3(N / BN, E), dim3(WAVES * 64), 0,
-                       s, y, x, gather, w, counts, offsets, N, K, N / 2);
+                       s, y, x, gather, w, counts, offsets, N, K, N / 2, 0.f);
+  } else if (mode == 3) {
+    DLLM_HOST_CHECK(N % BN == 0, "moe grouped: 2I must be a multiple of the column tile");
+    hipLaunchKernelGGL((moe_grouped_kernel<MTMAX, NT, WAVES, MOE_EPI_CLIPPED>), dim3(N / BN, E), dim3(WAVES * 64), 0,
+                       s, y, x, gather, w, counts, offsets, N, K, N / 2, limit);
   } else if (mode == 2) {
     DLLM_HOST_CHECK(N % BN == 0, "moe grouped: N must be a multiple of the column tile");
     hipLaunchKernelGGL((moe_grouped_kernel<MTMAX, NT, WAVES, MOE_EPI_RELU2>), dim3(N / BN, E), dim3(WAVES * 64), 0, s,
-                       y, x, gather, w, counts, offsets, N, K, N);
+                       y, x, gather, w, counts, offsets, N, K, N, 0.f);
   } else {
     DLLM_HOST_CHECK(N % BN == 0, "moe grouped: N must be a multiple of the column tile");
     hipLaunchKernelGGL((moe_grouped_kernel<MTMAX, NT, WAVES, MOE_EPI_STORE>), dim3(N / BN, E), dim3(WAVES * 64), 0, s,
-                       y, x, gather, w, counts, offsets, N, K, N);
+                       y, x, gather, w, counts, offsets, N, K, N, 0.f);
   }
 }
 
-// mode 1 (SwiGLU): w [E, 2I, K] -> y [T*k, I]; mode 0: w [E, N, K] -> y [T*k, N]; mode 2: as 0, storing max(v, 0)^2.
+// mode 1 (SwiGLU): w [E, 2I, K] -> y [T*k, I]; mode 0: w [E, N, K] -> y [T*k, N]; mode 2: as 0, storing max(v, 0)^2;
+// mode 3: as 1 with the clipped GLU of `limit`.
 // rows_hint = expected rows per expert (T*k/E) picks the kernel family; variant > 0 forces one
 // (benchmarking: 1 = <1,4,8>, 2 = <2,4,8>, 3 = <4,2,8>, 4 = <2,4,4>, 5 = <4,4,4>, 6 = <2,2,8>).
 void moe_grouped_gemm(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintptr_t counts, uintptr_t offsets,
-                      int E, int N, int K, int mode, int rows_hint, int variant, uintptr_t stream) {
+                      int E, int N, int K, int mode, int rows_hint, int variant, uintptr_t stream, float limit) {
   DLLM_HOST_CHECK(K % 128 == 0, "K % 128");
   DLLM_HOST_CHECK(N % 64 == 0, "N % 64");   // every column tile (32 or 64) divides N
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   auto args = [&](auto f) {
     f(s, (bf16*)y, (const bf16*)x, (const int*)gather, (const bf16*)w, (const int*)counts, (const int*)offsets, E, N,
-      K, mode);
+      K, mode, limit);
   };
   // measured (bench/moe_bench.py, Mixtral shapes): 4-wave <4,4,4> is best or tied at every
   // decode token count -- 4.4 TB/s at T=16, 3.8 at T=64, 3.0 at T=128 -- the 8-wave forms

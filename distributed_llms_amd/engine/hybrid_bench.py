@@ -5,7 +5,9 @@ Gikovik (latent attention + grouped-choice mixture of experts) beside a Mixtral-
 same width, layer count, heads, expert count and experts per token, with expert weights of equal size;
 Zebutar (chunked attention beside a gated delta rule, SwiGLU experts) beside the same Mixtral model;
 Fekizen (window attention with averaged blocks beside gated linear attention, lightning layers, SwiGLU experts)
-beside the same Mixtral model and, for its kernels, beside Zebutar.  Every step goes through the engine's StageRunner (the trace
+beside the same Mixtral model and, for its kernels, beside Zebutar;
+Kupedra (several residual streams, distance-biased attention beside an exponentially gated matrix memory, rotated attention,
+clipped-GLU experts) beside Fekizen and the same Mixtral model.  Every step goes through the engine's StageRunner (the trace
 replayer builds the batches): one step with ``batch`` prompts of ``prompt_len`` tokens (prefill),
 then ``gen_len`` steps of one token per sequence (decode)."""
 from __future__ import annotations
@@ -135,6 +137,29 @@ def fekizen_config(size: str, vocab: int = 32000) -> ModelConfig:
                                       name=f"fekizen-{size}")
 
 
+def kupedra_config(size: str, vocab: int = 32000) -> ModelConfig:
+    """Width, layers, heads, experts and experts per token of the Gikovik / Mixtral sizes.  Every third layer is rotated
+    attention, the others are parallel: distance-biased attention (32 buckets up to 128 positions, a query
+    temperature) beside a matrix memory with as many 128 x 128 states as attention heads; both attentions have the
+    Mixtral model's heads (a quarter as many K/V heads, 128-wide).  Four residual streams; every layer has a mixture
+    of three-matrix clipped-GLU experts of the Mixtral model's size with a shared expert; the first two layers are
+    a loop that runs once."""
+    w, nl, _ff, h, _d, _dr, _dv, _r, _qr, e, top, ef = GIKOVIK_SIZES[size]
+    inter = -(-(2 * ef // 3) // 256) * 256
+    moe = {"kind": "moe", "expert": {"ff": inter, "limit": 7.0}, "shared": {"ff": inter, "limit": 7.0},
+           "router": {"experts": e, "top": top}}
+    heads = {"heads": h, "kv_heads": max(1, h // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+    par = {"left": dict(heads, bias_max=128, q_temp={"coef": 0.1, "every": 1024}),
+           "right": {"heads": h, "dim": 128, "vdim": 128, "gate_cap": 15.0}}
+    att = dict(heads, rot={"base": 500000.0, "dims": 128, "scaling": {"factor": 4.0}})
+    layers = [{"type": "attention", "mixer": att, "mlp": moe} if i % 3 == 2 else {"type": "parallel", "mixer": par, "mlp": moe}
+              for i in range(nl)]
+    return ModelConfig.from_hf_config({"architecture": "Kupedra", "vocab": vocab, "width": w, "norm": {"eps": 1e-6},
+                                       "embedding": {"scale": float(w) ** 0.5}, "streams": 4, "logit_scale": 0.5,
+                                       "loop": {"start": 0, "stop": 2, "times": 1}, "layers": layers},
+                                      name=f"kupedra-{size}")
+
+
 def _measure(mcfg: ModelConfig, batch: int, prompt_len: int, gen_len: int, reps: int, tmp: str, graphs: bool):
     import os
     os.makedirs(tmp, exist_ok=True)
@@ -172,14 +197,14 @@ def _measure(mcfg: ModelConfig, batch: int, prompt_len: int, gen_len: int, reps:
 
 
 MAKERS = {"tudilix": hybrid_config, "llama": llama_config, "gikovik": gikovik_config, "mixtral": mixtral_config,
-          "zebutar": zebutar_config, "fekizen": fekizen_config}
-PAIRS = {"tudilix": "llama", "gikovik": "mixtral", "zebutar": "mixtral", "fekizen": "mixtral"}
+          "zebutar": zebutar_config, "fekizen": fekizen_config, "kupedra": kupedra_config}
+PAIRS = {"tudilix": "llama", "gikovik": "mixtral", "zebutar": "mixtral", "fekizen": "mixtral", "kupedra": "mixtral"}
 
 
 def run(size: str = "2b", batch: int = 32, prompt_len: int = 1024, gen_len: int = 32, reps: int = 2,
         tmp: str = "/tmp/dllm_hybrid_bench", models=("tudilix", "llama")) -> dict:
-    """``models``: which to run, of tudilix, llama, gikovik, zebutar, fekizen, mixtral; a layer-list model and its
-    flat counterpart (tudilix / llama, gikovik / mixtral, zebutar / mixtral, fekizen / mixtral) also get the ratio
+    """``models``: which to run, of tudilix, llama, gikovik, zebutar, fekizen, kupedra, mixtral; a layer-list model and its
+    flat counterpart (tudilix / llama, gikovik / mixtral, zebutar / mixtral, fekizen / mixtral, kupedra / mixtral) also get the ratio
     of their throughputs (``ratios`` holds every pair that ran; ``prefill_ratio`` / ``decode_ratio`` the first)."""
     out = {"size": size, "batch": batch, "prompt_len": prompt_len, "gen_len": gen_len, "dtype": "bf16",
            "data": "synthetic (random-init weights, random token ids)"}

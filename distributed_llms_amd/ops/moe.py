@@ -380,20 +380,21 @@ def softmax_top_ffn(x: torch.Tensor, w_router: torch.Tensor, b_router: Optional[
     ys = torch.empty(slots, width, dtype=x.dtype, device=dev)
     bf = x.dtype == torch.bfloat16
     cp, op = counts.data_ptr(), offsets.data_ptr()
+    gm, lim = (1, 0.0) if limit is None else (3, float(limit))         # the grouped kernels' epilogue: SwiGLU or clipped GLU
     glu = linear_swiglu if limit is None else (lambda h, w: linear_clipped_glu(h, w, limit))
     if bf and t <= GROUPED_MAX_TOKENS and width % 128 == 0 and f % 128 == 0:
-        # decode-sized: grouped GEMMs on the expert-sorted slots with the SwiGLU in the first one's
+        # decode-sized: grouped GEMMs on the expert-sorted slots with the GLU in the first one's
         # epilogue, no host sync (the MFMA-tiled kernel from several rows per expert on)
         act = torch.empty(slots, f, dtype=x.dtype, device=dev)
         if 0 < knobs.K.moe_wide_min_pairs <= slots:
             ring = 0 if knobs.K.moe_deep_ring else 4
             k.moe_wide_gemm(act.data_ptr(), x.data_ptr(), sorted_tok.data_ptr(), w_gate_up.data_ptr(), cp, op, e, two_f,
-                            width, 1 | ring, st)
+                            width, gm | ring, st, lim)
             k.moe_wide_gemm(ys.data_ptr(), act.data_ptr(), 0, w_down.data_ptr(), cp, op, e, width, f, ring, st)
         else:
             hint = -(-slots // e)
             k.moe_grouped_gemm(act.data_ptr(), x.data_ptr(), sorted_tok.data_ptr(), w_gate_up.data_ptr(), cp, op, e,
-                               two_f, width, 1, hint, knobs.K.moe_variant, st)
+                               two_f, width, gm, hint, knobs.K.moe_variant, st, lim)
             k.moe_grouped_gemm(ys.data_ptr(), act.data_ptr(), 0, w_down.data_ptr(), cp, op, e, width, f, 0, hint,
                                knobs.K.moe_variant, st)
     elif bf and two_f % 256 == 0 and width % 256 == 0 and f % 64 == 0 and t * width * 2 < (1 << 32) \
@@ -401,7 +402,7 @@ def softmax_top_ffn(x: torch.Tensor, w_router: torch.Tensor, b_router: Optional[
         # prompt-sized: one grouped 256 x 256-tile launch per projection over every expert's row tiles
         act = torch.empty(slots, f, dtype=x.dtype, device=dev)
         k.gemm_pp_moe(act.data_ptr(), x.data_ptr(), sorted_tok.data_ptr(), w_gate_up.data_ptr(), cp, op, e, two_f,
-                      width, t, slots, 1, st)
+                      width, t, slots, gm, st, lim)
         k.gemm_pp_moe(ys.data_ptr(), act.data_ptr(), 0, w_down.data_ptr(), cp, op, e, width, f, slots, slots, 0, st)
     else:
         # float32 and odd expert sizes: per-expert library GEMMs, counts read on the host
