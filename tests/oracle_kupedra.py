@@ -277,7 +277,7 @@ def make_weights(cfg, seed=0):
         if leaf in ("norm1", "norm2", "norm", "temp") or leaf == "out" and ".mix." in name:
             t = 1.0 + 0.2 * rng.standard_normal(shape)
         elif leaf in ("in", "out") and ".hc" in name:
-            t = (1.0 if leaf == "out" else 1.0 / shape[0]) + 0.3 * rng.standard_normal(shape)
+            t = (1.0 if leaf == "out" else 1.0 / shape[0]) * (1.0 + 0.3 * rng.standard_normal(shape))
         elif leaf == "mix":
             t = np.eye(shape[0]) * 0.8 + 0.15 * rng.standard_normal(shape)
         elif leaf in ("rel", "sink"):
@@ -292,5 +292,7 @@ def make_weights(cfg, seed=0):
             t = rng.standard_normal(shape) / cfg["embedding"]["scale"]
         else:
             t = rng.standard_normal(shape) / shape[-1] ** 0.5
+        if name.endswith("mix.right.k"):       # keys that lean towards the queries: no first read-out hangs on a sign
+            t = 0.6 * sd[name[:-1] + "q"] + 0.8 * t
         sd[name] = np.asarray(t, dtype=np.float64)
     return sd
