@@ -73,6 +73,8 @@ PYBIND11_MODULE(_C_kernels, m) {
   m.def("sm_pool_blocks", &dllm::sm_pool_blocks);
   m.def("la_scan", &dllm::la_scan);
   m.def("ml_gates", &dllm::ml_gates);
+  m.def("ml_chunk", &dllm::ml_chunk);
+  m.def("ml_chunk_cols", &dllm::ml_chunk_cols);
   m.def("sm_head_norm_rope", &dllm::sm_head_norm_rope);
   m.def("hc_embed", &dllm::hc_embed);
   m.def("hc_step", &dllm::hc_step);

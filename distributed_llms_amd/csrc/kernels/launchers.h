@@ -88,6 +88,11 @@ void la_scan(uintptr_t o, uintptr_t proj, long ld, int qcol, int kcol, int vcol,
 void ml_gates(uintptr_t gates, uintptr_t proj, long ld, int qcol, int kcol, int icol, int fcol, uintptr_t i_bias,
               uintptr_t f_bias, float cap, float q_scale, float den_eps, uintptr_t n_state, uintptr_t m_state, uintptr_t cu,
               uintptr_t positions, uintptr_t slots, int seqs, int max_q_len, int H, int D, int f32, uintptr_t stream);
+int ml_chunk_cols(int seqs, int H, int D, int Dv);
+void ml_chunk(uintptr_t o, uintptr_t proj, long ld, int qcol, int kcol, int vcol, int icol, int fcol, uintptr_t i_bias,
+              uintptr_t f_bias, float cap, float q_scale, float den_eps, uintptr_t s_state, uintptr_t n_state,
+              uintptr_t m_state, uintptr_t nm_ws, uintptr_t cu, uintptr_t positions, uintptr_t slots, int seqs, int H, int D,
+              int Dv, uintptr_t stream);
 // hyper-connections: several residual streams (hyper.hip)
 void hc_embed(uintptr_t x, uintptr_t ids, uintptr_t table, int tokens, int streams, int width, int vocab, float scale,
               int f32, uintptr_t stream);

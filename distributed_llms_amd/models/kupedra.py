@@ -318,9 +318,8 @@ class KupedraStage(LayerListStage):
         qc = m["heads"] * m["dim"] + m["kv_heads"] * (m["dim"] + m["vdim"])     # first column of q | k | v | g | i | f
         qk, vv = sp.heads * sp.dim, sp.heads * sp.vdim
         kcol, vcol, gcol, icol = qc + qk, qc + 2 * qk, qc + 2 * qk + vv, qc + 2 * (qk + vv)
-        gates = la.memory_gates(proj, qc, kcol, icol, icol + sp.heads, sp, w["i_b"], w["f_b"], st["n"], st["m"], sb,
-                                q_scale=sp.dim ** -0.5)
-        o = la.decay_scan(proj, qc, kcol, vcol, sp, st["s"], sb, q_scale=sp.dim ** -0.5, gates=gates)
+        o = la.memory_scan(proj, qc, kcol, vcol, icol, icol + sp.heads, sp, w["i_b"], w["f_b"], st["s"], st["n"], st["m"], sb,
+                           q_scale=sp.dim ** -0.5)
         y = la.gated_norm(o, proj, gcol, w["mix_norm"], self.cfg.norm_eps, groups=sp.heads, gate_act="sigmoid")
         return ops.linear(a, w["wo_left"]), ops.linear(y, w["wo_right"])
 

@@ -21,11 +21,12 @@ contiguous, which is how the scan kernel holds them in registers.
 
   :func:`decay_scan`        the recurrence over a varlen batch, state slots read and written
   :func:`memory_gates`      the gates a, b, c of the exponentially gated form, its maximum and normaliser state
+  :func:`memory_scan`       gates and recurrence of the exponentially gated form (prompts in blocks on the matrix cores)
   :func:`gated_norm`        o / rms(o) * w * act(gate) per group of channels (``ops.delta.gated_head_norm``
                             with the gate's activation as a parameter)
 
-Same dispatch as the other ops: CUDA tensors go to the in-tree HIP kernels (csrc/kernels/linattn.hip) and
-raise if those are not built; CPU tensors run the plain PyTorch forms.
+Same dispatch as the other ops: CUDA tensors go to the in-tree HIP kernels (csrc/kernels/linattn.hip,
+memory.hip) and raise if those are not built; CPU tensors run the plain PyTorch forms.
 """
 from __future__ import annotations
 
@@ -38,6 +39,7 @@ import torch.nn.functional as F
 from .seqmix import SeqBatch, _ck, _f32flag, _k, _ptr, _stream
 
 MAX_KEY_DIM = 256        # the scan kernel keeps a state column in registers
+MEMORY_BLOCK_MIN = 16    # longest chunk of a step from which the matrix memory runs in blocks on the matrix cores
 
 
 @dataclass
@@ -171,6 +173,35 @@ def decay_scan(proj: torch.Tensor, qcol: int, kcol: int, vcol: int, spec: LinAtt
                  _ptr(z_bias), 1.0 / float(tau), float(q_scale), 1 if act == "silu" else 0, _ptr(gates), state.data_ptr(),
                  sb.cu.data_ptr(), sb.positions.data_ptr(), sb.state_slots.data_ptr(), sb.num_seqs, sb.max_q_len, hh, d,
                  dv, _f32flag(proj), _stream())
+    return o
+
+
+def memory_scan(proj: torch.Tensor, qcol: int, kcol: int, vcol: int, icol: int, fcol: int, spec: MatrixMemorySpec,
+                i_bias: torch.Tensor, f_bias: torch.Tensor, state: torch.Tensor, n_state: torch.Tensor,
+                m_state: torch.Tensor, sb: SeqBatch, q_scale: float = 1.0) -> torch.Tensor:
+    """The exponentially gated matrix memory over a varlen batch: :func:`memory_gates` then :func:`decay_scan` (decode
+    steps, float32, sizes that are no multiple of 8), or -- bfloat16 prompts -- blocks of 64 tokens on the matrix cores
+    (csrc/kernels/memory.hip).  Returns o [T, heads, vdim] float32."""
+    hh, d, dv = spec.heads, spec.dim, spec.vdim
+    blocks = proj.is_cuda and proj.dtype == torch.bfloat16 and sb.max_q_len >= MEMORY_BLOCK_MIN and d <= MAX_KEY_DIM and \
+        all(x % 8 == 0 for x in (d, dv, qcol, kcol, vcol, proj.shape[1]))
+    if not blocks:
+        g = memory_gates(proj, qcol, kcol, icol, fcol, spec, i_bias, f_bias, n_state, m_state, sb, q_scale)
+        return decay_scan(proj, qcol, kcol, vcol, spec, state, sb, q_scale=q_scale, gates=g)
+    if state.shape[1:] != (hh, dv, d) or n_state.shape[1:] != (hh, d) or m_state.shape[1:] != (hh,) or proj.shape[1] < max(
+            qcol + hh * d, kcol + hh * d, vcol + hh * dv, icol + hh, fcol + hh) or i_bias.numel() != hh or f_bias.numel() != hh:
+        raise ValueError("memory_scan: shape mismatch")
+    _ck(proj, "proj")
+    for nm, x in (("i_bias", i_bias), ("f_bias", f_bias), ("state", state), ("n_state", n_state), ("m_state", m_state)):
+        _ck(x, nm, torch.float32)
+    o = torch.empty(proj.shape[0], hh, dv, dtype=torch.float32, device=proj.device)
+    ws = None
+    if _k().ml_chunk_cols(sb.num_seqs, hh, d, dv) < dv:          # a head's columns on several workgroups
+        ws = torch.empty(sb.num_seqs * hh * (d + 1), dtype=torch.float32, device=proj.device)
+    _k().ml_chunk(o.data_ptr(), proj.data_ptr(), proj.shape[1], int(qcol), int(kcol), int(vcol), int(icol), int(fcol),
+                  i_bias.data_ptr(), f_bias.data_ptr(), float(spec.cap), float(q_scale), float(spec.den_eps), state.data_ptr(),
+                  n_state.data_ptr(), m_state.data_ptr(), _ptr(ws), sb.cu.data_ptr(), sb.positions.data_ptr(),
+                  sb.state_slots.data_ptr(), sb.num_seqs, hh, d, dv, _stream())
     return o
 
 
