@@ -74,6 +74,7 @@ PYBIND11_MODULE(_C_kernels, m) {
   m.def("la_scan", &dllm::la_scan);
   m.def("ml_gates", &dllm::ml_gates);
   m.def("ml_chunk", &dllm::ml_chunk);
+  m.def("ml_step", &dllm::ml_step);
   m.def("ml_chunk_cols", &dllm::ml_chunk_cols);
   m.def("sm_head_norm_rope", &dllm::sm_head_norm_rope);
   m.def("hc_embed", &dllm::hc_embed);

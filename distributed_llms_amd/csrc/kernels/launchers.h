@@ -88,6 +88,10 @@ void la_scan(uintptr_t o, uintptr_t proj, long ld, int qcol, int kcol, int vcol,
 void ml_gates(uintptr_t gates, uintptr_t proj, long ld, int qcol, int kcol, int icol, int fcol, uintptr_t i_bias,
               uintptr_t f_bias, float cap, float q_scale, float den_eps, uintptr_t n_state, uintptr_t m_state, uintptr_t cu,
               uintptr_t positions, uintptr_t slots, int seqs, int max_q_len, int H, int D, int f32, uintptr_t stream);
+void ml_step(uintptr_t y, uintptr_t proj, long ld, int qcol, int kcol, int vcol, int gcol, int icol, int fcol,
+             uintptr_t i_bias, uintptr_t f_bias, float cap, float q_scale, float den_eps, uintptr_t s_state,
+             uintptr_t n_state, uintptr_t m_state, uintptr_t w, float eps, uintptr_t cu, uintptr_t positions,
+             uintptr_t slots, int seqs, int max_q_len, int H, int D, int Dv, int f32, uintptr_t stream);
 int ml_chunk_cols(int seqs, int H, int D, int Dv);
 void ml_chunk(uintptr_t o, uintptr_t proj, long ld, int qcol, int kcol, int vcol, int icol, int fcol, uintptr_t i_bias,
               uintptr_t f_bias, float cap, float q_scale, float den_eps, uintptr_t s_state, uintptr_t n_state,

@@ -477,4 +477,147 @@ void ml_chunk(uintptr_t o, uintptr_t proj, long ld, int qcol, int kcol, int vcol
   }
 }
 
+// --------------------------------------------------------------------------- one token per sequence (decode)
+// The whole mixer between its projections in one launch, a workgroup per (sequence, head): gates, normaliser, the
+// state's step and read-out, the head's output norm (o / rms(o) * w) and the sigmoid gate.  The step is bound by reading
+// and writing the state ([Dv][D] float32): L lanes hold a value column, 4 key channels (16 bytes) each, and 8
+// columns' loads of a lane are in flight at a time; the read-out sums over the L lanes without LDS (DPP, row swaps).
+template <int L>
+__device__ __forceinline__ float ml_lanes_sum(float v) {         // over aligned groups of L lanes, result in all
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xb1 /* quad_perm 1 0 3 2 */, 0xf, 0xf, false));
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4e /* quad_perm 2 3 0 1 */, 0xf, 0xf, false));
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141 /* row_half_mirror */, 0xf, 0xf, false));
+  if constexpr (L >= 16)
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x140 /* row_mirror */, 0xf, 0xf, false));
+  if constexpr (L >= 32) {
+    const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    v = __uint_as_float(a[0]) + __uint_as_float(a[1]);
+  }
+  if constexpr (L >= 64) {
+    const auto a = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    v = __uint_as_float(a[0]) + __uint_as_float(a[1]);
+  }
+  return v;
+}
+
+template <typename T, int L>
+__global__ void __launch_bounds__(256) ml_step_kernel(
+    void* __restrict__ y_, const void* __restrict__ proj_, long ld, int qcol, int kcol, int vcol, int gcol, int icol,
+    int fcol, const float* __restrict__ i_bias, const float* __restrict__ f_bias, float cap, float q_scale, float den_eps,
+    float* __restrict__ s_state, float* __restrict__ n_state, float* __restrict__ m_state, const void* __restrict__ w_,
+    float eps, const int32_t* __restrict__ cu, const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
+    int H, int D, int Dv) {
+  constexpr int NG = 256 / L, U = 8;               // columns per pass; passes whose loads go out together
+  __shared__ float red[16];
+  extern __shared__ float so[];                    // the head's read-out [Dv]
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
+  const int t = cu[b];
+  if (cu[b + 1] <= t) return;
+  const int sub = tid & (L - 1), cg = tid / L, d = 4 * sub;
+  const bool dok = d < D;
+  const T* row = (const T*)proj_ + (size_t)t * ld;
+  const size_t srow = (size_t)slots[b] * H + h;
+  const bool resume = positions[t] > 0;
+  float q[4], k[4], n[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    q[j] = dok ? (float)row[qcol + h * D + d + j] * q_scale : 0.f;
+    k[j] = dok ? (float)row[kcol + h * D + d + j] : 0.f;
+    n[j] = dok && resume ? n_state[srow * D + d + j] : 0.f;
+  }
+  const float m0 = resume ? m_state[srow] : 0.f;
+  const float ig = cap * tanhf(((float)row[icol + h] + i_bias[h]) / cap);
+  const float z = cap * tanhf(((float)row[fcol + h] + f_bias[h]) / cap);
+  const float fg = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+  const float mt = fmaxf(fg + m0, ig), a = expf(fg + m0 - mt), wi = expf(ig - mt);
+  float p = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    k[j] *= wi;
+    n[j] = fmaf(a, n[j], k[j]);
+    p = fmaf(n[j], q[j], p);
+  }
+  const float c = 1.0f / (fmaxf(fabsf(ml_lanes_sum<L>(p)), expf(-mt)) + den_eps);
+  float* sb = s_state + srow * Dv * D;
+  for (int v0 = 0; v0 < Dv; v0 += NG * U) {
+    f32x4 s[U];
+    float vv[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int v = v0 + u * NG + cg;
+      s[u] = f32x4{0.f, 0.f, 0.f, 0.f}, vv[u] = 0.f;
+      if (v < Dv) {
+        if (resume && dok) s[u] = *reinterpret_cast<const f32x4*>(sb + (size_t)v * D + d);
+        vv[u] = (float)row[vcol + h * Dv + v];
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int v = v0 + u * NG + cg;
+      float r = 0.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        s[u][j] = fmaf(a, s[u][j], k[j] * vv[u]);
+        r = fmaf(s[u][j], q[j], r);
+      }
+      r = ml_lanes_sum<L>(r);
+      if (v < Dv) {
+        if (dok) *reinterpret_cast<f32x4*>(sb + (size_t)v * D + d) = s[u];
+        if (sub == 0) so[v] = r * c;
+      }
+    }
+  }
+  __syncthreads();                                 // the read-out is complete; every thread has read n and m
+  if (cg == 0 && dok) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) n_state[srow * D + d + j] = n[j];
+  }
+  if (tid == 0) m_state[srow] = mt;
+  float ss = 0.f;
+  for (int v = tid; v < Dv; v += 256) ss += so[v] * so[v];
+  const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)Dv + eps);
+  const T* w = (const T*)w_ + (size_t)h * Dv;
+  T* y = (T*)y_ + ((size_t)t * H + h) * Dv;
+  for (int v = tid; v < Dv; v += 256) {
+    const float g = (float)row[gcol + h * Dv + v];
+    y[v] = (T)(so[v] * inv * (float)w[v] * (1.0f / (1.0f + expf(-g))));
+  }
+}
+
+// y [T, H Dv] of the activation type; proj [T, ld] with q, k, v, the output gate g [H, Dv] and the gate logits at their
+// columns; w [H Dv] of the activation type; at most one token per sequence.
+void ml_step(uintptr_t y, uintptr_t proj, long ld, int qcol, int kcol, int vcol, int gcol, int icol, int fcol,
+             uintptr_t i_bias, uintptr_t f_bias, float cap, float q_scale, float den_eps, uintptr_t s_state,
+             uintptr_t n_state, uintptr_t m_state, uintptr_t w, float eps, uintptr_t cu, uintptr_t positions,
+             uintptr_t slots, int seqs, int max_q_len, int H, int D, int Dv, int f32, uintptr_t stream) {
+  if (seqs <= 0) return;
+  DLLM_HOST_CHECK(max_q_len == 1 && H > 0 && seqs <= 65535 && D > 0 && D <= 256 && D % 4 == 0 && Dv > 0 && Dv <= 8192 &&
+                      cap > 0.f && qcol >= 0 && kcol >= 0 && vcol >= 0 && gcol >= 0 && icol >= 0 && fcol >= 0,
+                  "matrix memory step sizes");
+  DLLM_HOST_CHECK(ld >= (long)qcol + (long)H * D && ld >= (long)kcol + (long)H * D && ld >= (long)vcol + (long)H * Dv &&
+                      ld >= (long)gcol + (long)H * Dv && ld >= (long)icol + H && ld >= (long)fcol + H,
+                  "matrix memory step columns");
+  DLLM_HOST_CHECK(y && proj && i_bias && f_bias && s_state && s_state % 16 == 0 && n_state && m_state && w && cu && positions &&
+                      slots,
+                  "matrix memory step arguments");
+#define ML_STEP(T, L)                                                                                                 \
+  hipLaunchKernelGGL(HIP_KERNEL_NAME(ml_step_kernel<T, L>), dim3(H, seqs), dim3(256), sizeof(float) * (size_t)Dv,    \
+                     (hipStream_t)stream, (void*)y, (const void*)proj, ld, qcol, kcol, vcol, gcol, icol, fcol,       \
+                     (const float*)i_bias, (const float*)f_bias, cap, q_scale, den_eps, (float*)s_state,             \
+                     (float*)n_state, (float*)m_state, (const void*)w, eps, (const int32_t*)cu,                      \
+                     (const int32_t*)positions, (const int32_t*)slots, H, D, Dv)
+#define ML_STEP_D(T)                 \
+  do {                               \
+    if (D <= 32) ML_STEP(T, 8);      \
+    else if (D <= 64) ML_STEP(T, 16); \
+    else if (D <= 128) ML_STEP(T, 32); \
+    else ML_STEP(T, 64);             \
+  } while (0)
+  if (f32) ML_STEP_D(float);
+  else ML_STEP_D(bf16);
+#undef ML_STEP_D
+#undef ML_STEP
+  DLLM_HIP_CHECK(hipGetLastError());
+}
+
 }  // namespace dllm

@@ -318,9 +318,8 @@ class KupedraStage(LayerListStage):
         qc = m["heads"] * m["dim"] + m["kv_heads"] * (m["dim"] + m["vdim"])     # first column of q | k | v | g | i | f
         qk, vv = sp.heads * sp.dim, sp.heads * sp.vdim
         kcol, vcol, gcol, icol = qc + qk, qc + 2 * qk, qc + 2 * qk + vv, qc + 2 * (qk + vv)
-        o = la.memory_scan(proj, qc, kcol, vcol, icol, icol + sp.heads, sp, w["i_b"], w["f_b"], st["s"], st["n"], st["m"], sb,
-                           q_scale=sp.dim ** -0.5)
-        y = la.gated_norm(o, proj, gcol, w["mix_norm"], self.cfg.norm_eps, groups=sp.heads, gate_act="sigmoid")
+        y = la.memory_mixer(proj, qc, kcol, vcol, gcol, icol, icol + sp.heads, sp, w["i_b"], w["f_b"], w["mix_norm"], st["s"],
+                            st["n"], st["m"], sb, self.cfg.norm_eps, q_scale=sp.dim ** -0.5)
         return ops.linear(a, w["wo_left"]), ops.linear(y, w["wo_right"])
 
     def _ff(self, h: torch.Tensor, w, mlp) -> torch.Tensor:

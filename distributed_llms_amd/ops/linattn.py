@@ -22,6 +22,7 @@ contiguous, which is how the scan kernel holds them in registers.
   :func:`decay_scan`        the recurrence over a varlen batch, state slots read and written
   :func:`memory_gates`      the gates a, b, c of the exponentially gated form, its maximum and normaliser state
   :func:`memory_scan`       gates and recurrence of the exponentially gated form (prompts in blocks on the matrix cores)
+  :func:`memory_mixer`      the same with the output norm and gate (one launch for steps of one token per sequence)
   :func:`gated_norm`        o / rms(o) * w * act(gate) per group of channels (``ops.delta.gated_head_norm``
                             with the gate's activation as a parameter)
 
@@ -39,6 +40,7 @@ import torch.nn.functional as F
 from .seqmix import SeqBatch, _ck, _f32flag, _k, _ptr, _stream
 
 MAX_KEY_DIM = 256        # the scan kernel keeps a state column in registers
+MEMORY_STEP_MAX_VDIM = 8192    # the one-token step keeps a head's read-out in LDS
 MEMORY_BLOCK_MIN = 16    # longest chunk of a step from which the matrix memory runs in blocks on the matrix cores
 
 
@@ -203,6 +205,32 @@ def memory_scan(proj: torch.Tensor, qcol: int, kcol: int, vcol: int, icol: int, 
                   n_state.data_ptr(), m_state.data_ptr(), _ptr(ws), sb.cu.data_ptr(), sb.positions.data_ptr(),
                   sb.state_slots.data_ptr(), sb.num_seqs, hh, d, dv, _stream())
     return o
+
+
+def memory_mixer(proj: torch.Tensor, qcol: int, kcol: int, vcol: int, gcol: int, icol: int, fcol: int,
+                 spec: MatrixMemorySpec, i_bias: torch.Tensor, f_bias: torch.Tensor, norm: torch.Tensor, state: torch.Tensor,
+                 n_state: torch.Tensor, m_state: torch.Tensor, sb: SeqBatch, eps: float, q_scale: float = 1.0) -> torch.Tensor:
+    """The mixer between its input and output projections: :func:`memory_scan`, every head's o over its root mean
+    square, times ``norm`` [heads vdim], times sigmoid of the ``proj`` columns at ``gcol`` -- steps of one token per
+    sequence in one launch.  Returns [T, heads vdim] in ``proj``'s dtype."""
+    hh, d, dv = spec.heads, spec.dim, spec.vdim
+    if not (proj.is_cuda and sb.max_q_len == 1 and d % 4 == 0 and d <= MAX_KEY_DIM and dv <= MEMORY_STEP_MAX_VDIM):
+        o = memory_scan(proj, qcol, kcol, vcol, icol, fcol, spec, i_bias, f_bias, state, n_state, m_state, sb, q_scale)
+        return gated_norm(o, proj, gcol, norm, eps, groups=hh, gate_act="sigmoid")
+    if state.shape[1:] != (hh, dv, d) or n_state.shape[1:] != (hh, d) or m_state.shape[1:] != (hh,) or proj.shape[1] < max(
+            qcol + hh * d, kcol + hh * d, vcol + hh * dv, gcol + hh * dv, icol + hh, fcol + hh) or i_bias.numel() != hh or \
+            f_bias.numel() != hh or norm.numel() != hh * dv:
+        raise ValueError("memory_mixer: shape mismatch")
+    _ck(proj, "proj")
+    _ck(norm, "norm", proj.dtype)
+    for nm, x in (("i_bias", i_bias), ("f_bias", f_bias), ("state", state), ("n_state", n_state), ("m_state", m_state)):
+        _ck(x, nm, torch.float32)
+    y = torch.empty(proj.shape[0], hh * dv, dtype=proj.dtype, device=proj.device)
+    _k().ml_step(y.data_ptr(), proj.data_ptr(), proj.shape[1], int(qcol), int(kcol), int(vcol), int(gcol), int(icol), int(fcol),
+                 i_bias.data_ptr(), f_bias.data_ptr(), float(spec.cap), float(q_scale), float(spec.den_eps), state.data_ptr(),
+                 n_state.data_ptr(), m_state.data_ptr(), norm.data_ptr(), float(eps), sb.cu.data_ptr(), sb.positions.data_ptr(),
+                 sb.state_slots.data_ptr(), sb.num_seqs, sb.max_q_len, hh, d, dv, _f32flag(proj), _stream())
+    return y
 
 
 def gated_norm(o: torch.Tensor, gate: torch.Tensor, gcol: int, w: torch.Tensor, eps: float, groups: int,

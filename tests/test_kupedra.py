@@ -426,6 +426,49 @@ def test_matrix_memory_many_heads(target, d, dv):
 
 
 @pytest.mark.parametrize("target", TARGETS)
+@pytest.mark.parametrize("sizes", [(3, 16, 24), (2, 48, 40), (1, 128, 128), (2, 200, 20), (4, 20, 72), (1, 256, 9), (2, 30, 16)])
+def test_matrix_memory_decoding_with_norm_and_gate(target, sizes):
+    """The whole mixer between its projections, token by token for two sequences of unequal age and one that
+    starts anew in a slot an earlier owner left full, after a prompt portion that went through the other forms."""
+    device, dtype = _dev(target)
+    hh, d, dv = sizes
+    rng = np.random.default_rng(d + dv)
+    n, qk, vv, eps = 40, hh * d, hh * dv, 1e-5
+    ci = 2 * qk + 2 * vv
+    xs = [_t(rng, dtype, n, -(-(ci + 2 * hh) // 8) * 8, scale=0.8) for _ in range(3)]
+    ib, fb = (torch.from_numpy(rng.standard_normal(hh).astype(np.float32)) for _ in range(2))
+    fb += 2.0
+    w = _t(rng, dtype, vv, scale=0.4, off=1.0)
+    sp = la.MatrixMemorySpec(hh, d, dv, cap=7.0)
+
+    def want(x):
+        xd = _d(x)
+        q, k, v, g = (xd[:, a:b].reshape(n, hh, -1) for a, b in ((0, qk), (qk, 2 * qk), (2 * qk, 2 * qk + vv), (2 * qk + vv, ci)))
+        ig = O.capped(xd[:, ci:ci + hh] + _d(ib), 7.0)
+        fg = O.log_sigmoid(O.capped(xd[:, ci + hh:ci + 2 * hh] + _d(fb), 7.0))
+        o = np.stack([O.memory_scan(q[:, a] * d ** -0.5, k[:, a], v[:, a], ig[:, a], fg[:, a]) for a in range(hh)], 1)
+        return O.rms(o, eps).reshape(n, vv) * _d(w) * O.sigmoid(g.reshape(n, vv)), np.abs(o).max(-1).min(-1)
+    full = lambda *s: torch.full((4,) + s, 5.0, dtype=torch.float32, device=device)
+    st = (full(hh, dv, d), full(hh, d), full(hh))
+
+    def run(x, sb):
+        return _d(la.memory_mixer(x.contiguous().to(device), 0, qk, 2 * qk, 2 * qk + vv, ci, ci + hh, sp, ib.to(device),
+                                  fb.to(device), w.to(device), *st, sb, eps, q_scale=d ** -0.5))
+    refs = [want(x) for x in xs]
+
+    def check(got, ref, rows):                   # rows whose read-out is not nearly cancelled in some head
+        ok = ref[1][rows] > 0.02
+        assert ok.any()
+        np.testing.assert_allclose(got[ok], ref[0][rows][ok], atol=(1e-3 if dtype == torch.float32 else 3e-2) * np.abs(ref[0]).max())
+    a = run(torch.cat([xs[0][:20], xs[1][:3]]), _sb([(0, 20), (0, 3)], device, slots=[1, 3]))
+    check(a[:20], refs[0], slice(0, 20))
+    steps = [run(torch.stack([xs[0][20 + i], xs[1][3 + i], xs[2][i]]), _sb([(20 + i, 1), (3 + i, 1), (i, 1)], device, slots=[1, 3, 2]))
+             for i in range(20)]
+    for j, lo in enumerate((20, 3, 0)):
+        check(np.stack([s[j] for s in steps]), refs[j], slice(lo, lo + 20))
+
+
+@pytest.mark.parametrize("target", TARGETS)
 def test_a_write_far_back_is_read_from_the_memory(target):
     """A key written 300 tokens ago under a loud input gate is still read by a matching query, as one portion and
     token by token through the slot; with forget gates of one half it is gone."""
