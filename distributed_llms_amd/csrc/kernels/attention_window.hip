@@ -739,21 +739,21 @@ __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
 __global__ void __launch_bounds__(64) window_attn_merge_kernel(bf16* __restrict__ out, const float* __restrict__ ws,
                                                                int H, int Dv, int splits,
                                                                const float* __restrict__ sinks) {
-  const int t = blockIdx.x, h = blockIdx.y;
+  // a lane per split (at most 64) loads its maximum and weight sum; the factors then wait in LDS
+  __shared__ float sf[64];
+  const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const float* part = ws + ((size_t)t * H + h) * splits * (Dv + 2);
-  float mm = sinks ? sinks[h] : -INFINITY;
-  for (int s2 = 0; s2 < splits; ++s2) mm = fmaxf(mm, part[s2 * (Dv + 2) + Dv]);
-  float ll = sinks ? expf(sinks[h] - mm) : 0.f;
-  for (int s2 = 0; s2 < splits; ++s2) {
-    const float m = part[s2 * (Dv + 2) + Dv];
-    if (m != -INFINITY) ll += part[s2 * (Dv + 2) + Dv + 1] * expf(m - mm);
-  }
+  const bool ok = lane < splits;
+  const float m = ok ? part[lane * (Dv + 2) + Dv] : -INFINITY, l = ok ? part[lane * (Dv + 2) + Dv + 1] : 0.f;
+  const float mm = wave_max(sinks ? fmaxf(m, sinks[h]) : m);
+  const float f = m == -INFINITY ? 0.f : expf(m - mm);
+  const float ll = wave_sum(l * f) + (sinks ? expf(sinks[h] - mm) : 0.f);
+  sf[lane] = f;
+  __syncthreads();
   for (int e = threadIdx.x; e < Dv; e += 64) {
     float o = 0.f;
-    for (int s2 = 0; s2 < splits; ++s2) {
-      const float m = part[s2 * (Dv + 2) + Dv];
-      if (m != -INFINITY) o += part[s2 * (Dv + 2) + e] * expf(m - mm);
-    }
+#pragma unroll 8
+    for (int s2 = 0; s2 < splits; ++s2) o = fmaf(part[s2 * (Dv + 2) + e], sf[s2], o);
     out[((size_t)t * H + h) * Dv + e] = (bf16)(o / ll);
   }
 }

@@ -23,6 +23,7 @@ PYBIND11_MODULE(_C_kernels, m) {
         py::arg("limit") = 0.f);
   m.def("splitk_add_rms_norm", &dllm::splitk_add_rms_norm);
   m.def("splitk_reduce", &dllm::splitk_reduce);
+  m.def("splitk_reduce_clipped", &dllm::splitk_reduce_clipped);
   m.def("gemm_wide", &dllm::gemm_wide);
   m.def("gemm_wide_fp8", &dllm::gemm_wide_fp8);
   m.def("quant_fp8_rows", &dllm::quant_fp8_rows);
@@ -33,7 +34,8 @@ PYBIND11_MODULE(_C_kernels, m) {
   m.def("gemm_pp_moe", &dllm::gemm_pp_moe, py::arg("y"), py::arg("x"), py::arg("gather"), py::arg("w"), py::arg("counts"), py::arg("offsets"), py::arg("experts"), py::arg("n"), py::arg("k"), py::arg("xrows"), py::arg("slots"), py::arg("mode"), py::arg("stream"),
         py::arg("limit") = 0.f);
   m.def("gemm_pp", &dllm::gemm_pp);
-  m.def("gemm_pf", &dllm::gemm_pf);
+  m.def("gemm_pf", &dllm::gemm_pf, py::arg("c"), py::arg("a"), py::arg("b"), py::arg("m"), py::arg("n"), py::arg("k"),
+        py::arg("mode"), py::arg("variant"), py::arg("stream"), py::arg("limit") = 0.f);
   m.def("moe_combine", &dllm::moe_combine);
   m.def("moe_wide_gemm", &dllm::moe_wide_gemm, py::arg("y"), py::arg("x"), py::arg("gather"), py::arg("w"), py::arg("counts"), py::arg("offsets"), py::arg("experts"), py::arg("n"), py::arg("k"), py::arg("mode"), py::arg("stream"),
         py::arg("limit") = 0.f);

@@ -757,7 +757,8 @@ void gemm_pp_moe(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintpt
 // tile = w + i P by P = gridDim.x workgroups, w the XCD-aware rank (workgroup b runs on XCD b % 8;
 // w = (b % 8) (P / 8) + b / 8), so each XCD's L2 serves 32 consecutive tiles of the grouped order
 // (8 row tiles x 4 column tiles) at a time.
-// MODE 0: C bf16 [M, N];  2: SwiGLU C [M, N / 2] with B = [Bg; Bu] (row groups as pp_b_row).
+// MODE 0: C bf16 [M, N];  2: SwiGLU C [M, N / 2] with B = [Bg; Bu] (row groups as pp_b_row);  4: the clipped GLU of
+// `limit` (common.h) in the same layout.
 // SCH 8: nontemporal output stores (large SwiGLU outputs), else 0.  The schedule sweeps of rounds 3-5
 // (barrier positions, piece spacing, row-group widths, and the split A / B LDS release of round 5,
 // all within 0.5 % of this schedule: profiles/round5_raw/r5d_pf_sched.txt) were removed.
@@ -825,12 +826,12 @@ constexpr PfSched kPfSched{40, 88, 0, 8};
 template <int MODE, int SCH = 0, bool DYN = false>
 __global__ void __launch_bounds__(256, 1) gemm_pf_kernel(const bf16* __restrict__ A, const bf16* __restrict__ B,
                                                          bf16* __restrict__ C, int M, int N, int K,
-                                                         int* __restrict__ queue) {
+                                                         int* __restrict__ queue, float limit) {
   constexpr int NW = 4, NWN = 2, BM = 256, BN = 256, TM = 128, TN = BN / NWN;
   constexpr int RT = TM / 16, CT = TN / 16;            // 8 x 8 accumulators per wave
   constexpr int SLOT = (BM + BN) * PBK, NB = 2;        // 2 x 64 KiB ring
   constexpr int GA = BM * PBK * 2 / 1024 / NW, GB = BN * PBK * 2 / 1024 / NW, G = GA + GB;
-  constexpr bool SWIGLU = MODE == 2;
+  constexpr bool CLIPPED = MODE == 4, SWIGLU = MODE == 2 || CLIPPED;
   constexpr int OUTW = SWIGLU ? BN / 2 : BN;           // output tile width (elements)
   typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
   typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
@@ -1065,7 +1066,7 @@ __global__ void __launch_bounds__(256, 1) gemm_pf_kernel(const bf16* __restrict_
         if constexpr (SWIGLU) {
           const f32x4 g = acc[r][2 * i], u = acc[r][2 * i + 1];
 #pragma unroll
-          for (int v = 0; v < 4; ++v) hq[v] = f2bf(silu_f(g[v]) * u[v]);
+          for (int v = 0; v < 4; ++v) hq[v] = f2bf(CLIPPED ? clipped_glu_f(g[v], u[v], limit) : silu_f(g[v]) * u[v]);
         } else {
 #pragma unroll
           for (int v = 0; v < 4; ++v) hq[v] = f2bf(acc[r][i][v]);
@@ -1125,19 +1126,20 @@ int* pf_queue(hipStream_t s) {
 // 256 x 256 tiles, grid = min(tiles, CUs) rounded up to a multiple of 8.  variant bit 16: the
 // dynamic tile queue (DYN; needs K >= 128) instead of the static tile = w + i P walk; variant 8:
 // nontemporal output stores (by default: SwiGLU outputs > 256 MiB).
-void gemm_pf(uintptr_t c, uintptr_t a, uintptr_t b, int M, int N, int K, int mode, int variant, uintptr_t stream) {
+void gemm_pf(uintptr_t c, uintptr_t a, uintptr_t b, int M, int N, int K, int mode, int variant, uintptr_t stream,
+             float limit) {
   const bool dyn = (variant & 16) != 0;
   variant &= ~16;
   DLLM_HOST_CHECK(!dyn || K >= 2 * PBK, "the dynamic tile queue needs K >= 128");
   DLLM_HOST_CHECK(M >= 1, "M >= 1");
   DLLM_HOST_CHECK(K % PBK == 0 && K >= PBK, "K must be a positive multiple of 64");
   DLLM_HOST_CHECK(N % 256 == 0, "N must be a multiple of 256");
-  DLLM_HOST_CHECK(mode == 0 || mode == 1, "mode 0 (plain) or 1 (SwiGLU)");
+  DLLM_HOST_CHECK(mode == 0 || mode == 1 || mode == 3, "mode 0 (plain), 1 (SwiGLU) or 3 (clipped GLU)");
   DLLM_HOST_CHECK(variant == 0 || variant == 8, "variant 0 or 8 (nontemporal output stores)");
   // the output's byte range must stay below 2^31: rows past M are dropped by giving their stores
   // the offset 0x80000000, which has to lie outside the buffer's range
   DLLM_HOST_CHECK((long)M * K * 2 < (1L << 32) && (long)N * K * 2 < (1L << 32) &&
-                      (long)M * (mode == 1 ? N / 2 : N) * 2 < (1L << 31),
+                      (long)M * (mode != 0 ? N / 2 : N) * 2 < (1L << 31),
                   "operands must be < 4 GiB, the output < 2 GiB");
   // CUs of the current device, cached per device (a benign race: every thread stores the same value)
   static std::atomic<int> cus_of[64];
@@ -1157,8 +1159,12 @@ void gemm_pf(uintptr_t c, uintptr_t a, uintptr_t b, int M, int N, int K, int mod
   int* q = dyn ? pf_queue(s) : nullptr;
 #define DLLM_PF_GO(MODE_, SCH_, DYN_)                                                                         \
   hipLaunchKernelGGL((gemm_pf_kernel<MODE_, SCH_, DYN_>), dim3((unsigned)grid), dim3(256), 0, s, (const bf16*)a, \
-                     (const bf16*)b, (bf16*)c, M, N, K, q)
-  const bool nt_store = variant == 8 || (mode == 1 && (long)M * (N / 2) * 2 > (256L << 20));
+                     (const bf16*)b, (bf16*)c, M, N, K, q, limit)
+  const bool nt_store = variant == 8 || (mode != 0 && (long)M * (N / 2) * 2 > (256L << 20));
+  if (mode == 3) {
+    if (dyn) { if (nt_store) DLLM_PF_GO(4, 8, true); else DLLM_PF_GO(4, 0, true); }
+    else { if (nt_store) DLLM_PF_GO(4, 8, false); else DLLM_PF_GO(4, 0, false); }
+  } else
   if (mode == 1) {
     if (dyn) { if (nt_store) DLLM_PF_GO(2, 8, true); else DLLM_PF_GO(2, 0, true); }
     else { if (nt_store) DLLM_PF_GO(2, 8, false); else DLLM_PF_GO(2, 0, false); }

@@ -41,8 +41,14 @@ void hc_embed(uintptr_t x, uintptr_t ids, uintptr_t table, int tokens, int strea
               int f32, uintptr_t stream) {
   if (tokens <= 0) return;
   DLLM_HOST_CHECK(streams > 0 && width > 0 && vocab > 0 && x && ids && table, "hyper-connection embedding arguments");
-  SM_DISPATCH_V(f32, width % 8 == 0, hc_embed_kernel, dim3(tokens), dim3(256), 0, stream, (float*)x, (const int32_t*)ids,
-                (const void*)table, streams, width, vocab, scale);
+  const bool vec = width % 4 == 0 && x % 16 == 0 && table % (f32 ? 16 : 8) == 0;
+#define HC_EMBED(T, V)                                                                                               \
+  hipLaunchKernelGGL(HIP_KERNEL_NAME(hc_embed_kernel<T, V>), dim3(tokens), dim3(256), 0, (hipStream_t)stream, (float*)x, \
+                     (const int32_t*)ids, (const void*)table, streams, width, vocab, scale)
+  if (f32) { if (vec) HC_EMBED(float, 4); else HC_EMBED(float, 1); }
+  else { if (vec) HC_EMBED(bf16, 4); else HC_EMBED(bf16, 1); }
+#undef HC_EMBED
+  DLLM_HIP_CHECK(hipGetLastError());
 }
 
 template <typename T, int V, int S, bool EXACT>

@@ -481,7 +481,8 @@ void ml_chunk(uintptr_t o, uintptr_t proj, long ld, int qcol, int kcol, int vcol
 // The whole mixer between its projections in one launch, a workgroup per (sequence, head): gates, normaliser, the
 // state's step and read-out, the head's output norm (o / rms(o) * w) and the sigmoid gate.  The step is bound by reading
 // and writing the state ([Dv][D] float32): L lanes hold a value column, 4 key channels (16 bytes) each, and 8
-// columns' loads of a lane are in flight at a time; the read-out sums over the L lanes without LDS (DPP, row swaps).
+// columns' loads of a lane are in flight at a time (with few sequences and heads: 16 waves, so that one workgroup
+// has its whole state in flight); the read-out sums over the L lanes without LDS (DPP, row swaps).
 template <int L>
 __device__ __forceinline__ float ml_lanes_sum(float v) {         // over aligned groups of L lanes, result in all
   v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xb1 /* quad_perm 1 0 3 2 */, 0xf, 0xf, false));
@@ -500,14 +501,14 @@ __device__ __forceinline__ float ml_lanes_sum(float v) {         // over aligned
   return v;
 }
 
-template <typename T, int L>
-__global__ void __launch_bounds__(256) ml_step_kernel(
+template <typename T, int L, int NT>
+__global__ void __launch_bounds__(NT) ml_step_kernel(
     void* __restrict__ y_, const void* __restrict__ proj_, long ld, int qcol, int kcol, int vcol, int gcol, int icol,
     int fcol, const float* __restrict__ i_bias, const float* __restrict__ f_bias, float cap, float q_scale, float den_eps,
     float* __restrict__ s_state, float* __restrict__ n_state, float* __restrict__ m_state, const void* __restrict__ w_,
     float eps, const int32_t* __restrict__ cu, const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
     int H, int D, int Dv) {
-  constexpr int NG = 256 / L, U = 8;               // columns per pass; passes whose loads go out together
+  constexpr int NG = NT / L, U = NT == 256 ? 8 : 4;    // columns per pass; passes whose loads go out together
   __shared__ float red[16];
   extern __shared__ float so[];                    // the head's read-out [Dv]
   const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
@@ -574,11 +575,11 @@ __global__ void __launch_bounds__(256) ml_step_kernel(
   }
   if (tid == 0) m_state[srow] = mt;
   float ss = 0.f;
-  for (int v = tid; v < Dv; v += 256) ss += so[v] * so[v];
+  for (int v = tid; v < Dv; v += NT) ss += so[v] * so[v];
   const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)Dv + eps);
   const T* w = (const T*)w_ + (size_t)h * Dv;
   T* y = (T*)y_ + ((size_t)t * H + h) * Dv;
-  for (int v = tid; v < Dv; v += 256) {
+  for (int v = tid; v < Dv; v += NT) {
     const float g = (float)row[gcol + h * Dv + v];
     y[v] = (T)(so[v] * inv * (float)w[v] * (1.0f / (1.0f + expf(-g))));
   }
@@ -600,12 +601,13 @@ void ml_step(uintptr_t y, uintptr_t proj, long ld, int qcol, int kcol, int vcol,
   DLLM_HOST_CHECK(y && proj && i_bias && f_bias && s_state && s_state % 16 == 0 && n_state && m_state && w && cu && positions &&
                       slots,
                   "matrix memory step arguments");
-#define ML_STEP(T, L)                                                                                                 \
-  hipLaunchKernelGGL(HIP_KERNEL_NAME(ml_step_kernel<T, L>), dim3(H, seqs), dim3(256), sizeof(float) * (size_t)Dv,    \
+#define ML_STEP_N(T, L, NT)                                                                                                 \
+  hipLaunchKernelGGL(HIP_KERNEL_NAME(ml_step_kernel<T, L, NT>), dim3(H, seqs), dim3(NT), sizeof(float) * (size_t)Dv,    \
                      (hipStream_t)stream, (void*)y, (const void*)proj, ld, qcol, kcol, vcol, gcol, icol, fcol,       \
                      (const float*)i_bias, (const float*)f_bias, cap, q_scale, den_eps, (float*)s_state,             \
                      (float*)n_state, (float*)m_state, (const void*)w, eps, (const int32_t*)cu,                      \
                      (const int32_t*)positions, (const int32_t*)slots, H, D, Dv)
+#define ML_STEP(T, L) do { if ((long)H * seqs < 256) ML_STEP_N(T, L, 1024); else ML_STEP_N(T, L, 256); } while (0)
 #define ML_STEP_D(T)                 \
   do {                               \
     if (D <= 32) ML_STEP(T, 8);      \
@@ -617,6 +619,7 @@ void ml_step(uintptr_t y, uintptr_t proj, long ld, int qcol, int kcol, int vcol,
   else ML_STEP_D(bf16);
 #undef ML_STEP_D
 #undef ML_STEP
+#undef ML_STEP_N
   DLLM_HIP_CHECK(hipGetLastError());
 }
 

@@ -11,11 +11,14 @@
 
 namespace dllm {
 
-// out[m, n] = sum_s P[s, m, n] (+ bias[n]);  swiglu: out[m, j] = silu(sum P[m, j]) * sum P[m, I + j]
+// out[m, n] = sum_s P[s, m, n] (+ bias[n]);  ACT 1: out[m, j] = silu(sum P[m, j]) * sum P[m, I + j];  ACT 2: the
+// clipped GLU of `limit` (common.h) of the same pair
 // Each thread reduces V = 8 consecutive outputs (16-byte slab loads; 4 where ncols % 8 != 0).
-template <bool SWIGLU, int SC, int V>
+template <int ACT, int SC, int V>
 __global__ void __launch_bounds__(256) splitk_reduce_kernel(bf16* __restrict__ out, const float* __restrict__ P,
-                                                            const bf16* __restrict__ bias, int S_, int M, int N) {
+                                                            const bf16* __restrict__ bias, int S_, int M, int N,
+                                                            float limit) {
+  constexpr bool SWIGLU = ACT != 0;                    // gate and up columns are read together
   // SC > 0: compile-time slab count -> every slab load of a vector is in flight before the first
   // add (nontemporal: the slabs are read once); SC == 0: runtime loop
   static_assert(V == 4 || V == 8, "4 or 8 outputs per thread");
@@ -64,7 +67,8 @@ __global__ void __launch_bounds__(256) splitk_reduce_kernel(bf16* __restrict__ o
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         float x = a[h][j];
-        if (SWIGLU) x = silu_f(x) * u[h][j];
+        if (ACT == 2) x = clipped_glu_f(x, u[h][j], limit);
+        else if (ACT == 1) x = silu_f(x) * u[h][j];
         else if (bias) x += bf2f(bias[c + 4 * h + j]);
         o[h][j] = f2bf(x);
       }
@@ -242,8 +246,11 @@ void splitk_add_rms_norm_q8(uintptr_t y, uintptr_t residual, uintptr_t ws, int S
 }
 
 // plain split-K reduce of the partial slabs a split GEMM left (mode 2 of gemm_wide / gemm_sq / gemm_pp): out = bf16(sum_s P[s]) (+bias)
-void splitk_reduce_ex(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M, int N, int swiglu,
-                      uintptr_t stream) {
+// act 1: SwiGLU, act 2: clipped GLU of `limit` -- out [M, N / 2] from gate | up columns
+void splitk_reduce_ex(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M, int N, int act, uintptr_t stream,
+                      float limit) {
+  DLLM_HOST_CHECK(act >= 0 && act <= 2, "split-K reduce activation");
+  const bool swiglu = act != 0;
   DLLM_HOST_CHECK(N % (swiglu ? 8 : 4) == 0, "N alignment");
   const int ncols = swiglu ? N / 2 : N;
   const bool v8 = ncols % 8 == 0;
@@ -253,7 +260,7 @@ void splitk_reduce_ex(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M,
   hipStream_t st = reinterpret_cast<hipStream_t>(stream);
   const bf16* b = swiglu ? nullptr : (const bf16*)bias;
   auto go = [&](auto kern) {
-    hipLaunchKernelGGL(kern, dim3((unsigned)blocks), dim3(256), 0, st, (bf16*)out, (const float*)ws, b, S, M, N);
+    hipLaunchKernelGGL(kern, dim3((unsigned)blocks), dim3(256), 0, st, (bf16*)out, (const float*)ws, b, S, M, N, limit);
   };
 #define DLLM_SKR2(SW, V)                                               \
   do {                                                                 \
@@ -271,7 +278,9 @@ void splitk_reduce_ex(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M,
   do {                                                                 \
     if (v8) DLLM_SKR2(SW, 8); else DLLM_SKR2(SW, 4);                   \
   } while (0)
-  if (swiglu) DLLM_SKR(true); else DLLM_SKR(false);
+  if (act == 2) DLLM_SKR(2);
+  else if (act == 1) DLLM_SKR(1);
+  else DLLM_SKR(0);
 #undef DLLM_SKR
 #undef DLLM_SKR2
   DLLM_HIP_CHECK(hipGetLastError());
@@ -279,6 +288,11 @@ void splitk_reduce_ex(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M,
 
 void splitk_reduce(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M, int N, uintptr_t stream) {
   splitk_reduce_ex(out, ws, bias, S, M, N, 0, stream);
+}
+
+// out [M, N / 2] = the clipped GLU of the summed gate | up slabs
+void splitk_reduce_clipped(uintptr_t out, uintptr_t ws, int S, int M, int N, float limit, uintptr_t stream) {
+  splitk_reduce_ex(out, ws, 0, S, M, N, 2, stream, limit);
 }
 
 }  // namespace dllm

@@ -304,10 +304,11 @@ def linear_pp(x: torch.Tensor, w: torch.Tensor, splits: int = 0, swiglu: bool = 
     return y
 
 
-def linear_pf(x: torch.Tensor, w: torch.Tensor, swiglu: bool = False, variant: int = 0) -> torch.Tensor:
+def linear_pf(x: torch.Tensor, w: torch.Tensor, swiglu: bool = False, variant: int = 0,
+              limit: Optional[float] = None) -> torch.Tensor:
     """Persistent prefill GEMM (gemm_pf in csrc/kernels/gemm_pp.hip): schedule 2's 256 x 256 tiles,
     one workgroup per CU walking its tiles with the LDS-DMA pipeline running across tile
-    boundaries; optional fused SwiGLU (``w`` = [Wg; Wu], y [M, N / 2]).  ``variant`` 8: nontemporal
+    boundaries; optional fused SwiGLU (``w`` = [Wg; Wu], y [M, N / 2]) or -- ``limit`` -- clipped GLU.  ``variant`` 8: nontemporal
     output stores (the default for SwiGLU outputs > 256 MiB); the tiles come from per-XCD device
     queues while knobs.pf_dynamic says so (bit 16 of the launcher's variant)."""
     k = x.shape[-1]
@@ -317,7 +318,8 @@ def linear_pf(x: torch.Tensor, w: torch.Tensor, swiglu: bool = False, variant: i
         raise ValueError("linear_pf: bf16 contiguous operands")
     if n % 256 or k % 64:
         raise ValueError("linear_pf: N % 256 and K % 64")
-    y = torch.empty(*x.shape[:-1], n // 2 if swiglu else n, dtype=x.dtype, device=x.device)
+    glu = swiglu or limit is not None
+    y = torch.empty(*x.shape[:-1], n // 2 if glu else n, dtype=x.dtype, device=x.device)
     dyn = pf_dynamic() and k >= 128
     if torch.cuda.is_current_stream_capturing():
         # inside a graph: the static tile walk.  A tile queue is per stream and self-resetting, but
@@ -325,8 +327,9 @@ def linear_pf(x: torch.Tensor, w: torch.Tensor, swiglu: bool = False, variant: i
         dyn = False
     if dyn:
         variant |= 16                  # per-XCD dynamic tile queues (gemm_pp.hip, DYN)
-    _ext.kernels().gemm_pf(y.data_ptr(), x.data_ptr(), w.data_ptr(), m, n, k, 1 if swiglu else 0, variant,
-                           torch.cuda.current_stream().cuda_stream)
+    _ext.kernels().gemm_pf(y.data_ptr(), x.data_ptr(), w.data_ptr(), m, n, k,
+                           3 if limit is not None else (1 if swiglu else 0), variant, torch.cuda.current_stream().cuda_stream,
+                           0.0 if limit is None else float(limit))
     return y
 
 
@@ -388,6 +391,28 @@ def linear_sq(x: torch.Tensor, w: torch.Tensor, splits: int = 0, swiglu: bool = 
     _ext.kernels().gemm_sq(y.data_ptr(), x.data_ptr(), w.data_ptr(), ws.data_ptr(), ws.numel(), m, n, k, s,
                            1 if swiglu else 0, v, stream)
     return y
+
+
+def linear_clipped_glu(x: torch.Tensor, w_gate_up: torch.Tensor, limit: float) -> Optional[torch.Tensor]:
+    """g sigmoid(1.702 g) (u + 1), g = min(x Wg^T, limit), u = clamp(x Wu^T, -limit, limit), W = [Wg; Wu], with the
+    activation in the persistent GEMM's epilogue (prompts) or in the split-K reduction (decode); None if the
+    shape takes neither."""
+    k = x.shape[-1]
+    n = w_gate_up.shape[0]
+    m = x.numel() // k
+    if x.dtype != torch.bfloat16 or n % 256:
+        return None
+    if not _use_wide(m, n, k, x, w_gate_up) and _use_pp(m, n, k, x, w_gate_up, knobs.K.pp_swiglu_min_m) \
+            and knobs.K.pp_persistent and m * (n // 2) * 2 < (1 << 31) and pf_fills(m, n, x.device):
+        return linear_pf(x, w_gate_up, limit=limit)
+    y = linear(x, w_gate_up, defer=True)
+    if isinstance(y, SplitKPartial):
+        out = torch.empty(*x.shape[:-1], n // 2, dtype=x.dtype, device=x.device)
+        _ext.kernels().splitk_reduce_clipped(out.data_ptr(), y.ws.data_ptr(), y.splits, y.m, y.n, float(limit),
+                                             torch.cuda.current_stream().cuda_stream)
+        return out
+    from .seqmix import clipped_glu
+    return clipped_glu(y, None, limit)
 
 
 def linear_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor) -> Optional[torch.Tensor]:

@@ -301,8 +301,12 @@ def route_softmax_all(logits: torch.Tensor, top: int, scale: float = 1.0):
 
 def linear_clipped_glu(x: torch.Tensor, w_gate_up: torch.Tensor, limit: float, alpha: float = 1.702) -> torch.Tensor:
     """g sigmoid(alpha g) (u + 1) with g = min(x Wg^T, limit), u = clamp(x Wu^T, -limit, limit), W = [Wg; Wu]."""
-    from . import linear
+    from . import gemm, linear
     from .seqmix import clipped_glu
+    if x.is_cuda and alpha == 1.702:                # the constant of the fused epilogues (kGluAlpha in common.h)
+        y = gemm.linear_clipped_glu(x, w_gate_up, limit)
+        if y is not None:
+            return y
     return clipped_glu(linear(x, w_gate_up), None, limit, alpha)
 
 

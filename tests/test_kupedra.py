@@ -550,6 +550,23 @@ def test_clipped_experts_weighted_over_all_logits(target, sizes, tokens):
         assert np.median([O.route(r, top)[1].sum() for r in z]) < 0.995
 
 
+@pytest.mark.parametrize("target", TARGETS)
+@pytest.mark.parametrize("tokens,width,ff", [(1, 256, 128), (3, 72, 24), (33, 512, 1024), (200, 2048, 256), (700, 256, 256),
+                                             (8192, 128, 1024)])
+def test_dense_clipped_glu(target, tokens, width, ff):
+    """Gate clipped from above only, up from both sides and shifted by one: decode sizes (in the split-K reduction),
+    prompt sizes (in the persistent GEMM's epilogue) and sizes that take neither."""
+    device, dtype = _dev(target)
+    rng = np.random.default_rng(ff)
+    x, w = _t(rng, dtype, tokens, width), _t(rng, dtype, 2 * ff, width, scale=2.0 * width ** -0.5)
+    got = _d(moe.linear_clipped_glu(x.to(device), w.to(device), 1.1))
+    rows = np.unique(np.linspace(0, tokens - 1, 80).astype(int))
+    want = O.clipped_expert(_d(x)[rows], {"gate": _d(w)[:ff], "up": _d(w)[ff:], "down": np.eye(ff)}, 1.1)
+    np.testing.assert_allclose(got[rows], want, atol=2e-5 if dtype == torch.float32 else 3e-2)
+    g = _d(x)[rows] @ _d(w)[:ff].T
+    assert (g > 1.1).any() and (g < -1.1).any() and want.min() < -0.1
+
+
 # ------------------------------------------------------------------------------ the engine
 @pytest.mark.parametrize("target", TARGETS)
 @pytest.mark.parametrize("name", ["a", "b", "c"])
