@@ -22,7 +22,7 @@ from typing import Any, Dict, List, Optional
 @dataclass
 class ModelConfig:
     name: str
-    arch: str                      # "llama" (Llama-2/3), "mixtral", "gpt2"; layer-list models: "tudilix", "gikovik", "zebutar", "fekizen", "kupedra"
+    arch: str                      # "llama" (Llama-2/3), "mixtral", "gpt2"; layer-list models: "tudilix", "gikovik", "zebutar", "fekizen", "kupedra", "basopel"
     vocab_size: int
     hidden_size: int
     intermediate_size: int
@@ -49,7 +49,7 @@ class ModelConfig:
     # their weights (every repetition gets separate caches); and the width of the per-layer token input
     loop: Optional[Dict[str, int]] = None
     token_side_dim: int = 0
-    embed_scale: float = 1.0       # arch "fekizen" (with ``max_position`` rows of learned positions), "kupedra": token embeddings enter times this
+    embed_scale: float = 1.0       # arch "fekizen" (with ``max_position`` rows of learned positions), "kupedra", "basopel": token embeddings enter times this
     streams: int = 1               # arch "kupedra": residual streams per token (hyper-connections)
     logit_scale: float = 1.0       # arch "kupedra": the head's product times this
 
@@ -150,6 +150,10 @@ class ModelConfig:
             if self.loop:
                 d["loop"] = dict(self.loop)
             return d
+        if self.arch == "basopel":
+            return {"architecture": "Basopel", "layers": [dict(l) for l in self.layers], "norm": {"eps": self.norm_eps},
+                    "vocab": self.vocab_size, "width": self.hidden_size, "embedding": {"scale": self.embed_scale},
+                    "_dllm_name": self.name}
         if self.arch == "zebutar":
             return {"architecture": "Zebutar", "layers": [dict(l) for l in self.layers], "norm": {"eps": self.norm_eps},
                     "vocab": self.vocab_size, "width": self.hidden_size, "_dllm_name": self.name}
@@ -199,6 +203,8 @@ class ModelConfig:
             return _from_fekizen(cfg, name)
         if cfg.get("architecture") == "Kupedra":
             return _from_kupedra(cfg, name)
+        if cfg.get("architecture") == "Basopel":
+            return _from_basopel(cfg, name)
         mt = cfg.get("model_type", "llama")
         name = name or cfg.get("_dllm_name") or cfg.get("_name_or_path") or mt
         eos = cfg.get("eos_token_id", 2)
@@ -377,6 +383,30 @@ def _from_kupedra(cfg: Dict[str, Any], name: Optional[str] = None) -> ModelConfi
         logit_scale=float(1.0 if cfg.get("logit_scale") is None else cfg["logit_scale"]))
 
 
+def _from_basopel(cfg: Dict[str, Any], name: Optional[str] = None) -> ModelConfig:
+    """A ``config.json`` with "architecture": "Basopel": ``width``, ``vocab``, ``norm.eps``, ``embedding.scale``, ``layers``
+    (per layer ``type`` "attention" | "attention_2" | "latent_attention", ``mixer`` sizes, ``mlp`` None | dense)."""
+    layers = [dict(l) for l in cfg["layers"]]
+    if not layers:
+        raise ValueError("layer-list config without layers")
+    for l in layers:
+        if l["type"] not in ("attention", "attention_2", "latent_attention"):
+            raise ValueError(f"unsupported layer type {l['type']!r} (attention, attention_2, latent_attention)")
+        if l.get("mlp") is not None and l["mlp"].get("kind", "dense") != "dense":
+            raise ValueError(f"unsupported mlp kind {l['mlp'].get('kind')!r} (dense)")
+    extra = set(cfg.get("norm", {})) - {"eps"}
+    if extra:
+        raise ValueError(f"unsupported norm options {sorted(extra)}")
+    mix = [l["mixer"] for l in layers]
+    return ModelConfig(
+        name=name or cfg.get("_dllm_name") or "basopel", arch="basopel", vocab_size=int(cfg["vocab"]),
+        hidden_size=int(cfg["width"]), intermediate_size=int(max([l["mlp"]["ff"] for l in layers if l.get("mlp")] or [0])),
+        num_layers=len(layers), num_heads=max(m["heads"] for m in mix), num_kv_heads=max(m.get("kv_heads", 1) for m in mix),
+        head_dim=max(m["kv_rank"] + m["rot_dim"] if "kv_rank" in m else max(m["dim"], m["vdim"]) for m in mix),
+        max_position=1 << 30, norm_eps=float(cfg["norm"]["eps"]), bos_token_id=-1, eos_token_id=-1, tie_embeddings=True,
+        layers=layers, embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)))
+
+
 _LLAMA3_ROPE = {"rope_type": "llama3", "factor": 8.0, "low_freq_factor": 1.0,
                 "high_freq_factor": 4.0, "original_max_position_embeddings": 8192}
 
@@ -507,6 +537,21 @@ PRESETS: Dict[str, ModelConfig] = {
             {"type": "attention", "mixer": {"heads": 2, "kv_heads": 2, "dim": 16, "vdim": 16, "scale": 0.25,
                                             "rot": {"base": 500.0, "dims": 8}}, "mlp": None},
         ]}, name="tiny-kupedra"),
+    "tiny-basopel": _from_basopel({
+        "architecture": "Basopel", "vocab": 272, "width": 96, "norm": {"eps": 1e-6}, "embedding": {"scale": 9.0},
+        "layers": [
+            {"type": "attention", "mixer": {"heads": 3, "kv_heads": 1, "dim": 32, "vdim": 24, "scale": 0.2, "bias_max": 40,
+                                            "mask": {"size": 20, "keep_first": 3}, "v_mix": True},
+             "mlp": {"kind": "dense", "ff": 160}},
+            {"type": "latent_attention", "mixer": {"heads": 4, "dim": 16, "rot_dim": 8, "vdim": 24, "kv_rank": 40,
+                                                   "scale": 0.2, "mask": {"size": 33},
+                                                   "rot": {"base": 10000.0, "dims": 8}},
+             "mlp": None},
+            {"type": "attention_2", "mixer": {"heads": 2, "kv_heads": 1, "dim": 16, "vdim": 24, "scale": 0.25, "softcap": 20.0,
+                                              "mask": {"size": 24}, "v_mix": True,
+                                              "rot": {"base": 500.0, "dims": 8, "scaling": {"factor": 2.0}}},
+             "mlp": {"kind": "dense", "ff": 128}},
+        ]}, name="tiny-basopel"),
     "tiny-gpt2": ModelConfig(
         name="tiny-gpt2", arch="gpt2", vocab_size=512, hidden_size=128,
         intermediate_size=512, num_layers=4, num_heads=2, num_kv_heads=2, head_dim=64,

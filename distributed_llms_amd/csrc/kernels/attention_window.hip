@@ -13,6 +13,10 @@
 // `bias` (float32 [H, nbias], or null) is added to head h's scaled score of a key n positions before the query:
 // bias[h][min(n, nbias - 1)] (a learned distance bias, expanded from its buckets by the caller; a tile all of
 // whose keys are nbias - 1 or more back adds one constant).
+// `keep` > 0 (not beside averaged caches): a query at position p also sees the first `keep` positions of its sequence;
+// those that lie before its window, [0, nkeep(p) - 1] with nkeep(p) = min(keep, win_lo(p)), are visited first, as the
+// averaged entries are.  `gate` (T, row stride gate_ld, or null): head h's output is multiplied by
+// sigmoid(gate[t * gate_ld + h]).
 // Scores, softmax weights and the weighted sum are float32; T is the storage
 // type (bf16 or float).  Head sizes, window and block size are runtime values.
 //
@@ -50,6 +54,13 @@ __device__ __forceinline__ int win_lo(int pos, int window, int chunk) {
 __device__ __forceinline__ int win_npool(int pos, int window, int pool) {
   return pool > 0 ? max(pos - window + 1, 0) / pool : 0;
 }
+
+// Entries a query at `pos` visits before its window: averaged ones, or the sequence's first tokens that stay visible.
+__device__ __forceinline__ int win_nfirst(int pos, int window, int chunk, int pool, int keep) {
+  return pool > 0 ? win_npool(pos, window, pool) : min(keep, win_lo(pos, window, chunk));
+}
+
+__device__ __forceinline__ float gate_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 // softcap tanh(s / softcap) from exp2 and a reciprocal (the matrix-core kernels; the row kernel, which is
 // the float32 path, calls tanhf): tanh(x) = 1 - 2 / (e^(2x) + 1), exact at both ends (e -> inf, e -> 0)
@@ -110,7 +121,7 @@ __global__ void __launch_bounds__(kWinTile) window_attn_row_kernel(
     const int32_t* __restrict__ positions, const int32_t* __restrict__ tok_seq, int t0, int H, int G, int D, int Dv,
     int bs, int window, int chunk, float scale, const float* __restrict__ sinks, float softcap,
     const void* __restrict__ kp_, const void* __restrict__ vp_, int pool, int pbs, const float* __restrict__ bias,
-    int nbias) {
+    int nbias, int keep, const void* __restrict__ gate_, long gate_ld) {
   extern __shared__ float lds[];
   float* qs = lds;                       // [D]
   float* p = qs + D;                     // [kWinTile]
@@ -169,8 +180,11 @@ __global__ void __launch_bounds__(kWinTile) window_attn_row_kernel(
       __syncthreads();                            // before the next tile overwrites p and rows
     }
   };
-  const int np = win_npool(pos, window, pool);
-  if (np > 0) run((const T*)kp_, (const T*)vp_, pbs, 0, np - 1);
+  const int np = win_nfirst(pos, window, chunk, pool, keep);
+  if (np > 0) {
+    if (pool > 0) run((const T*)kp_, (const T*)vp_, pbs, 0, np - 1);
+    else run((const T*)k_cache_, (const T*)v_cache_, bs, 0, np - 1);
+  }
   run((const T*)k_cache_, (const T*)v_cache_, bs, lo, pos);
   // a sink adds exp(sink) to the denominator; nothing is attended to through it
   float fin = 1.0f / l;
@@ -178,6 +192,7 @@ __global__ void __launch_bounds__(kWinTile) window_attn_row_kernel(
     const float sk = sinks[h], mf = fmaxf(m, sk), cf = expf(m - mf);
     fin = cf / (l * cf + expf(sk - mf));
   }
+  if (gate_) fin *= gate_f(wld((const T*)gate_ + (size_t)t * gate_ld + h));
   // sum the key subgroups
   T* out = (T*)out_ + ((size_t)t * H + h) * Dv;
 #pragma unroll
@@ -202,7 +217,9 @@ static size_t win_row_lds(int D, int Dv) {
 static void launch_rows(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                         int max_blocks, uintptr_t positions, uintptr_t tok_seq, int t0, int rows, int H, int G, int D,
                         int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, float softcap, uintptr_t kp,
-                        uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int f32, uintptr_t stream) {
+                        uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int keep, uintptr_t gate,
+                        long gate_ld, int f32, uintptr_t stream) {
+  DLLM_HOST_CHECK(keep >= 0 && (keep == 0 || pool == 0) && (!gate || gate_ld >= H), "window attention kept tokens / gate");
   DLLM_HOST_CHECK(!bias || (nbias >= 1 && pool == 0), "window attention distance bias");
   DLLM_HOST_CHECK(H > 0 && G > 0 && H % G == 0 && D > 0 && Dv > 0 && Dv <= kWinTile * kWinMaxAcc, "window attention heads");
   DLLM_HOST_CHECK(pool == 0 || (pool > 0 && kp && vp && pbs > 0 && chunk == 0), "window attention averaged caches");
@@ -214,13 +231,13 @@ static void launch_rows(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t
                        (hipStream_t)stream, (void*)out, (const void*)q, (const void*)k_cache, (const void*)v_cache,
                        (const int32_t*)block_tables, max_blocks, (const int32_t*)positions, (const int32_t*)tok_seq, t0,
                        H, G, D, Dv, bs, window, chunk, scale, (const float*)sinks, softcap, (const void*)kp, (const void*)vp,
-                       pool, pbs, (const float*)bias, nbias);
+                       pool, pbs, (const float*)bias, nbias, keep, (const void*)gate, gate_ld);
   else
     hipLaunchKernelGGL(HIP_KERNEL_NAME(window_attn_row_kernel<bf16>), dim3(rows, H), dim3(kWinTile), lds,
                        (hipStream_t)stream, (void*)out, (const void*)q, (const void*)k_cache, (const void*)v_cache,
                        (const int32_t*)block_tables, max_blocks, (const int32_t*)positions, (const int32_t*)tok_seq, t0,
                        H, G, D, Dv, bs, window, chunk, scale, (const float*)sinks, softcap, (const void*)kp, (const void*)vp,
-                       pool, pbs, (const float*)bias, nbias);
+                       pool, pbs, (const float*)bias, nbias, keep, (const void*)gate, gate_ld);
   DLLM_HIP_CHECK(hipGetLastError());
 }
 
@@ -262,7 +279,7 @@ __global__ void __launch_bounds__(256) window_attn_tile_kernel(
     const int32_t* __restrict__ cu, const int32_t* __restrict__ positions, int seq0, int nseq, int nqt, int H, int G,
     int D, int Dv, int bs, int window, int chunk, float scale, const float* __restrict__ sinks, int sub, float softcap,
     const bf16* __restrict__ kp_cache, const bf16* __restrict__ vp_cache, int pool, int pbs,
-    const float* __restrict__ bias, int nbias) {
+    const float* __restrict__ bias, int nbias, int keep, const bf16* __restrict__ gate, long gate_ld) {
   constexpr int kQT = QT, kTQ = 64 * QT;
   constexpr int DP = 32 * NQK, KROW = DP + kPad, VROW = kTK + kPad;
   constexpr int KPT = (kTK * (DP / 8) + 255) / 256, VPT = (16 * NDV * (kTK / 8) + 255) / 256;   // 16-byte pieces per thread
@@ -485,13 +502,16 @@ __global__ void __launch_bounds__(256) window_attn_tile_kernel(
   };
   const int tile_last = start + min(q0 + kTQ, n) - 1;                  // position of the tile's last query
   const int wave_last = start + min(wq0 + 16 * kQT - 1, n - 1);        // of the wave's last query
-  // ---- phase 1: the averaged entries (entry indices are the keys): query at p sees [0, npool(p) - 1]
-  const int np_tile = win_npool(tile_last, window, pool);
+  // ---- phase 1: the averaged entries (entry indices are the keys) or the kept first tokens: query at p sees
+  // [0, nfirst(p) - 1], not decreasing in p
+  const int np_tile = win_nfirst(tile_last, window, chunk, pool, keep);
   if (np_tile > 0) {                                                   // uniform over the workgroup
-    ck = kp_cache, cv = vp_cache, cbs = pbs, cbsh = __ffs(pbs) - 1, last_pos = np_tile - 1;
+    if (pool > 0) ck = kp_cache, cv = vp_cache, cbs = pbs, cbsh = __ffs(pbs) - 1;
+    last_pos = np_tile - 1;
 #pragma unroll
-    for (int c2 = 0; c2 < kQT; ++c2) lo_q[c2] = 0, hi_q[c2] = win_npool(qpos[c2], window, pool) - 1;
-    run(0, 0, win_npool(wave_last, window, pool) - 1, 0, win_npool(start + wq0, window, pool) - 1);
+    for (int c2 = 0; c2 < kQT; ++c2) lo_q[c2] = 0, hi_q[c2] = win_nfirst(qpos[c2], window, chunk, pool, keep) - 1;
+    run(0, 0, win_nfirst(wave_last, window, chunk, pool, keep) - 1, 0,
+        win_nfirst(start + wq0, window, chunk, pool, keep) - 1);
     __syncthreads();                                                   // before the next phase's first fetch lands in LDS
   }
   // ---- phase 2: the tokens of the window
@@ -514,6 +534,7 @@ __global__ void __launch_bounds__(256) window_attn_tile_kernel(
       const float sk = sinks[h] * kLog2e, mf = fmaxf(m[c2], sk), cf = __builtin_amdgcn_exp2f(m[c2] - mf);
       inv = cf / (l[c2] * cf + __builtin_amdgcn_exp2f(sk - mf));
     }
+    if (gate) inv *= gate_f(bf2f(gate[(size_t)(lo_t + ql[c2]) * gate_ld + h]));
     bf16* orow = out + ((size_t)(lo_t + ql[c2]) * H + h) * Dv;
 #pragma unroll
     for (int dt = 0; dt < NDV; ++dt) {
@@ -532,7 +553,8 @@ template <int NQK, int NDV, int QT, bool BIAS>
 static void launch_tile(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                         int max_blocks, uintptr_t cu, uintptr_t positions, int seq0, int nseq, int max_q_len, int H,
                         int G, int D, int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, float softcap,
-                        uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, uintptr_t stream) {
+                        uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int keep, uintptr_t gate,
+                        long gate_ld, uintptr_t stream) {
   constexpr int kTQ = 64 * QT;
   const int nqt = (max_q_len + kTQ - 1) / kTQ;
   const int pairs = nseq * G, per_pair = nqt * (H / G);
@@ -543,7 +565,8 @@ static void launch_tile(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t
                      dim3(256), BIAS && nbias <= kBiasLds ? sizeof(float) * nbias : 0, (hipStream_t)stream, (bf16*)out, (const bf16*)q, (const bf16*)k_cache,
                      (const bf16*)v_cache, (const int32_t*)block_tables, max_blocks, (const int32_t*)cu,
                      (const int32_t*)positions, seq0, nseq, nqt, H, G, D, Dv, bs, window, chunk, scale, (const float*)sinks, sub,
-                     softcap, (const bf16*)kp, (const bf16*)vp, pool, pbs, (const float*)bias, nbias);
+                     softcap, (const bf16*)kp, (const bf16*)vp, pool, pbs, (const float*)bias, nbias, keep,
+                     (const bf16*)gate, gate_ld);
   DLLM_HIP_CHECK(hipGetLastError());
 }
 
@@ -563,7 +586,7 @@ __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
     const int32_t* __restrict__ positions, const int32_t* __restrict__ tok_seq, int H, int G, int D, int Dv, int bs,
     int window, int chunk, float scale, const float* __restrict__ sinks, int hpw, int splits, float* __restrict__ ws,
     float softcap, const bf16* __restrict__ kp_cache, const bf16* __restrict__ vp_cache, int pool, int pbs,
-    const float* __restrict__ bias, int nbias) {
+    const float* __restrict__ bias, int nbias, int keep, const bf16* __restrict__ gate, long gate_ld) {
   constexpr int DVP = 16 * NDV;
   __shared__ float so[kDW][16][DVP + 1];
   __shared__ float sml[kDW][2][16];
@@ -597,17 +620,19 @@ __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
   float m = -INFINITY, l = 0.f;
   // keys of this lane's A rows inside a tile: first half row col -> key 8 (col / 4) + col % 4, second half + 4
   const int jr = 8 * (col >> 2) + (col & 3);
-  // The row's tiles of 32 keys: first the averaged entries (tiles 0 .. ptile - 1 over entries [0, np - 1] of
-  // the averaged caches), then the window's tokens (tiles from the 32-aligned k00 over positions [lo, pos]).
-  const int np = win_npool(pos, window, pool), ptile = (np + 31) >> 5;
-  const int pbsh = pool > 0 ? __ffs(pbs) - 1 : 0;
+  // The row's tiles of 32 keys: first the averaged entries or kept first tokens (tiles 0 .. ptile - 1 over entries
+  // [0, np - 1] of their cache), then the window's tokens (tiles from the 32-aligned k00 over positions [lo, pos]).
+  const int np = win_nfirst(pos, window, chunk, pool, keep), ptile = (np + 31) >> 5;
+  const bf16* fk_cache = pool > 0 ? kp_cache : k_cache;
+  const bf16* fv_cache = pool > 0 ? vp_cache : v_cache;
+  const int fbs = pool > 0 ? pbs : bs, pbsh = __ffs(fbs) - 1;
   const int k00 = lo & ~31, ntile = ptile + ((pos - k00) >> 5) + 1;
   bf16x8 ka[NQK], kb[NQK];
   auto load_k = [&](int ti) {
     const bool pooled = ti < ptile;
     const int k0 = pooled ? 32 * ti : k00 + 32 * (ti - ptile), hi = pooled ? np - 1 : pos;
-    const bf16* kc = pooled ? kp_cache : k_cache;
-    const int cb = pooled ? pbs : bs, sh = pooled ? pbsh : bsh;
+    const bf16* kc = pooled ? fk_cache : k_cache;
+    const int cb = pooled ? fbs : bs, sh = pooled ? pbsh : bsh;
     const int j1 = min(k0 + jr, hi), j2 = min(k0 + jr + 4, hi);
     const bf16* r1 = kc + (((size_t)bt[j1 >> sh] * G + g) * cb + (j1 & (cb - 1))) * D;
     const bf16* r2 = kc + (((size_t)bt[j2 >> sh] * G + g) * cb + (j2 & (cb - 1))) * D;
@@ -636,8 +661,8 @@ __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
     const bool pooled = ti < ptile;
     const int k0 = pooled ? 32 * ti : k00 + 32 * (ti - ptile);
     const int rlo = pooled ? 0 : lo, rhi = pooled ? np - 1 : pos;
-    const bf16* vcache = pooled ? vp_cache : v_cache;
-    const int cb = pooled ? pbs : bs, sh = pooled ? pbsh : bsh;
+    const bf16* vcache = pooled ? fv_cache : v_cache;
+    const int cb = pooled ? fbs : bs, sh = pooled ? pbsh : bsh;
     // this tile's V^T pieces (8 keys from k0 + 8 grp, clamped to the last piece that exists) go out first
     const int kp8 = min(k0 + 8 * grp, rhi & ~7);
     const bf16* vbase = vcache + ((size_t)bt[kp8 >> sh] * G + g) * Dv * cb + (kp8 & (cb - 1));
@@ -730,7 +755,9 @@ __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
       ll += sml[w][1][hh] * f;
       o += so[w][hh][e] * f;
     }
-    out[((size_t)t * H + hb + hh) * Dv + e] = (bf16)(o / ll);
+    o /= ll;
+    if (gate) o *= gate_f(bf2f(gate[(size_t)t * gate_ld + hb + hh]));
+    out[((size_t)t * H + hb + hh) * Dv + e] = (bf16)o;
   }
 }
 
@@ -738,7 +765,8 @@ __global__ void __launch_bounds__(64 * kDW) window_attn_decode_kernel(
 // sums relative to the split's maximum, the maximum, the weight sum) -> out [rows, H, Dv]
 __global__ void __launch_bounds__(64) window_attn_merge_kernel(bf16* __restrict__ out, const float* __restrict__ ws,
                                                                int H, int Dv, int splits,
-                                                               const float* __restrict__ sinks) {
+                                                               const float* __restrict__ sinks,
+                                                               const bf16* __restrict__ gate, long gate_ld) {
   // a lane per split (at most 64) loads its maximum and weight sum; the factors then wait in LDS
   __shared__ float sf[64];
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -748,13 +776,14 @@ __global__ void __launch_bounds__(64) window_attn_merge_kernel(bf16* __restrict_
   const float mm = wave_max(sinks ? fmaxf(m, sinks[h]) : m);
   const float f = m == -INFINITY ? 0.f : expf(m - mm);
   const float ll = wave_sum(l * f) + (sinks ? expf(sinks[h] - mm) : 0.f);
+  const float fin = (gate ? gate_f(bf2f(gate[(size_t)t * gate_ld + h])) : 1.0f) / ll;
   sf[lane] = f;
   __syncthreads();
   for (int e = threadIdx.x; e < Dv; e += 64) {
     float o = 0.f;
 #pragma unroll 8
     for (int s2 = 0; s2 < splits; ++s2) o = fmaf(part[s2 * (Dv + 2) + e], sf[s2], o);
-    out[((size_t)t * H + h) * Dv + e] = (bf16)(o / ll);
+    out[((size_t)t * H + h) * Dv + e] = (bf16)(o * fin);
   }
 }
 
@@ -762,7 +791,8 @@ template <int NQK, int NDV, bool BIAS>
 static void launch_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                           int max_blocks, uintptr_t positions, uintptr_t tok_seq, int rows, int H, int G, int D,
                           int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, int splits, uintptr_t ws,
-                          float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, uintptr_t stream) {
+                          float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int keep,
+                          uintptr_t gate, long gate_ld, uintptr_t stream) {
   // heads per workgroup: 16 (all MFMA columns) when rows x K/V heads x key runs fill the chip, else halved
   // until about half the CUs have a workgroup -- the keys are re-read from L2, the columns left idle cost
   // nothing.  Key runs come first: a workgroup holds a CU's registers alone, so the call takes
@@ -776,11 +806,11 @@ static void launch_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr
                      (hipStream_t)stream, (bf16*)out, (const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache,
                      (const int32_t*)block_tables, max_blocks, (const int32_t*)positions, (const int32_t*)tok_seq, H, G,
                      D, Dv, bs, window, chunk, scale, (const float*)sinks, hpw, splits, (float*)ws, softcap, (const bf16*)kp,
-                     (const bf16*)vp, pool, pbs, (const float*)bias, nbias);
+                     (const bf16*)vp, pool, pbs, (const float*)bias, nbias, keep, (const bf16*)gate, gate_ld);
   DLLM_HIP_CHECK(hipGetLastError());
   if (splits > 1) {
     hipLaunchKernelGGL(window_attn_merge_kernel, dim3(rows, H), dim3(64), 0, (hipStream_t)stream, (bf16*)out,
-                       (const float*)ws, H, Dv, splits, (const float*)sinks);
+                       (const float*)ws, H, Dv, splits, (const float*)sinks, (const bf16*)gate, gate_ld);
     DLLM_HIP_CHECK(hipGetLastError());
   }
 }
@@ -798,23 +828,24 @@ static bool win_mfma_ok(int f32, int H, int G, int D, int Dv, int bs, int pool, 
 void sm_window_attn_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                            int max_blocks, uintptr_t positions, uintptr_t tok_seq, int rows, int H, int G, int D,
                            int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, int splits, uintptr_t ws,
-                           float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int f32,
-                           uintptr_t stream) {
+                           float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int keep,
+                           uintptr_t gate, long gate_ld, int f32, uintptr_t stream) {
   if (rows <= 0) return;
   if (win_mfma_ok(f32, H, G, D, Dv, bs, pool, pbs) && (long)G * ((H / G + 1) / 2) <= 65535) {
     DLLM_HOST_CHECK(window >= 1 && chunk >= 0 && max_blocks > 0, "window attention sizes");
     DLLM_HOST_CHECK(pool == 0 || (pool > 0 && kp && vp && chunk == 0), "window attention averaged caches");
     DLLM_HOST_CHECK(!bias || (nbias >= 1 && pool == 0), "window attention distance bias");
+    DLLM_HOST_CHECK(keep >= 0 && (keep == 0 || pool == 0) && (!gate || gate_ld >= H), "window attention kept tokens / gate");
 #define WIN_DEC(NQK, NDV)                                                                                          \
   do {                                                                                                             \
     if (bias)                                                                                                      \
       launch_decode<NQK, NDV, true>(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, rows, H, G, \
                                     D, Dv, bs, window, chunk, scale, sinks, splits, ws, softcap, kp, vp, pool, pbs, \
-                                    bias, nbias, stream);                                                          \
+                                    bias, nbias, keep, gate, gate_ld, stream);                                     \
     else                                                                                                           \
       launch_decode<NQK, NDV, false>(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, rows, H, G, \
                                      D, Dv, bs, window, chunk, scale, sinks, splits, ws, softcap, kp, vp, pool, pbs, \
-                                     0, 0, stream);                                                                \
+                                     0, 0, keep, gate, gate_ld, stream);                                           \
   } while (0)
     if (D <= 64 && Dv <= 64) WIN_DEC(2, 4);
     else if (D <= 128 && Dv <= 128) WIN_DEC(4, 8);
@@ -823,7 +854,7 @@ void sm_window_attn_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintpt
     return;
   }
   launch_rows(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, 0, rows, H, G, D, Dv, bs, window,
-              chunk, scale, sinks, softcap, kp, vp, pool, pbs, bias, nbias, f32, stream);
+              chunk, scale, sinks, softcap, kp, vp, pool, pbs, bias, nbias, keep, gate, gate_ld, f32, stream);
 }
 
 // Prompt chunks: tokens [t0 .. tokens) of sequences [seq0, seqs).
@@ -831,7 +862,8 @@ void sm_window_attn_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintp
                             int max_blocks, uintptr_t cu, uintptr_t positions, uintptr_t tok_seq, int seq0, int seqs,
                             int tokens, int max_q_len, int H, int G, int D, int Dv, int bs, int window, int chunk,
                             float scale, uintptr_t sinks, float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs,
-                            uintptr_t bias, int nbias, int f32, uintptr_t stream) {
+                            uintptr_t bias, int nbias, int keep, uintptr_t gate, long gate_ld, int f32,
+                            uintptr_t stream) {
   // tokens of the decode rows come first: one per sequence before seq0
   const int t0 = seq0;
   if (tokens <= t0) return;
@@ -840,16 +872,17 @@ void sm_window_attn_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintp
     DLLM_HOST_CHECK(bs > 0 && window >= 1 && chunk >= 0 && max_blocks > 0, "window attention sizes");
     DLLM_HOST_CHECK(pool == 0 || (pool > 0 && kp && vp && chunk == 0), "window attention averaged caches");
     DLLM_HOST_CHECK(!bias || (nbias >= 1 && pool == 0), "window attention distance bias");
+    DLLM_HOST_CHECK(keep >= 0 && (keep == 0 || pool == 0) && (!gate || gate_ld >= H), "window attention kept tokens / gate");
 #define WIN_TILE(NQK, NDV, QT)                                                                                     \
   do {                                                                                                             \
     if (bias)                                                                                                      \
       launch_tile<NQK, NDV, QT, true>(out, q, k_cache, v_cache, block_tables, max_blocks, cu, positions, seq0,     \
                                       seqs - seq0, max_q_len, H, G, D, Dv, bs, window, chunk, scale, sinks, softcap, kp, \
-                                      vp, pool, pbs, bias, nbias, stream);                                         \
+                                      vp, pool, pbs, bias, nbias, keep, gate, gate_ld, stream);                    \
     else                                                                                                           \
       launch_tile<NQK, NDV, QT, false>(out, q, k_cache, v_cache, block_tables, max_blocks, cu, positions, seq0,    \
                                        seqs - seq0, max_q_len, H, G, D, Dv, bs, window, chunk, scale, sinks, softcap, kp, \
-                                       vp, pool, pbs, 0, 0, stream);                                               \
+                                       vp, pool, pbs, 0, 0, keep, gate, gate_ld, stream);                          \
   } while (0)
     if (D <= 64 && Dv <= 64) WIN_TILE(2, 4, 1);
     else if (D <= 128 && Dv <= 128) WIN_TILE(4, 8, 1);
@@ -858,7 +891,7 @@ void sm_window_attn_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintp
     return;
   }
   launch_rows(out, q, k_cache, v_cache, block_tables, max_blocks, positions, tok_seq, t0, tokens - t0, H, G, D, Dv, bs,
-              window, chunk, scale, sinks, softcap, kp, vp, pool, pbs, bias, nbias, f32, stream);
+              window, chunk, scale, sinks, softcap, kp, vp, pool, pbs, bias, nbias, keep, gate, gate_ld, f32, stream);
 }
 
 }  // namespace dllm

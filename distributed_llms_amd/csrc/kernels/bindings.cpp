@@ -24,6 +24,7 @@ PYBIND11_MODULE(_C_kernels, m) {
   m.def("splitk_add_rms_norm", &dllm::splitk_add_rms_norm);
   m.def("splitk_reduce", &dllm::splitk_reduce);
   m.def("splitk_reduce_clipped", &dllm::splitk_reduce_clipped);
+  m.def("splitk_reduce_gelu", &dllm::splitk_reduce_gelu);
   m.def("gemm_wide", &dllm::gemm_wide);
   m.def("gemm_wide_fp8", &dllm::gemm_wide_fp8);
   m.def("quant_fp8_rows", &dllm::quant_fp8_rows);
@@ -45,6 +46,9 @@ PYBIND11_MODULE(_C_kernels, m) {
   m.def("paged_attention_prefill", &dllm::paged_attention_prefill);
   m.def("sm_embed_f32", &dllm::sm_embed_f32);
   m.def("sm_rms_norm", &dllm::sm_rms_norm);
+  m.def("sm_layer_norm", &dllm::sm_layer_norm);
+  m.def("sm_post_layer_norm_add", &dllm::sm_post_layer_norm_add);
+  m.def("sm_gelu_glu", &dllm::sm_gelu_glu);
   m.def("sm_post_norm_add", &dllm::sm_post_norm_add);
   m.def("sm_causal_conv", &dllm::sm_causal_conv);
   m.def("sm_rglru_gates", &dllm::sm_rglru_gates);

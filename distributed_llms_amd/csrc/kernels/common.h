@@ -89,6 +89,12 @@ __device__ __forceinline__ float clipped_glu_f(float g, float u, float limit) {
   return g * __builtin_amdgcn_rcpf(1.f + __expf(-kGluAlpha * g)) * (u + 1.0f);
 }
 
+// gelu (tanh form) of the gate times up, 0.5 (1 + tanh(z)) = 1 / (1 + e^(-2 z)): the epilogue form (rounded to bf16)
+__device__ __forceinline__ float gelu_glu_f(float g, float u) {
+  const float z2 = 1.5957691216057308f * (g + 0.044715f * g * g * g);
+  return g * __builtin_amdgcn_rcpf(1.f + __expf(-z2)) * u;
+}
+
 // f32 -> bf16 via the compiler cast: gfx950 emits v_cvt_pk_bf16_f32 (RNE, NaN-preserving).
 __device__ __forceinline__ bf16 f2bf(float x) { return (bf16)x; }
 __device__ __forceinline__ float bf2f(bf16 x) { return (float)x; }

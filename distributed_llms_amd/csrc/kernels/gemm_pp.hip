@@ -758,7 +758,7 @@ void gemm_pp_moe(uintptr_t y, uintptr_t x, uintptr_t gather, uintptr_t w, uintpt
 // w = (b % 8) (P / 8) + b / 8), so each XCD's L2 serves 32 consecutive tiles of the grouped order
 // (8 row tiles x 4 column tiles) at a time.
 // MODE 0: C bf16 [M, N];  2: SwiGLU C [M, N / 2] with B = [Bg; Bu] (row groups as pp_b_row);  4: the clipped GLU of
-// `limit` (common.h) in the same layout.
+// `limit` (common.h) in the same layout;  5: its gelu GLU.
 // SCH 8: nontemporal output stores (large SwiGLU outputs), else 0.  The schedule sweeps of rounds 3-5
 // (barrier positions, piece spacing, row-group widths, and the split A / B LDS release of round 5,
 // all within 0.5 % of this schedule: profiles/round5_raw/r5d_pf_sched.txt) were removed.
@@ -831,7 +831,7 @@ __global__ void __launch_bounds__(256, 1) gemm_pf_kernel(const bf16* __restrict_
   constexpr int RT = TM / 16, CT = TN / 16;            // 8 x 8 accumulators per wave
   constexpr int SLOT = (BM + BN) * PBK, NB = 2;        // 2 x 64 KiB ring
   constexpr int GA = BM * PBK * 2 / 1024 / NW, GB = BN * PBK * 2 / 1024 / NW, G = GA + GB;
-  constexpr bool CLIPPED = MODE == 4, SWIGLU = MODE == 2 || CLIPPED;
+  constexpr bool CLIPPED = MODE == 4, GELU = MODE == 5, SWIGLU = MODE == 2 || CLIPPED || GELU;
   constexpr int OUTW = SWIGLU ? BN / 2 : BN;           // output tile width (elements)
   typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
   typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
@@ -1066,7 +1066,8 @@ __global__ void __launch_bounds__(256, 1) gemm_pf_kernel(const bf16* __restrict_
         if constexpr (SWIGLU) {
           const f32x4 g = acc[r][2 * i], u = acc[r][2 * i + 1];
 #pragma unroll
-          for (int v = 0; v < 4; ++v) hq[v] = f2bf(CLIPPED ? clipped_glu_f(g[v], u[v], limit) : silu_f(g[v]) * u[v]);
+          for (int v = 0; v < 4; ++v)
+            hq[v] = f2bf(GELU ? gelu_glu_f(g[v], u[v]) : CLIPPED ? clipped_glu_f(g[v], u[v], limit) : silu_f(g[v]) * u[v]);
         } else {
 #pragma unroll
           for (int v = 0; v < 4; ++v) hq[v] = f2bf(acc[r][i][v]);
@@ -1134,7 +1135,7 @@ void gemm_pf(uintptr_t c, uintptr_t a, uintptr_t b, int M, int N, int K, int mod
   DLLM_HOST_CHECK(M >= 1, "M >= 1");
   DLLM_HOST_CHECK(K % PBK == 0 && K >= PBK, "K must be a positive multiple of 64");
   DLLM_HOST_CHECK(N % 256 == 0, "N must be a multiple of 256");
-  DLLM_HOST_CHECK(mode == 0 || mode == 1 || mode == 3, "mode 0 (plain), 1 (SwiGLU) or 3 (clipped GLU)");
+  DLLM_HOST_CHECK(mode == 0 || mode == 1 || mode == 3 || mode == 4, "mode 0 (plain), 1 (SwiGLU), 3 (clipped GLU) or 4 (gelu GLU)");
   DLLM_HOST_CHECK(variant == 0 || variant == 8, "variant 0 or 8 (nontemporal output stores)");
   // the output's byte range must stay below 2^31: rows past M are dropped by giving their stores
   // the offset 0x80000000, which has to lie outside the buffer's range
@@ -1161,6 +1162,10 @@ void gemm_pf(uintptr_t c, uintptr_t a, uintptr_t b, int M, int N, int K, int mod
   hipLaunchKernelGGL((gemm_pf_kernel<MODE_, SCH_, DYN_>), dim3((unsigned)grid), dim3(256), 0, s, (const bf16*)a, \
                      (const bf16*)b, (bf16*)c, M, N, K, q, limit)
   const bool nt_store = variant == 8 || (mode != 0 && (long)M * (N / 2) * 2 > (256L << 20));
+  if (mode == 4) {
+    if (dyn) { if (nt_store) DLLM_PF_GO(5, 8, true); else DLLM_PF_GO(5, 0, true); }
+    else { if (nt_store) DLLM_PF_GO(5, 8, false); else DLLM_PF_GO(5, 0, false); }
+  } else
   if (mode == 3) {
     if (dyn) { if (nt_store) DLLM_PF_GO(4, 8, true); else DLLM_PF_GO(4, 0, true); }
     else { if (nt_store) DLLM_PF_GO(4, 8, false); else DLLM_PF_GO(4, 0, false); }

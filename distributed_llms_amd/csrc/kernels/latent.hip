@@ -8,10 +8,10 @@
 // run.  The cache holds the latent in the two layouts those kernels read: k [NB, 1, BS, rank + rot_dim]
 // (row per key: latent | rotated part) and v [NB, 1, rank, BS] (transposed inside a block).
 //
-//   lat_prep       per token: RMS norm of the query latent -> cq; RMS norm of the key/value latent and
-//                  the interleaved-pair rotation of the shared key part, appended to both caches
+//   lat_prep       per token: RMS norm of the query latent (if there is one) -> cq; RMS norm of the key/value
+//                  latent and the rotation of the shared key part, appended to both caches
 //   lat_q_pack     per token: [H, T, rank] folded queries + the rotated part of q -> q~ [T, H, rank + rot_dim]
-//   lat_head_gate  [H, T, vdim] head outputs x sigmoid(gate[t, h]) -> [T, H * vdim]
+//   lat_head_gate  [H, T, vdim] head outputs x sigmoid(gate[t, h]) or sigmoid(gate[t, h, e]) -> [T, H * vdim]
 //   par_add        x += a (+ b) on the float32 stream, optionally also the stream rounded to T
 //   stream_cat     [x | x0] rounded to T (input of a projection of two streams); stream_set: x = (float)a
 //   side_gate      gelu_tanh(z) * table[token, off : off + dim]
@@ -27,12 +27,43 @@
 
 namespace dllm {
 
+// Pair i < ceil(rot_dim / 2) of a rotated part: elements (2i, 2i + 1), or -- half, for the nfreq turning pairs --
+// (i, i + nfreq); the pairs beyond those are the elements that do not turn.
+struct RotPair {
+  int a, b;
+};
+__device__ __forceinline__ RotPair rot_pair(int i, int nfreq, int half) {
+  return half && i < nfreq ? RotPair{i, i + nfreq} : RotPair{2 * i, 2 * i + 1};
+}
+
+// The pairs of one row's rotated part [rot_dim], pair i per lane and step: dst = src turned by pos * freqs
+template <typename T>
+__device__ __forceinline__ void rotate_row(T* __restrict__ dst, const T* __restrict__ src, int i, int rot_dim, int half,
+                                           const float* __restrict__ freqs, int nfreq, float pos) {
+  const RotPair p = rot_pair(i, nfreq, half);
+  const float u = ldf(src + p.a);
+  if (p.b >= rot_dim) {                                      // a last single element
+    stf(dst + p.a, u);
+    return;
+  }
+  const float v = ldf(src + p.b);
+  float a = u, b = v;
+  if (i < nfreq) {
+    const float ang = pos * freqs[i];
+    const float c = cosf(ang), s = sinf(ang);
+    a = u * c - v * s;
+    b = v * c + u * s;
+  }
+  stf(dst + p.a, a);
+  stf(dst + p.b, b);
+}
+
 // --------------------------------------------------------------------------- latent input stage
 template <typename T>
 __global__ void __launch_bounds__(256) lat_prep_kernel(
     void* __restrict__ cq_, const void* __restrict__ down_, long ld, int q_off, int q_rank,
     const void* __restrict__ qn_w_, int c_off, int rank, const void* __restrict__ cn_w_, int r_off, int rot_dim,
-    const float* __restrict__ freqs, int nfreq, const int32_t* __restrict__ positions,
+    int half, const float* __restrict__ freqs, int nfreq, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ slot_mapping, void* __restrict__ k_cache_, void* __restrict__ v_cache_, int bs,
     float eps) {
   __shared__ float red[16];
@@ -69,23 +100,12 @@ __global__ void __launch_bounds__(256) lat_prep_kernel(
     vblk[(size_t)i * bs] = c;
   }
   const float pos = (float)positions[t];
-  for (int i = tid; i < rot_dim / 2; i += 256) {
-    const float u = ldf(row + r_off + 2 * i), v = ldf(row + r_off + 2 * i + 1);
-    float a = u, b = v;
-    if (i < nfreq) {
-      const float ang = pos * freqs[i];
-      const float c = cosf(ang), s = sinf(ang);
-      a = u * c - v * s;
-      b = v * c + u * s;
-    }
-    stf(krow + rank + 2 * i, a);
-    stf(krow + rank + 2 * i + 1, b);
-  }
-  if ((rot_dim & 1) && tid == 0) krow[D - 1] = row[r_off + rot_dim - 1];
+  for (int i = tid; i < (rot_dim + 1) / 2; i += 256)
+    rotate_row<T>(krow + rank, row + r_off, i, rot_dim, half, freqs, nfreq, pos);
 }
 
 void lat_prep(uintptr_t cq, uintptr_t down, long ld, int q_off, int q_rank, uintptr_t qn_w, int c_off, int rank,
-              uintptr_t cn_w, int r_off, int rot_dim, uintptr_t freqs, int nfreq, uintptr_t positions,
+              uintptr_t cn_w, int r_off, int rot_dim, int half, uintptr_t freqs, int nfreq, uintptr_t positions,
               uintptr_t slot_mapping, uintptr_t k_cache, uintptr_t v_cache, int bs, float eps, int tokens, int f32,
               uintptr_t stream) {
   if (tokens <= 0) return;
@@ -96,7 +116,7 @@ void lat_prep(uintptr_t cq, uintptr_t down, long ld, int q_off, int q_rank, uint
   DLLM_HOST_CHECK((q_rank == 0 || (cq && qn_w)) && cn_w && k_cache && v_cache && (nfreq == 0 || freqs),
                   "latent arguments");
   SM_DISPATCH(f32, lat_prep_kernel, dim3(tokens), dim3(256), 0, stream, (void*)cq, (const void*)down, ld, q_off,
-              q_rank, (const void*)qn_w, c_off, rank, (const void*)cn_w, r_off, rot_dim, (const float*)freqs, nfreq,
+              q_rank, (const void*)qn_w, c_off, rank, (const void*)cn_w, r_off, rot_dim, half, (const float*)freqs, nfreq,
               (const int32_t*)positions, (const int32_t*)slot_mapping, (void*)k_cache, (void*)v_cache, bs, eps);
 }
 
@@ -106,14 +126,15 @@ void lat_prep(uintptr_t cq, uintptr_t down, long ld, int q_off, int q_rank, uint
 // rotation pairs of all heads, a pair per lane.
 template <typename T, int V>
 __global__ void __launch_bounds__(256) lat_q_pack_kernel(void* __restrict__ out_, const void* __restrict__ qa_,
-                                                         const void* __restrict__ q_, int tokens, int H, int rank,
-                                                         int dim, int rot_dim, const float* __restrict__ freqs,
-                                                         int nfreq, const int32_t* __restrict__ positions) {
+                                                         const void* __restrict__ q_, long ldq, int tokens, int H,
+                                                         int rank, int dim, int rot_dim, int half,
+                                                         const float* __restrict__ freqs, int nfreq,
+                                                         const int32_t* __restrict__ positions) {
   const int t = blockIdx.x;
   const int D = rank + rot_dim, dq = dim + rot_dim;
   T* out = (T*)out_ + (size_t)t * H * D;
   const T* qa = (const T*)qa_ + (size_t)t * rank;
-  const T* q = (const T*)q_ + (size_t)t * H * dq + dim;
+  const T* q = (const T*)q_ + (size_t)t * ldq + dim;
   const int cpr = rank / V;                                  // chunks per head
   for (int idx = threadIdx.x; idx < H * cpr; idx += 256) {
     const int h = idx / cpr, c = idx - h * cpr;
@@ -125,33 +146,18 @@ __global__ void __launch_bounds__(256) lat_q_pack_kernel(void* __restrict__ out_
   const int ppr = (rot_dim + 1) / 2;                         // pairs per head (a last single element counts as one)
   for (int idx = threadIdx.x; idx < H * ppr; idx += 256) {
     const int h = idx / ppr, i = idx - h * ppr;
-    const T* qr = q + h * dq + 2 * i;
-    T* o = out + h * D + rank + 2 * i;
-    const float u = ldf(qr);
-    if (2 * i + 1 >= rot_dim) {
-      stf(o, u);
-      continue;
-    }
-    const float w = ldf(qr + 1);
-    float a = u, b2 = w;
-    if (i < nfreq) {
-      const float ang = pos * freqs[i];
-      const float c = cosf(ang), s = sinf(ang);
-      a = u * c - w * s;
-      b2 = w * c + u * s;
-    }
-    stf(o, a);
-    stf(o + 1, b2);
+    rotate_row<T>(out + h * D + rank, q + h * dq, i, rot_dim, half, freqs, nfreq, pos);
   }
 }
 
-void lat_q_pack(uintptr_t out, uintptr_t qa, uintptr_t q, int tokens, int H, int rank, int dim, int rot_dim,
-                uintptr_t freqs, int nfreq, uintptr_t positions, int f32, uintptr_t stream) {
+void lat_q_pack(uintptr_t out, uintptr_t qa, uintptr_t q, long ldq, int tokens, int H, int rank, int dim, int rot_dim,
+                int half, uintptr_t freqs, int nfreq, uintptr_t positions, int f32, uintptr_t stream) {
   if (tokens <= 0) return;
   DLLM_HOST_CHECK(H > 0 && rank > 0 && dim >= 0 && rot_dim >= 0 && 2 * nfreq <= rot_dim, "latent query sizes");
-  DLLM_HOST_CHECK(out && qa && (rot_dim == 0 || q) && (nfreq == 0 || freqs), "latent query arguments");
+  DLLM_HOST_CHECK(out && qa && (rot_dim == 0 || q) && (nfreq == 0 || freqs) && ldq >= (long)H * (dim + rot_dim),
+                  "latent query arguments");
   SM_DISPATCH_V(f32, rank % 8 == 0 && rot_dim % 8 == 0, lat_q_pack_kernel, dim3(tokens), dim3(256), 0, stream,
-                (void*)out, (const void*)qa, (const void*)q, tokens, H, rank, dim, rot_dim, (const float*)freqs, nfreq,
+                (void*)out, (const void*)qa, (const void*)q, ldq, tokens, H, rank, dim, rot_dim, half, (const float*)freqs, nfreq,
                 (const int32_t*)positions);
 }
 
@@ -162,15 +168,15 @@ void lat_q_pack(uintptr_t out, uintptr_t qa, uintptr_t q, int tokens, int H, int
 // Consecutive threads own consecutive output columns, so every weight row is read in whole lines; the
 // token's vector sits in LDS as float; sums are float32.
 template <typename T>
-__global__ void __launch_bounds__(256) lat_q_fold_kernel(void* __restrict__ out_, const void* __restrict__ q_,
+__global__ void __launch_bounds__(256) lat_q_fold_kernel(void* __restrict__ out_, const void* __restrict__ q_, long ldq,
                                                          const void* __restrict__ wuk_, int H, int rank, int dim,
-                                                         int rot_dim, const float* __restrict__ freqs, int nfreq,
+                                                         int rot_dim, int half, const float* __restrict__ freqs, int nfreq,
                                                          const int32_t* __restrict__ positions) {
   extern __shared__ float qs[];                              // [dim]
   const int t = blockIdx.x, h = blockIdx.y;
   const int D = rank + rot_dim, dq = dim + rot_dim;
   T* out = (T*)out_ + ((size_t)t * H + h) * D;
-  const T* q = (const T*)q_ + ((size_t)t * H + h) * dq;
+  const T* q = (const T*)q_ + (size_t)t * ldq + h * dq;
   const T* w = (const T*)wuk_ + (size_t)h * dim * rank;
   for (int d = threadIdx.x; d < dim; d += 256) qs[d] = ldf(q + d);
   __syncthreads();
@@ -180,32 +186,15 @@ __global__ void __launch_bounds__(256) lat_q_fold_kernel(void* __restrict__ out_
     stf(out + j, acc);
   }
   const float pos = (float)positions[t];
-  for (int i = threadIdx.x; i < (rot_dim + 1) / 2; i += 256) {
-    const T* qr = q + dim + 2 * i;
-    T* o = out + rank + 2 * i;
-    const float u = ldf(qr);
-    if (2 * i + 1 >= rot_dim) {
-      stf(o, u);
-      continue;
-    }
-    const float v = ldf(qr + 1);
-    float a = u, b = v;
-    if (i < nfreq) {
-      const float ang = pos * freqs[i];
-      const float c = cosf(ang), s = sinf(ang);
-      a = u * c - v * s;
-      b = v * c + u * s;
-    }
-    stf(o, a);
-    stf(o + 1, b);
-  }
+  for (int i = threadIdx.x; i < (rot_dim + 1) / 2; i += 256)
+    rotate_row<T>(out + rank, q + dim, i, rot_dim, half, freqs, nfreq, pos);
 }
 
 // bf16 with 8 | rank: a thread owns 8 consecutive outputs (16-byte weight loads) and every ng-th input
 // row; the ng partial sums of an output meet in LDS.
 __global__ void __launch_bounds__(256) lat_q_fold_vec_kernel(bf16* __restrict__ out_, const bf16* __restrict__ q_,
-                                                             const bf16* __restrict__ wuk, int H, int rank, int dim,
-                                                             int rot_dim, const float* __restrict__ freqs, int nfreq,
+                                                             long ldq, const bf16* __restrict__ wuk, int H, int rank,
+                                                             int dim, int rot_dim, int half, const float* __restrict__ freqs, int nfreq,
                                                              const int32_t* __restrict__ positions, int ng) {
   extern __shared__ float sm[];
   float* qs = sm;                                            // [dim]
@@ -213,7 +202,7 @@ __global__ void __launch_bounds__(256) lat_q_fold_vec_kernel(bf16* __restrict__ 
   const int t = blockIdx.x, h = blockIdx.y;
   const int D = rank + rot_dim, dq = dim + rot_dim;
   bf16* out = out_ + ((size_t)t * H + h) * D;
-  const bf16* q = q_ + ((size_t)t * H + h) * dq;
+  const bf16* q = q_ + (size_t)t * ldq + h * dq;
   const bf16* w = wuk + (size_t)h * dim * rank;
   for (int d = threadIdx.x; d < dim; d += 256) qs[d] = bf2f(q[d]);
   __syncthreads();
@@ -236,54 +225,37 @@ __global__ void __launch_bounds__(256) lat_q_fold_vec_kernel(bf16* __restrict__ 
     out[j] = f2bf(s);
   }
   const float pos = (float)positions[t];
-  for (int i = threadIdx.x; i < (rot_dim + 1) / 2; i += 256) {
-    const bf16* qr = q + dim + 2 * i;
-    bf16* o = out + rank + 2 * i;
-    const float u = bf2f(qr[0]);
-    if (2 * i + 1 >= rot_dim) {
-      o[0] = f2bf(u);
-      continue;
-    }
-    const float v = bf2f(qr[1]);
-    float a = u, b = v;
-    if (i < nfreq) {
-      const float ang = pos * freqs[i];
-      const float cs = cosf(ang), sn = sinf(ang);
-      a = u * cs - v * sn;
-      b = v * cs + u * sn;
-    }
-    o[0] = f2bf(a);
-    o[1] = f2bf(b);
-  }
+  for (int i = threadIdx.x; i < (rot_dim + 1) / 2; i += 256)
+    rotate_row<bf16>(out + rank, q + dim, i, rot_dim, half, freqs, nfreq, pos);
 }
 
 // groups of input rows for the vector forms: as many as 256 threads allow, at most one per input row
 static int fold_groups(int out_width, int in_width) { return std::max(1, std::min(256 / (out_width / 8), in_width)); }
 
-void lat_q_fold(uintptr_t out, uintptr_t q, uintptr_t wuk, int tokens, int H, int rank, int dim, int rot_dim,
-                uintptr_t freqs, int nfreq, uintptr_t positions, int f32, uintptr_t stream) {
+void lat_q_fold(uintptr_t out, uintptr_t q, long ldq, uintptr_t wuk, int tokens, int H, int rank, int dim, int rot_dim,
+                int half, uintptr_t freqs, int nfreq, uintptr_t positions, int f32, uintptr_t stream) {
   if (tokens <= 0) return;
   DLLM_HOST_CHECK(H > 0 && H <= 65535 && rank > 0 && dim > 0 && dim <= 8192 && rot_dim >= 0 && 2 * nfreq <= rot_dim,
                   "latent query sizes");
-  DLLM_HOST_CHECK(out && q && wuk && (nfreq == 0 || freqs), "latent query arguments");
+  DLLM_HOST_CHECK(out && q && wuk && (nfreq == 0 || freqs) && ldq >= (long)H * (dim + rot_dim), "latent query arguments");
   if (!f32 && rank % 8 == 0 && rank <= 2048) {
     const int ng = fold_groups(rank, dim);
     hipLaunchKernelGGL(lat_q_fold_vec_kernel, dim3(tokens, H), dim3(256), sizeof(float) * ((size_t)dim + (size_t)ng * rank),
-                       (hipStream_t)stream, (bf16*)out, (const bf16*)q, (const bf16*)wuk, H, rank, dim, rot_dim,
+                       (hipStream_t)stream, (bf16*)out, (const bf16*)q, ldq, (const bf16*)wuk, H, rank, dim, rot_dim, half,
                        (const float*)freqs, nfreq, (const int32_t*)positions, ng);
     DLLM_HIP_CHECK(hipGetLastError());
     return;
   }
   SM_DISPATCH(f32, lat_q_fold_kernel, dim3(tokens, H), dim3(256), sizeof(float) * dim, stream, (void*)out,
-              (const void*)q, (const void*)wuk, H, rank, dim, rot_dim, (const float*)freqs, nfreq,
+              (const void*)q, ldq, (const void*)wuk, H, rank, dim, rot_dim, half, (const float*)freqs, nfreq,
               (const int32_t*)positions);
 }
 
 template <typename T>
 __global__ void __launch_bounds__(256) lat_v_unfold_kernel(void* __restrict__ out_, const void* __restrict__ o_,
                                                            const void* __restrict__ wuv_t_,
-                                                           const void* __restrict__ gate_, long ld, int H, int rank,
-                                                           int vdim) {
+                                                           const void* __restrict__ gate_, long ld, int wide, int H,
+                                                           int rank, int vdim) {
   extern __shared__ float os[];                              // [rank]
   const int t = blockIdx.x, h = blockIdx.y;
   T* out = (T*)out_ + ((size_t)t * H + h) * vdim;
@@ -292,8 +264,8 @@ __global__ void __launch_bounds__(256) lat_v_unfold_kernel(void* __restrict__ ou
   const T* gate = (const T*)gate_;
   for (int r = threadIdx.x; r < rank; r += 256) os[r] = ldf(o + r);
   __syncthreads();
-  const float g = gate ? 1.0f / (1.0f + expf(-ldf(gate + (size_t)t * ld + h))) : 1.0f;
   for (int e = threadIdx.x; e < vdim; e += 256) {
+    const float g = gate ? 1.0f / (1.0f + expf(-ldf(gate + (size_t)t * ld + (wide ? h * vdim + e : h)))) : 1.0f;
     float acc = 0.f;
     for (int r = 0; r < rank; ++r) acc = fmaf(os[r], ldf(w + (size_t)r * vdim + e), acc);
     // the product is rounded to the activation type before the gate, like the batched product it stands for
@@ -305,8 +277,8 @@ __global__ void __launch_bounds__(256) lat_v_unfold_kernel(void* __restrict__ ou
 
 __global__ void __launch_bounds__(256) lat_v_unfold_vec_kernel(bf16* __restrict__ out_, const bf16* __restrict__ o_,
                                                                const bf16* __restrict__ wuv_t,
-                                                               const bf16* __restrict__ gate, long ld, int H, int rank,
-                                                               int vdim, int ng) {
+                                                               const bf16* __restrict__ gate, long ld, int wide, int H,
+                                                               int rank, int vdim, int ng) {
   extern __shared__ float sm[];
   float* os = sm;                                            // [rank]
   float* red = sm + rank;                                    // [ng][vdim]
@@ -329,16 +301,17 @@ __global__ void __launch_bounds__(256) lat_v_unfold_vec_kernel(bf16* __restrict_
     for (int i = 0; i < 8; ++i) red[g * vdim + 8 * c + i] = acc[i];
   }
   __syncthreads();
-  const float gt = gate ? 1.0f / (1.0f + expf(-bf2f(gate[(size_t)t * ld + h]))) : 1.0f;
   for (int e = threadIdx.x; e < vdim; e += 256) {
+    const float gt = gate ? 1.0f / (1.0f + expf(-bf2f(gate[(size_t)t * ld + (wide ? h * vdim + e : h)]))) : 1.0f;
     float s = 0.f;
     for (int g2 = 0; g2 < ng; ++g2) s += red[g2 * vdim + e];
     out[e] = f2bf(bf2f(f2bf(s)) * gt);           // rounded before the gate, like the batched product it stands for
   }
 }
 
-void lat_v_unfold(uintptr_t out, uintptr_t o, uintptr_t wuv_t, uintptr_t gate, long ld, int tokens, int H, int rank,
-                  int vdim, int f32, uintptr_t stream) {
+// `wide`: one gate logit per output element (gate[t * ld + h * vdim + e]) instead of one per head (gate[t * ld + h])
+void lat_v_unfold(uintptr_t out, uintptr_t o, uintptr_t wuv_t, uintptr_t gate, long ld, int wide, int tokens, int H,
+                  int rank, int vdim, int f32, uintptr_t stream) {
   if (tokens <= 0) return;
   DLLM_HOST_CHECK(H > 0 && H <= 65535 && rank > 0 && rank <= 8192 && vdim > 0 && out && o && wuv_t,
                   "latent value arguments");
@@ -346,40 +319,48 @@ void lat_v_unfold(uintptr_t out, uintptr_t o, uintptr_t wuv_t, uintptr_t gate, l
     const int ng = fold_groups(vdim, rank);
     hipLaunchKernelGGL(lat_v_unfold_vec_kernel, dim3(tokens, H), dim3(256),
                        sizeof(float) * ((size_t)rank + (size_t)ng * vdim), (hipStream_t)stream, (bf16*)out,
-                       (const bf16*)o, (const bf16*)wuv_t, (const bf16*)gate, ld, H, rank, vdim, ng);
+                       (const bf16*)o, (const bf16*)wuv_t, (const bf16*)gate, ld, wide, H, rank, vdim, ng);
     DLLM_HIP_CHECK(hipGetLastError());
     return;
   }
   SM_DISPATCH(f32, lat_v_unfold_kernel, dim3(tokens, H), dim3(256), sizeof(float) * rank, stream, (void*)out,
-              (const void*)o, (const void*)wuv_t, (const void*)gate, ld, H, rank, vdim);
+              (const void*)o, (const void*)wuv_t, (const void*)gate, ld, wide, H, rank, vdim);
 }
 
-// out [T, H * vdim] = o [H, T, vdim] * sigmoid(gate[t * ld + h]) (gate null: a plain transposing copy);
-// one workgroup per (token, head)
+// out [T, H * vdim] = o [H, T, vdim] * sigmoid(gate[t * ld + h]) -- wide: * sigmoid(gate[t * ld + h * vdim + e]) --
+// (gate null: a plain transposing copy); one workgroup per (token, head)
 template <typename T, int V>
 __global__ void __launch_bounds__(64) lat_head_gate_kernel(void* __restrict__ out_, const void* __restrict__ o_,
-                                                           const void* __restrict__ gate_, long ld, int tokens, int H,
-                                                           int vdim) {
+                                                           const void* __restrict__ gate_, long ld, int wide,
+                                                           int tokens, int H, int vdim) {
   const int t = blockIdx.x, h = blockIdx.y;
   T* out = (T*)out_ + ((size_t)t * H + h) * vdim;
   const T* o = (const T*)o_ + ((size_t)h * tokens + t) * vdim;
   const T* gate = (const T*)gate_;
-  const float g = gate ? 1.0f / (1.0f + expf(-ldf(gate + (size_t)t * ld + h))) : 1.0f;
+  const float g = gate && !wide ? 1.0f / (1.0f + expf(-ldf(gate + (size_t)t * ld + h))) : 1.0f;
   for (int e = threadIdx.x * V; e < vdim; e += 64 * V) {
     float v[V];
     ldv<V>(o + e, v);
+    if (gate && wide) {
+      float z[V];
+      ldv<V>(gate + (size_t)t * ld + (size_t)h * vdim + e, z);
 #pragma unroll
-    for (int j = 0; j < V; ++j) v[j] *= g;
+      for (int j = 0; j < V; ++j) v[j] *= 1.0f / (1.0f + expf(-z[j]));
+    } else {
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] *= g;
+    }
     stv<V>(out + e, v);
   }
 }
 
-void lat_head_gate(uintptr_t out, uintptr_t o, uintptr_t gate, long ld, int tokens, int H, int vdim, int f32,
+void lat_head_gate(uintptr_t out, uintptr_t o, uintptr_t gate, long ld, int wide, int tokens, int H, int vdim, int f32,
                    uintptr_t stream) {
   if (tokens <= 0) return;
   DLLM_HOST_CHECK(H > 0 && H <= 65535 && vdim > 0 && out && o, "head gate arguments");
-  SM_DISPATCH_V(f32, vdim % 8 == 0, lat_head_gate_kernel, dim3(tokens, H), dim3(64), 0, stream, (void*)out,
-                (const void*)o, (const void*)gate, ld, tokens, H, vdim);
+  const bool vec = vdim % 8 == 0 && (!wide || (ld % 8 == 0 && gate % (f32 ? 32 : 16) == 0));
+  SM_DISPATCH_V(f32, vec, lat_head_gate_kernel, dim3(tokens, H), dim3(64), 0, stream, (void*)out, (const void*)o,
+                (const void*)gate, ld, wide, tokens, H, vdim);
 }
 
 // --------------------------------------------------------------------------- parallel layer: x += a + b

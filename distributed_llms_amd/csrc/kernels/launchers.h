@@ -28,6 +28,7 @@ void splitk_reduce(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M, in
 void splitk_reduce_ex(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M, int N, int act, uintptr_t stream,
                       float limit = 0.f);
 void splitk_reduce_clipped(uintptr_t out, uintptr_t ws, int S, int M, int N, float limit, uintptr_t stream);
+void splitk_reduce_gelu(uintptr_t out, uintptr_t ws, int S, int M, int N, uintptr_t stream);
 int gemm_wide(uintptr_t c, uintptr_t a, uintptr_t b, uintptr_t ws, long ws_floats, int M, int N, int K, int splits,
               int mode, int variant, uintptr_t stream);
 int gemm_wide_fp8(uintptr_t c, uintptr_t a, uintptr_t a_scale, uintptr_t b, uintptr_t b_scale, uintptr_t ws,
@@ -71,8 +72,14 @@ void paged_attention_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uint
 
 // ---- layer-list models with per-sequence state (seqmix.hip, attention_window.hip); f32: activations
 // are float (else bf16)
-void sm_embed_f32(uintptr_t out, uintptr_t ids, uintptr_t table, int tokens, int width, int vocab, int f32,
+void sm_embed_f32(uintptr_t out, uintptr_t ids, uintptr_t table, int tokens, int width, int vocab, float scale, int f32,
                   uintptr_t stream);
+void sm_layer_norm(uintptr_t y, uintptr_t x, uintptr_t w, uintptr_t b, int rows, int width, float eps, int f32,
+                   uintptr_t stream);
+void sm_post_layer_norm_add(uintptr_t x, uintptr_t o, int parts, uintptr_t bias, uintptr_t w_post, uintptr_t b_post,
+                            uintptr_t w_next, uintptr_t b_next, uintptr_t h, int rows, int width, float eps, int f32,
+                            uintptr_t stream);
+void sm_gelu_glu(uintptr_t out, uintptr_t gu, int tokens, int F, int f32, uintptr_t stream);
 void sm_embed_norm(uintptr_t x, uintptr_t h, uintptr_t ids, uintptr_t table, uintptr_t w, int tokens, int width,
                    int vocab, float eps, float offset, float scale, uintptr_t pos_table, uintptr_t positions,
                    int max_pos, int f32, uintptr_t stream);
@@ -127,7 +134,8 @@ void sm_softcap(uintptr_t out, uintptr_t x, long n, float cap, float scale, int 
 void sm_head_norm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_t q_norm, uintptr_t k_norm,
                        uintptr_t freqs, int nrot, int norm_last, float eps, uintptr_t q_mul, float temp_coef, int temp_every,
                        uintptr_t k_cache, uintptr_t v_cache, uintptr_t slot_mapping, uintptr_t positions, int tokens, int H,
-                       int G, int D, int Dv, int bs, int f32, uintptr_t stream);
+                       int G, int D, int Dv, int bs, uintptr_t bias, uintptr_t v_in, uintptr_t v_out, float lam, int f32,
+                       uintptr_t stream);
 void sm_attn_prep(uintptr_t q_out, uintptr_t qkv, uintptr_t conv_w, uintptr_t state, uintptr_t q_norm,
                   uintptr_t k_norm, uintptr_t freqs, int nrot, float mag, float eps, uintptr_t k_cache,
                   uintptr_t v_cache, uintptr_t slot_mapping, uintptr_t cu, uintptr_t positions, uintptr_t tok_seq,
@@ -136,29 +144,30 @@ void sm_attn_prep(uintptr_t q_out, uintptr_t qkv, uintptr_t conv_w, uintptr_t st
 void sm_rownorm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_t q_norm, uintptr_t k_norm,
                      uintptr_t freqs, int nrot, float eps, uintptr_t k_cache, uintptr_t v_cache, uintptr_t slot_mapping,
                      uintptr_t positions, int tokens, int H, int G, int D, int Dv, int bs, float mag, int v_from_k,
-                     int f32, uintptr_t stream);
+                     uintptr_t bias, uintptr_t v_in, uintptr_t v_out, float lam, int f32, uintptr_t stream);
 void sm_window_attn_decode(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                            int max_blocks, uintptr_t positions, uintptr_t tok_seq, int rows, int H, int G, int D,
                            int Dv, int bs, int window, int chunk, float scale, uintptr_t sinks, int splits, uintptr_t ws,
-                           float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int f32,
-                           uintptr_t stream);
+                           float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs, uintptr_t bias, int nbias, int keep,
+                           uintptr_t gate, long gate_ld, int f32, uintptr_t stream);
 void sm_window_attn_prefill(uintptr_t out, uintptr_t q, uintptr_t k_cache, uintptr_t v_cache, uintptr_t block_tables,
                             int max_blocks, uintptr_t cu, uintptr_t positions, uintptr_t tok_seq, int seq0, int seqs,
                             int tokens, int max_q_len, int H, int G, int D, int Dv, int bs, int window, int chunk,
                             float scale, uintptr_t sinks, float softcap, uintptr_t kp, uintptr_t vp, int pool, int pbs,
-                            uintptr_t bias, int nbias, int f32, uintptr_t stream);
+                            uintptr_t bias, int nbias, int keep, uintptr_t gate, long gate_ld, int f32,
+                            uintptr_t stream);
 // latent attention input stage and parallel layers on a float32 stream (latent.hip)
 void lat_prep(uintptr_t cq, uintptr_t down, long ld, int q_off, int q_rank, uintptr_t qn_w, int c_off, int rank,
-              uintptr_t cn_w, int r_off, int rot_dim, uintptr_t freqs, int nfreq, uintptr_t positions,
+              uintptr_t cn_w, int r_off, int rot_dim, int half, uintptr_t freqs, int nfreq, uintptr_t positions,
               uintptr_t slot_mapping, uintptr_t k_cache, uintptr_t v_cache, int bs, float eps, int tokens, int f32,
               uintptr_t stream);
-void lat_q_pack(uintptr_t out, uintptr_t qa, uintptr_t q, int tokens, int H, int rank, int dim, int rot_dim,
-                uintptr_t freqs, int nfreq, uintptr_t positions, int f32, uintptr_t stream);
-void lat_q_fold(uintptr_t out, uintptr_t q, uintptr_t wuk, int tokens, int H, int rank, int dim, int rot_dim,
-                uintptr_t freqs, int nfreq, uintptr_t positions, int f32, uintptr_t stream);
-void lat_v_unfold(uintptr_t out, uintptr_t o, uintptr_t wuv_t, uintptr_t gate, long ld, int tokens, int H, int rank,
-                  int vdim, int f32, uintptr_t stream);
-void lat_head_gate(uintptr_t out, uintptr_t o, uintptr_t gate, long ld, int tokens, int H, int vdim, int f32,
+void lat_q_pack(uintptr_t out, uintptr_t qa, uintptr_t q, long ldq, int tokens, int H, int rank, int dim, int rot_dim,
+                int half, uintptr_t freqs, int nfreq, uintptr_t positions, int f32, uintptr_t stream);
+void lat_q_fold(uintptr_t out, uintptr_t q, long ldq, uintptr_t wuk, int tokens, int H, int rank, int dim, int rot_dim,
+                int half, uintptr_t freqs, int nfreq, uintptr_t positions, int f32, uintptr_t stream);
+void lat_v_unfold(uintptr_t out, uintptr_t o, uintptr_t wuv_t, uintptr_t gate, long ld, int wide, int tokens, int H,
+                  int rank, int vdim, int f32, uintptr_t stream);
+void lat_head_gate(uintptr_t out, uintptr_t o, uintptr_t gate, long ld, int wide, int tokens, int H, int vdim, int f32,
                    uintptr_t stream);
 void par_add(uintptr_t x, uintptr_t a, uintptr_t b, uintptr_t x_rounded, long n, int f32, uintptr_t stream);
 void stream_cat(uintptr_t out, uintptr_t x, uintptr_t x0, int rows, int width, int f32, uintptr_t stream);

@@ -5,8 +5,9 @@
 // projection norm + half-split rotation + paged append; per-head norm before or after a paired rotation, with query
 // factors, + paged append), embedding (+ learned positions) + norm, the close of
 // pre-norm sublayers (one or two outputs, each normed apart), a token shift whose previous row lives in a state
-// slot, the entry of a looped span, the averaged keys / values of blocks of positions, a clipped GLU and the
-// logit soft cap.
+// slot, the entry of a looped span, sublayers between two layer norms, the averaged keys / values of blocks of
+// positions, clipped and gelu GLUs and the logit soft cap.  The attention input stages take projection biases and
+// values shared between layers.
 //
 // Every kernel is a template over the activation type T (bf16 or float): the float32 build is the
 // exact path (true 32-bit everywhere), the bf16 build keeps in float32 what feeds a norm, a
@@ -23,21 +24,22 @@ namespace dllm {
 // --------------------------------------------------------------------------- embedding -> f32
 template <typename T>
 __global__ void __launch_bounds__(256) sm_embed_kernel(float* __restrict__ out, const int32_t* __restrict__ ids,
-                                                       const void* __restrict__ table_, int width, int vocab) {
+                                                       const void* __restrict__ table_, int width, int vocab,
+                                                       float scale) {
   const T* table = (const T*)table_;
   int id = ids[blockIdx.x];
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
   const T* src = table + (size_t)id * width;
   float* dst = out + (size_t)blockIdx.x * width;
-  for (int i = threadIdx.x; i < width; i += 256) dst[i] = ldf(src + i);
+  for (int i = threadIdx.x; i < width; i += 256) dst[i] = ldf(src + i) * scale;
 }
 
-void sm_embed_f32(uintptr_t out, uintptr_t ids, uintptr_t table, int tokens, int width, int vocab, int f32,
+void sm_embed_f32(uintptr_t out, uintptr_t ids, uintptr_t table, int tokens, int width, int vocab, float scale, int f32,
                   uintptr_t stream) {
   if (tokens <= 0) return;
   DLLM_HOST_CHECK(width > 0 && vocab > 0, "embed sizes");
   SM_DISPATCH(f32, sm_embed_kernel, dim3(tokens), dim3(256), 0, stream, (float*)out, (const int32_t*)ids,
-              (const void*)table, width, vocab);
+              (const void*)table, width, vocab, scale);
 }
 
 // --------------------------------------------------------------------------- embedding + RMS norm -> f32 stream
@@ -212,6 +214,176 @@ void sm_post_norm_add(uintptr_t x, uintptr_t o, uintptr_t bias, uintptr_t w_post
   SM_DISPATCH_V(f32, width % 8 == 0, sm_post_norm_add_kernel, dim3(rows), dim3(256), 0, stream, (float*)x,
                 (const void*)o, (const void*)bias, (const void*)w_post, (const void*)w_next, (void*)h, width, eps, mult,
                 offset, (const void*)o2, s1, s2);
+}
+
+// --------------------------------------------------------------------------- layer norms on the float32 stream
+// One workgroup per row, the row in registers (NV pieces of V consecutive elements per lane): the mean first, then the
+// mean of the squared deviations from it.
+template <int V, int NV>
+__device__ __forceinline__ void ln_stats(const float (&v)[NV][V], int width, float eps, float* red, float& mean, float& inv) {
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  float s = 0.f;
+#pragma unroll
+  for (int k = 0; k < NV; ++k)
+#pragma unroll
+    for (int j = 0; j < V; ++j) s += v[k][j];                          // places beyond the row hold 0
+  s = wave_sum(s);
+  if (lane == 0) red[wid] = s;
+  __syncthreads();
+  mean = (red[0] + red[1] + red[2] + red[3]) / (float)width;
+  float q = 0.f;
+#pragma unroll
+  for (int k = 0; k < NV; ++k)
+    if ((k * 256 + (int)threadIdx.x) * V < width) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) q += (v[k][j] - mean) * (v[k][j] - mean);
+    }
+  q = wave_sum(q);
+  if (lane == 0) red[4 + wid] = q;
+  __syncthreads();
+  inv = 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)width + eps);
+}
+
+template <typename T, int V, int NV>
+__global__ void __launch_bounds__(256) sm_layer_norm_kernel(void* __restrict__ y_, const float* __restrict__ x,
+                                                            const void* __restrict__ w_, const void* __restrict__ b_,
+                                                            int width, float eps) {
+  __shared__ float red[8];
+  const float* xr = x + (size_t)blockIdx.x * width;
+  float v[NV][V], w[NV][V], b[NV][V];
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = (k * 256 + threadIdx.x) * V;
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[k][j] = 0.f;
+    if (i < width) {
+      ldv<V>(xr + i, v[k]);
+      ldv<V>((const T*)w_ + i, w[k]);
+      ldv<V>((const T*)b_ + i, b[k]);
+    }
+  }
+  float mean, inv;
+  ln_stats<V, NV>(v, width, eps, red, mean, inv);
+  T* y = (T*)y_ + (size_t)blockIdx.x * width;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = (k * 256 + threadIdx.x) * V;
+    if (i < width) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[k][j] = (v[k][j] - mean) * inv * w[k][j] + b[k][j];
+      stv<V>(y + i, v[k]);
+    }
+  }
+}
+
+// The close of a sublayer between two layer norms: x += layer_norm(o + bias) (weight wp, bias bp; `bias` null: none), and
+// with wn: h = layer_norm(x) (wn, bn), the next sublayer's input.  parts > 0: o is the sum of that many split-K slabs
+// [rows, width] (common.h part_load; bf16 results, rounded as the reduction of a split product rounds them).
+template <typename T, int V, int NV>
+__global__ void __launch_bounds__(256) sm_post_layer_norm_kernel(
+    float* __restrict__ x, const void* __restrict__ o_, int parts, const void* __restrict__ bias_,
+    const void* __restrict__ wp_, const void* __restrict__ bp_, const void* __restrict__ wn_, const void* __restrict__ bn_,
+    void* __restrict__ h_, int width, float eps) {
+  __shared__ float red[16];
+  const size_t row = (size_t)blockIdx.x * width;
+  float* xr = x + row;
+  float v[NV][V], xv[NV][V], w[NV][V], b[NV][V];
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = (k * 256 + threadIdx.x) * V;
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[k][j] = xv[k][j] = 0.f;
+    if (i < width) {
+      if (V == 4 && parts > 0) {
+        const float* P = (const float*)o_;
+        const size_t slab = (size_t)gridDim.x * width;
+        f32x4 a = {0.f, 0.f, 0.f, 0.f};
+        for (int s = 0; s < parts; ++s) a += part_load4<true>(P, s * slab + row + i);
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[k][j] = bf2f(f2bf(a[j & 3]));
+      } else {
+        ldv<V>((const T*)o_ + row + i, v[k]);
+      }
+      ldv<V>(xr + i, xv[k]);
+      ldv<V>((const T*)wp_ + i, w[k]);
+      ldv<V>((const T*)bp_ + i, b[k]);
+      if (bias_) {
+        float c[V];
+        ldv<V>((const T*)bias_ + i, c);
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[k][j] += c[j];
+      }
+    }
+  }
+  float mean, inv;
+  ln_stats<V, NV>(v, width, eps, red, mean, inv);
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = (k * 256 + threadIdx.x) * V;
+    if (i < width) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) xv[k][j] += (v[k][j] - mean) * inv * w[k][j] + b[k][j];
+      stv<V>(xr + i, xv[k]);
+      if (wn_) {
+        ldv<V>((const T*)wn_ + i, w[k]);
+        ldv<V>((const T*)bn_ + i, b[k]);
+      }
+    }
+  }
+  if (!wn_) return;
+  ln_stats<V, NV>(xv, width, eps, red + 8, mean, inv);
+  T* h = (T*)h_ + row;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = (k * 256 + threadIdx.x) * V;
+    if (i < width) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) xv[k][j] = (xv[k][j] - mean) * inv * w[k][j] + b[k][j];
+      stv<V>(h + i, xv[k]);
+    }
+  }
+}
+
+// V = 4 elements per lane and piece (width a multiple of 4), else one; the fewest pieces that hold the row
+#define SM_LN_DISPATCH(f32, width, KERNEL, grid, stream, ...)                                                        \
+  do {                                                                                                             \
+    DLLM_HOST_CHECK((width) > 0 && (width) <= 16384, "layer norm width");                                          \
+    const int np_ = ((width) + ((width) % 4 ? 255 : 1023)) / ((width) % 4 ? 256 : 1024);                           \
+    if ((width) % 4 == 0) {                                                                                        \
+      if (np_ <= 1) SM_LN_GO(f32, KERNEL, 4, 1, grid, stream, __VA_ARGS__);                                        \
+      else if (np_ <= 2) SM_LN_GO(f32, KERNEL, 4, 2, grid, stream, __VA_ARGS__);                                   \
+      else if (np_ <= 3) SM_LN_GO(f32, KERNEL, 4, 3, grid, stream, __VA_ARGS__);                                   \
+      else if (np_ <= 4) SM_LN_GO(f32, KERNEL, 4, 4, grid, stream, __VA_ARGS__);                                   \
+      else if (np_ <= 8) SM_LN_GO(f32, KERNEL, 4, 8, grid, stream, __VA_ARGS__);                                   \
+      else SM_LN_GO(f32, KERNEL, 4, 16, grid, stream, __VA_ARGS__);                                                \
+    } else if (np_ <= 4) SM_LN_GO(f32, KERNEL, 1, 4, grid, stream, __VA_ARGS__);                                   \
+    else if (np_ <= 16) SM_LN_GO(f32, KERNEL, 1, 16, grid, stream, __VA_ARGS__);                                   \
+    else SM_LN_GO(f32, KERNEL, 1, 64, grid, stream, __VA_ARGS__);                                                  \
+    DLLM_HIP_CHECK(hipGetLastError());                                                                             \
+  } while (0)
+#define SM_LN_GO(f32, KERNEL, V, NV, grid, stream, ...)                                                              \
+  do {                                                                                                             \
+    if (f32) hipLaunchKernelGGL(HIP_KERNEL_NAME(KERNEL<float, V, NV>), grid, dim3(256), 0, (hipStream_t)(stream), __VA_ARGS__); \
+    else hipLaunchKernelGGL(HIP_KERNEL_NAME(KERNEL<bf16, V, NV>), grid, dim3(256), 0, (hipStream_t)(stream), __VA_ARGS__);      \
+  } while (0)
+
+void sm_layer_norm(uintptr_t y, uintptr_t x, uintptr_t w, uintptr_t b, int rows, int width, float eps, int f32,
+                   uintptr_t stream) {
+  if (rows <= 0) return;
+  DLLM_HOST_CHECK(y && x && w && b, "layer norm arguments");
+  SM_LN_DISPATCH(f32, width, sm_layer_norm_kernel, dim3(rows), stream, (void*)y, (const float*)x, (const void*)w,
+                 (const void*)b, width, eps);
+}
+
+void sm_post_layer_norm_add(uintptr_t x, uintptr_t o, int parts, uintptr_t bias, uintptr_t w_post, uintptr_t b_post,
+                            uintptr_t w_next, uintptr_t b_next, uintptr_t h, int rows, int width, float eps, int f32,
+                            uintptr_t stream) {
+  if (rows <= 0) return;
+  DLLM_HOST_CHECK(x && o && w_post && b_post && (!w_next || (b_next && h)), "post_layer_norm_add arguments");
+  DLLM_HOST_CHECK(parts >= 0 && (parts == 0 || (!f32 && width % 4 == 0)), "post_layer_norm_add slabs");
+  SM_LN_DISPATCH(f32, width, sm_post_layer_norm_kernel, dim3(rows), stream, (float*)x, (const void*)o, parts,
+                 (const void*)bias, (const void*)w_post, (const void*)b_post, (const void*)w_next, (const void*)b_next,
+                 (void*)h, width, eps);
 }
 
 // --------------------------------------------------------------------------- entry of a looped span
@@ -944,6 +1116,35 @@ void sm_clipped_glu(uintptr_t out, uintptr_t gu, uintptr_t bias, int tokens, int
                 (void*)out, (const void*)gu, (const void*)bias, F, limit, alpha);
 }
 
+// --------------------------------------------------------------------------- gelu GLU
+// out [T, F] = gelu_tanh(gate) * up of a fused gate | up projection
+template <typename T, int V>
+__global__ void __launch_bounds__(256) sm_gelu_glu_kernel(void* __restrict__ out_, const void* __restrict__ gu_, int F) {
+  const T* gu = (const T*)gu_ + (size_t)blockIdx.x * 2 * F;
+  T* out = (T*)out_ + (size_t)blockIdx.x * F;
+  for (int c = (blockIdx.y * 256 + threadIdx.x) * V; c < F; c += gridDim.y * 256 * V) {
+    float g[V], u[V];
+    ldv<V>(gu + c, g);
+    ldv<V>(gu + F + c, u);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      // 0.5 (1 + tanh(z)) = 1 / (1 + e^(-2 z))
+      const float z = 0.7978845608028654f * (g[j] + 0.044715f * g[j] * g[j] * g[j]);
+      g[j] = g[j] / (1.0f + expf(-2.0f * z)) * u[j];
+    }
+    stv<V>(out + c, g);
+  }
+}
+
+void sm_gelu_glu(uintptr_t out, uintptr_t gu, int tokens, int F, int f32, uintptr_t stream) {
+  if (tokens <= 0 || F <= 0) return;
+  DLLM_HOST_CHECK(out && gu, "gelu_glu arguments");
+  const int vec = F % 8 == 0;
+  const int per = 256 * (vec ? 8 : 1);
+  SM_DISPATCH_V(f32, vec, sm_gelu_glu_kernel, dim3(tokens, std::min(16, (F + per - 1) / per)), dim3(256), 0, stream,
+                (void*)out, (const void*)gu, F);
+}
+
 // --------------------------------------------------------------------------- logit soft cap
 template <typename T>
 __global__ void __launch_bounds__(256) sm_softcap_kernel(float* __restrict__ out, const void* __restrict__ x_, long n,
@@ -1143,6 +1344,32 @@ void sm_attn_prep(uintptr_t q_out, uintptr_t qkv, uintptr_t conv_w, uintptr_t st
     launch_conv_state(state, qkv, (long)C, cu, positions, slots, seqs, C, taps, f32, C % 8 == 0, stream);
 }
 
+// --------------------------------------------------------------------------- values of an attention input stage
+template <typename T> __device__ __forceinline__ void add8(float (&x)[8], const T* p) {
+  float b[8];
+  ldv<8>(p, b);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) x[i] += b[i];
+}
+
+// Appends one token's values v [G Dv] (+ vb, when given) to the transposed cache; with v_in (another layer's values of the
+// token) v <- (1 - lam) v + lam v_in first; with v_out the values are also written there, row-major.  float32 arithmetic.
+template <typename T>
+__device__ __forceinline__ void append_values(const T* __restrict__ v, const T* __restrict__ vb, const T* __restrict__ v_in,
+                                              T* __restrict__ v_out, float lam, T* __restrict__ vc, int blk, int off, int G,
+                                              int Dv, int bs) {
+  for (int e = threadIdx.x; e < G * Dv; e += blockDim.x) {
+    const int g = e / Dv, c = e - g * Dv;
+    float x = ldf(v + e);
+    if (vb) x += ldf(vb + e);
+    if (v_in) x = (1.0f - lam) * x + lam * ldf(v_in + e);
+    T y;
+    stf(&y, x);
+    if (v_out) v_out[e] = y;
+    vc[(((size_t)blk * G + g) * Dv + c) * bs + off] = y;
+  }
+}
+
 // --------------------------------------------------------------------------- attention input: row norm + half-split rotation + append
 // From a fused projection row [.. | q (H D) | k (G D) | v (G Dv) | ..] (row stride ld, q at column `col0`):
 // an RMS norm over the WHOLE q projection and over the whole k projection (all heads at once, plain
@@ -1150,14 +1377,16 @@ void sm_attn_prep(uintptr_t q_out, uintptr_t qkv, uintptr_t conv_w, uintptr_t st
 // dimensions of every head: dimension i < nrot is paired with dimension i + nrot, the pair turns by
 // float(pos) * freqs[i] (cos and sin times `mag`).  q goes to q_out [T, H, D]; k and v (unchanged) are appended
 // at slot_mapping to caches k [NB, G, BS, D] / v [NB, G, Dv, BS].  `v_from_k`: the row has no v columns and
-// the values are the k columns as projected, before norm and rotation (Dv = D).
+// the values are the k columns as projected, before norm and rotation (Dv = D).  `pb` (or null): biases of the projected
+// q | k | v columns, added before anything else; v_in / v_out / lam: values shared between layers (append_values).
 // One workgroup per token; norms, angles and the rotation are float32.
 template <typename T>
 __global__ void __launch_bounds__(256) sm_rownorm_rope_kernel(
     void* __restrict__ q_out_, const void* __restrict__ qkv_, long ld, int col0, const void* __restrict__ qw_,
     const void* __restrict__ kw_, const float* __restrict__ freqs, int nrot, float eps, void* __restrict__ k_cache_,
     void* __restrict__ v_cache_, const int32_t* __restrict__ slot_mapping, const int32_t* __restrict__ positions, int H,
-    int G, int D, int Dv, int bs, float mag, int v_from_k) {
+    int G, int D, int Dv, int bs, float mag, int v_from_k, const void* __restrict__ pb_, const void* __restrict__ v_in_,
+    void* __restrict__ v_out_, float lam) {
   __shared__ float red[16];
   extern __shared__ float csn[];                   // cos | sin of the token's nrot angles
   const int t = blockIdx.x, tid = threadIdx.x;
@@ -1173,11 +1402,14 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_kernel(
   const T* qw = (const T*)qw_;
   const T* kw = (const T*)kw_;
   const int nq = H * D, nk = G * D, nv = G * Dv;
+  const T* qb = (const T*)pb_;
+  const T* kb = qb ? qb + nq : nullptr;
+  auto at = [](const T* p, const T* b, int e) { return b ? ldf(p + e) + ldf(b + e) : ldf(p + e); };
   float iq = 1.f, ik = 1.f;
   if (qw) {
     float sq = 0.f, sk = 0.f;
-    for (int e = tid; e < nq; e += 256) { const float x = ldf(q + e); sq += x * x; }
-    for (int e = tid; e < nk; e += 256) { const float x = ldf(k + e); sk += x * x; }
+    for (int e = tid; e < nq; e += 256) { const float x = at(q, qb, e); sq += x * x; }
+    for (int e = tid; e < nk; e += 256) { const float x = at(k, kb, e); sk += x * x; }
     sq = block_sum(sq, red);
     sk = block_sum(sk, red);
     iq = 1.0f / sqrtf(sq / (float)nq + eps), ik = 1.0f / sqrtf(sk / (float)nk + eps);
@@ -1192,15 +1424,16 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_kernel(
     const bool isq = e < nq;
     const int ee = isq ? e : e - nq;
     const T* src = isq ? q : k;
+    const T* sb = isq ? qb : kb;
     const T* w = isq ? qw : kw;
     const float inv = isq ? iq : ik;
     const int hd = ee / D, d = ee - hd * D;
-    float x = ldf(src + ee);
+    float x = at(src, sb, ee);
     if (w) x = x * inv * ldf(w + ee);
     if (d < 2 * nrot) {
       const int i = d < nrot ? d : d - nrot;
       const int pe = d < nrot ? ee + nrot : ee - nrot;          // the pair's other dimension
-      float y = ldf(src + pe);
+      float y = at(src, sb, pe);
       if (w) y = y * inv * ldf(w + pe);
       const float cs = csn[i], sn = csn[nrot + i];
       x = d < nrot ? x * cs - y * sn : x * cs + y * sn;
@@ -1208,10 +1441,8 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_kernel(
     if (isq) stf(q_out + ee, x);
     else stf(kc + (((size_t)blk * G + hd) * bs + off) * D + d, x);
   }
-  for (int e = tid; e < nv; e += 256) {
-    const int g = e / Dv, c = e - g * Dv;
-    vc[(((size_t)blk * G + g) * Dv + c) * bs + off] = v[e];
-  }
+  append_values<T>(v, kb ? kb + nk : nullptr, v_in_ ? (const T*)v_in_ + (size_t)t * nv : nullptr,
+                   v_out_ ? (T*)v_out_ + (size_t)t * nv : nullptr, lam, vc, blk, off, G, Dv, bs);
 }
 
 // The same with 8 consecutive dimensions per lane (16-byte loads and stores for bf16): head size, rotated
@@ -1222,7 +1453,8 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
     void* __restrict__ q_out_, const void* __restrict__ qkv_, long ld, int col0, const void* __restrict__ qw_,
     const void* __restrict__ kw_, const float* __restrict__ freqs, int nrot, float eps, void* __restrict__ k_cache_,
     void* __restrict__ v_cache_, const int32_t* __restrict__ slot_mapping, const int32_t* __restrict__ positions, int H,
-    int G, int D, int Dv, int bs, float mag, int v_from_k) {
+    int G, int D, int Dv, int bs, float mag, int v_from_k, const void* __restrict__ pb_, const void* __restrict__ v_in_,
+    void* __restrict__ v_out_, float lam) {
   __shared__ float red[32];
   extern __shared__ float csn[];                   // cos | sin of the token's nrot angles
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
@@ -1235,12 +1467,14 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
   const T* q = (const T*)qkv_ + (size_t)t * ld + col0;
   const int nq = H * D, nk = G * D, nv = G * Dv;
   const T* v = v_from_k ? q + nq : q + nq + nk;
+  const T* pb = (const T*)pb_;
   const bool normed = qw_ != nullptr;
   float sq = 0.f, sk = 0.f;
   if (normed) {
     for (int e = tid * 8; e < nq + nk; e += 2048) {
       float x[8];
       ldv<8>(q + e, x);
+      if (pb) add8(x, pb + e);
       float a = 0.f;
 #pragma unroll
       for (int i = 0; i < 8; ++i) a += x[i] * x[i];
@@ -1269,6 +1503,7 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
     const int hd = ee / D, d = ee - hd * D;
     float x[8], g[8];
     ldv<8>(q + e, x);
+    if (pb) add8(x, pb + e);
     if (normed) {
       ldv<8>(w, g);
 #pragma unroll
@@ -1279,6 +1514,7 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
       const int po = first ? nrot : -nrot, i0 = first ? d : d - nrot;
       float y[8], gy[8];
       ldv<8>(q + e + po, y);
+      if (pb) add8(y, pb + e + po);
       if (normed) {
         ldv<8>(w + po, gy);
 #pragma unroll
@@ -1293,33 +1529,33 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
     if (isq) stv<8>(q_out + ee, x);
     else stv<8>(kc + (((size_t)blk * G + hd) * bs + off) * D + d, x);
   }
-  for (int e = tid; e < nv; e += 256) {
-    const int g = e / Dv, c = e - g * Dv;
-    vc[(((size_t)blk * G + g) * Dv + c) * bs + off] = v[e];
-  }
+  append_values<T>(v, pb ? pb + nq + nk : nullptr, v_in_ ? (const T*)v_in_ + (size_t)t * nv : nullptr,
+                   v_out_ ? (T*)v_out_ + (size_t)t * nv : nullptr, lam, vc, blk, off, G, Dv, bs);
 }
 
 void sm_rownorm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_t q_norm, uintptr_t k_norm,
                      uintptr_t freqs, int nrot, float eps, uintptr_t k_cache, uintptr_t v_cache, uintptr_t slot_mapping,
                      uintptr_t positions, int tokens, int H, int G, int D, int Dv, int bs, float mag, int v_from_k,
-                     int f32, uintptr_t stream) {
+                     uintptr_t bias, uintptr_t v_in, uintptr_t v_out, float lam, int f32, uintptr_t stream) {
   if (tokens <= 0) return;
   DLLM_HOST_CHECK(H > 0 && G > 0 && D > 0 && Dv > 0 && bs > 0 && nrot >= 0 && 2 * nrot <= D && col0 >= 0 &&
                       ld >= col0 + (long)H * D + (long)G * D + (v_from_k ? 0 : (long)G * Dv) && (!v_from_k || Dv == D),
                   "rownorm_rope sizes");
+  DLLM_HOST_CHECK(!v_from_k || (!bias && !v_in && !v_out), "rownorm_rope values from keys");
   DLLM_HOST_CHECK(q_out && k_cache && v_cache && (!q_norm == !k_norm) && (nrot == 0 || freqs), "rownorm_rope arguments");
   const int esz = f32 ? 4 : 2;
   if (D % 8 == 0 && nrot % 8 == 0 && ld % 8 == 0 && col0 % 8 == 0 && qkv % (8 * esz) == 0 && q_norm % (8 * esz) == 0 &&
-      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0) {
+      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0 && bias % (8 * esz) == 0) {
     SM_DISPATCH(f32, sm_rownorm_rope_vec_kernel, dim3(tokens), dim3(256), 2 * (size_t)nrot * sizeof(float), stream,
                 (void*)q_out, (const void*)qkv, ld, col0, (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot,
                 eps, (void*)k_cache, (void*)v_cache, (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs,
-                mag, v_from_k);
+                mag, v_from_k, (const void*)bias, (const void*)v_in, (void*)v_out, lam);
     return;
   }
   SM_DISPATCH(f32, sm_rownorm_rope_kernel, dim3(tokens), dim3(256), 2 * (size_t)nrot * sizeof(float), stream, (void*)q_out, (const void*)qkv, ld, col0,
               (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot, eps, (void*)k_cache, (void*)v_cache,
-              (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, mag, v_from_k);
+              (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, mag, v_from_k,
+              (const void*)bias, (const void*)v_in, (void*)v_out, lam);
 }
 
 // --------------------------------------------------------------------------- attention input: per-head norm, paired rotation, append
@@ -1328,7 +1564,9 @@ void sm_rownorm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_
 // given) before or -- `norm_last` -- after the rotation of its first 2 nrot dimensions, pairs (2i, 2i + 1) turning by
 // float(pos) * freqs[i].  q is then multiplied by q_mul[h] (when given) and, with temp_every > 0, by
 // 1 + temp_coef ln(floor((pos + 1) / temp_every) + 1).  q goes to q_out [T, H, D]; k and v (unchanged) are appended at
-// slot_mapping to caches k [NB, G, BS, D] / v [NB, G, Dv, BS].  Norms, angles and factors are float32.
+// slot_mapping to caches k [NB, G, BS, D] / v [NB, G, Dv, BS].  Norms, angles and factors are float32.  `pb` (or null):
+// biases of the projected q | k | v columns, added before anything else; v_in / v_out / lam: values shared between
+// layers (append_values).
 //
 // One workgroup per token; 8 consecutive dimensions per lane, a head on an aligned group of `lph` lanes (a power of
 // two, 8 lph >= D): the mean square is a butterfly inside the group, the rotation stays inside a lane.
@@ -1342,7 +1580,8 @@ __global__ void __launch_bounds__(256) sm_head_norm_rope_vec_kernel(
     const void* __restrict__ kw_, const float* __restrict__ freqs, int nrot, int norm_last, float eps,
     const float* __restrict__ q_mul, float temp_coef, int temp_every, void* __restrict__ k_cache_,
     void* __restrict__ v_cache_, const int32_t* __restrict__ slot_mapping, const int32_t* __restrict__ positions, int H,
-    int G, int D, int Dv, int bs, int lph) {
+    int G, int D, int Dv, int bs, int lph, const void* __restrict__ pb_, const void* __restrict__ v_in_,
+    void* __restrict__ v_out_, float lam) {
   extern __shared__ float csn[];                   // cos | sin of the token's nrot angles
   const int t = blockIdx.x, tid = threadIdx.x, pos = positions[t];
   const float fpos = (float)pos;
@@ -1354,6 +1593,7 @@ __global__ void __launch_bounds__(256) sm_head_norm_rope_vec_kernel(
   const T* q = (const T*)qkv_ + (size_t)t * ld + col0;
   const int nq = H * D, nk = G * D, nv = G * Dv;
   const T* v = q + nq + nk;
+  const T* pb = (const T*)pb_;
   const int slot = slot_mapping[t], blk = slot / bs, off = slot - blk * bs;
   T* q_out = (T*)q_out_ + (size_t)t * nq;
   T* kc = (T*)k_cache_;
@@ -1369,7 +1609,10 @@ __global__ void __launch_bounds__(256) sm_head_norm_rope_vec_kernel(
     float x[8];
 #pragma unroll
     for (int i = 0; i < 8; ++i) x[i] = 0.f;
-    if (ok) ldv<8>(q + (size_t)head * D + d, x);
+    if (ok) {
+      ldv<8>(q + (size_t)head * D + d, x);
+      if (pb) add8(x, pb + head * D + d);
+    }
     float ss = 0.f;
     auto turn = [&]() {
 #pragma unroll
@@ -1408,10 +1651,8 @@ __global__ void __launch_bounds__(256) sm_head_norm_rope_vec_kernel(
       stv<8>(kc + (((size_t)blk * G + (head - H)) * bs + off) * D + d, x);
     }
   }
-  for (int e = tid; e < nv; e += 256) {
-    const int g = e / Dv, c = e - g * Dv;
-    vc[(((size_t)blk * G + g) * Dv + c) * bs + off] = v[e];
-  }
+  append_values<T>(v, pb ? pb + nq + nk : nullptr, v_in_ ? (const T*)v_in_ + (size_t)t * nv : nullptr,
+                   v_out_ ? (T*)v_out_ + (size_t)t * nv : nullptr, lam, vc, blk, off, G, Dv, bs);
 }
 
 // The same for any head size: a wave per (token, head), the head's values in LDS.
@@ -1421,16 +1662,19 @@ __global__ void __launch_bounds__(64) sm_head_norm_rope_kernel(
     const void* __restrict__ kw_, const float* __restrict__ freqs, int nrot, int norm_last, float eps,
     const float* __restrict__ q_mul, float temp_coef, int temp_every, void* __restrict__ k_cache_,
     void* __restrict__ v_cache_, const int32_t* __restrict__ slot_mapping, const int32_t* __restrict__ positions, int H,
-    int G, int D, int Dv, int bs, int) {
+    int G, int D, int Dv, int bs, int, const void* __restrict__ pb_, const void* __restrict__ v_in_,
+    void* __restrict__ v_out_, float lam) {
   extern __shared__ float hv[];                    // the head's values [D]
   const int t = blockIdx.x, head = blockIdx.y, lane = threadIdx.x, pos = positions[t];
   const T* q = (const T*)qkv_ + (size_t)t * ld + col0;
+  const T* pb = (const T*)pb_;
   const int slot = slot_mapping[t], blk = slot / bs, off = slot - blk * bs;
   if (head >= H + G) {                             // a value head
     const int g = head - H - G;
-    const T* v = q + (size_t)(H + G) * D + (size_t)g * Dv;
-    T* dst = (T*)v_cache_ + ((size_t)blk * G + g) * Dv * bs + off;
-    for (int c = lane; c < Dv; c += 64) dst[(size_t)c * bs] = v[c];
+    const size_t v0 = ((size_t)t * G + g) * Dv;          // this head's place in the shared values
+    append_values<T>(q + (size_t)(H + G) * D + (size_t)g * Dv, pb ? pb + (H + G) * D + g * Dv : nullptr,
+                     v_in_ ? (const T*)v_in_ + v0 : nullptr, v_out_ ? (T*)v_out_ + v0 : nullptr, lam,
+                     (T*)v_cache_ + (size_t)g * Dv * bs, blk * G, off, 1, Dv, bs);
     return;
   }
   const bool isq = head < H;
@@ -1447,7 +1691,7 @@ __global__ void __launch_bounds__(64) sm_head_norm_rope_kernel(
     }
     __syncthreads();
   };
-  for (int e = lane; e < D; e += 64) hv[e] = ldf(src + e);
+  for (int e = lane; e < D; e += 64) hv[e] = ldf(src + e) + (pb ? ldf(pb + head * D + e) : 0.f);
   __syncthreads();
   if (norm_last) turn();
   float ss = 0.f;
@@ -1467,7 +1711,8 @@ __global__ void __launch_bounds__(64) sm_head_norm_rope_kernel(
 void sm_head_norm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_t q_norm, uintptr_t k_norm,
                        uintptr_t freqs, int nrot, int norm_last, float eps, uintptr_t q_mul, float temp_coef, int temp_every,
                        uintptr_t k_cache, uintptr_t v_cache, uintptr_t slot_mapping, uintptr_t positions, int tokens, int H,
-                       int G, int D, int Dv, int bs, int f32, uintptr_t stream) {
+                       int G, int D, int Dv, int bs, uintptr_t bias, uintptr_t v_in, uintptr_t v_out, float lam, int f32,
+                       uintptr_t stream) {
   if (tokens <= 0) return;
   DLLM_HOST_CHECK(H > 0 && G > 0 && D > 0 && Dv > 0 && bs > 0 && nrot >= 0 && 2 * nrot <= D && col0 >= 0 && temp_every >= 0 &&
                       H + 2 * G <= 65535 && D <= 8192 && ld >= col0 + (long)H * D + (long)G * (D + Dv),
@@ -1477,19 +1722,21 @@ void sm_head_norm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintpt
                   "head_norm_rope arguments");
   const int esz = f32 ? 4 : 2;
   if (D % 8 == 0 && D <= 512 && ld % 8 == 0 && col0 % 8 == 0 && qkv % (8 * esz) == 0 && q_norm % (8 * esz) == 0 &&
-      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0) {
+      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0 && bias % (8 * esz) == 0) {
     int lph = 1;
     while (8 * lph < D) lph *= 2;
     SM_DISPATCH(f32, sm_head_norm_rope_vec_kernel, dim3(tokens), dim3(256), 2 * (size_t)nrot * sizeof(float), stream,
                 (void*)q_out, (const void*)qkv, ld, col0, (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot,
                 norm_last, eps, (const float*)q_mul, temp_coef, temp_every, (void*)k_cache, (void*)v_cache,
-                (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, lph);
+                (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, lph,
+                (const void*)bias, (const void*)v_in, (void*)v_out, lam);
     return;
   }
   SM_DISPATCH(f32, sm_head_norm_rope_kernel, dim3(tokens, H + 2 * G), dim3(64), (size_t)D * sizeof(float), stream,
               (void*)q_out, (const void*)qkv, ld, col0, (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot,
               norm_last, eps, (const float*)q_mul, temp_coef, temp_every, (void*)k_cache, (void*)v_cache,
-              (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, 0);
+              (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, 0, (const void*)bias, (const void*)v_in,
+              (void*)v_out, lam);
 }
 
 // --------------------------------------------------------------------------- averaged blocks of old keys

@@ -12,7 +12,7 @@
 namespace dllm {
 
 // out[m, n] = sum_s P[s, m, n] (+ bias[n]);  ACT 1: out[m, j] = silu(sum P[m, j]) * sum P[m, I + j];  ACT 2: the
-// clipped GLU of `limit` (common.h) of the same pair
+// clipped GLU of `limit` (common.h) of the same pair;  ACT 3: its gelu GLU
 // Each thread reduces V = 8 consecutive outputs (16-byte slab loads; 4 where ncols % 8 != 0).
 template <int ACT, int SC, int V>
 __global__ void __launch_bounds__(256) splitk_reduce_kernel(bf16* __restrict__ out, const float* __restrict__ P,
@@ -67,7 +67,8 @@ __global__ void __launch_bounds__(256) splitk_reduce_kernel(bf16* __restrict__ o
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         float x = a[h][j];
-        if (ACT == 2) x = clipped_glu_f(x, u[h][j], limit);
+        if (ACT == 3) x = gelu_glu_f(x, u[h][j]);
+        else if (ACT == 2) x = clipped_glu_f(x, u[h][j], limit);
         else if (ACT == 1) x = silu_f(x) * u[h][j];
         else if (bias) x += bf2f(bias[c + 4 * h + j]);
         o[h][j] = f2bf(x);
@@ -246,10 +247,10 @@ void splitk_add_rms_norm_q8(uintptr_t y, uintptr_t residual, uintptr_t ws, int S
 }
 
 // plain split-K reduce of the partial slabs a split GEMM left (mode 2 of gemm_wide / gemm_sq / gemm_pp): out = bf16(sum_s P[s]) (+bias)
-// act 1: SwiGLU, act 2: clipped GLU of `limit` -- out [M, N / 2] from gate | up columns
+// act 1: SwiGLU, act 2: clipped GLU of `limit`, act 3: gelu GLU -- out [M, N / 2] from gate | up columns
 void splitk_reduce_ex(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M, int N, int act, uintptr_t stream,
                       float limit) {
-  DLLM_HOST_CHECK(act >= 0 && act <= 2, "split-K reduce activation");
+  DLLM_HOST_CHECK(act >= 0 && act <= 3, "split-K reduce activation");
   const bool swiglu = act != 0;
   DLLM_HOST_CHECK(N % (swiglu ? 8 : 4) == 0, "N alignment");
   const int ncols = swiglu ? N / 2 : N;
@@ -278,7 +279,8 @@ void splitk_reduce_ex(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M,
   do {                                                                 \
     if (v8) DLLM_SKR2(SW, 8); else DLLM_SKR2(SW, 4);                   \
   } while (0)
-  if (act == 2) DLLM_SKR(2);
+  if (act == 3) DLLM_SKR(3);
+  else if (act == 2) DLLM_SKR(2);
   else if (act == 1) DLLM_SKR(1);
   else DLLM_SKR(0);
 #undef DLLM_SKR
@@ -293,6 +295,11 @@ void splitk_reduce(uintptr_t out, uintptr_t ws, uintptr_t bias, int S, int M, in
 // out [M, N / 2] = the clipped GLU of the summed gate | up slabs
 void splitk_reduce_clipped(uintptr_t out, uintptr_t ws, int S, int M, int N, float limit, uintptr_t stream) {
   splitk_reduce_ex(out, ws, 0, S, M, N, 2, stream, limit);
+}
+
+// out [M, N / 2] = gelu_tanh(gate) * up of the summed gate | up slabs
+void splitk_reduce_gelu(uintptr_t out, uintptr_t ws, int S, int M, int N, uintptr_t stream) {
+  splitk_reduce_ex(out, ws, 0, S, M, N, 3, stream);
 }
 
 }  // namespace dllm

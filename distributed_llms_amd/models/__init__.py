@@ -17,6 +17,9 @@ def stage_class(arch: str):
     if arch == "kupedra":
         from .kupedra import KupedraStage
         return KupedraStage
+    if arch == "basopel":
+        from .basopel import BasopelStage
+        return BasopelStage
     if arch in ("llama", "mixtral", "gpt2"):
         from .stage import ModelStage
         return ModelStage

@@ -305,10 +305,11 @@ def linear_pp(x: torch.Tensor, w: torch.Tensor, splits: int = 0, swiglu: bool = 
 
 
 def linear_pf(x: torch.Tensor, w: torch.Tensor, swiglu: bool = False, variant: int = 0,
-              limit: Optional[float] = None) -> torch.Tensor:
+              limit: Optional[float] = None, gelu: bool = False) -> torch.Tensor:
     """Persistent prefill GEMM (gemm_pf in csrc/kernels/gemm_pp.hip): schedule 2's 256 x 256 tiles,
     one workgroup per CU walking its tiles with the LDS-DMA pipeline running across tile
-    boundaries; optional fused SwiGLU (``w`` = [Wg; Wu], y [M, N / 2]) or -- ``limit`` -- clipped GLU.  ``variant`` 8: nontemporal
+    boundaries; optional fused SwiGLU (``w`` = [Wg; Wu], y [M, N / 2]) or -- ``limit`` -- clipped GLU or -- ``gelu`` --
+    gelu_tanh GLU.  ``variant`` 8: nontemporal
     output stores (the default for SwiGLU outputs > 256 MiB); the tiles come from per-XCD device
     queues while knobs.pf_dynamic says so (bit 16 of the launcher's variant)."""
     k = x.shape[-1]
@@ -318,7 +319,7 @@ def linear_pf(x: torch.Tensor, w: torch.Tensor, swiglu: bool = False, variant: i
         raise ValueError("linear_pf: bf16 contiguous operands")
     if n % 256 or k % 64:
         raise ValueError("linear_pf: N % 256 and K % 64")
-    glu = swiglu or limit is not None
+    glu = swiglu or gelu or limit is not None
     y = torch.empty(*x.shape[:-1], n // 2 if glu else n, dtype=x.dtype, device=x.device)
     dyn = pf_dynamic() and k >= 128
     if torch.cuda.is_current_stream_capturing():
@@ -328,7 +329,7 @@ def linear_pf(x: torch.Tensor, w: torch.Tensor, swiglu: bool = False, variant: i
     if dyn:
         variant |= 16                  # per-XCD dynamic tile queues (gemm_pp.hip, DYN)
     _ext.kernels().gemm_pf(y.data_ptr(), x.data_ptr(), w.data_ptr(), m, n, k,
-                           3 if limit is not None else (1 if swiglu else 0), variant, torch.cuda.current_stream().cuda_stream,
+                           4 if gelu else 3 if limit is not None else (1 if swiglu else 0), variant, torch.cuda.current_stream().cuda_stream,
                            0.0 if limit is None else float(limit))
     return y
 
@@ -393,10 +394,9 @@ def linear_sq(x: torch.Tensor, w: torch.Tensor, splits: int = 0, swiglu: bool = 
     return y
 
 
-def linear_clipped_glu(x: torch.Tensor, w_gate_up: torch.Tensor, limit: float) -> Optional[torch.Tensor]:
-    """g sigmoid(1.702 g) (u + 1), g = min(x Wg^T, limit), u = clamp(x Wu^T, -limit, limit), W = [Wg; Wu], with the
-    activation in the persistent GEMM's epilogue (prompts) or in the split-K reduction (decode); None if the
-    shape takes neither."""
+def _linear_glu(x: torch.Tensor, w_gate_up: torch.Tensor, limit: Optional[float]) -> Optional[torch.Tensor]:
+    """A GLU of x Wg^T and x Wu^T, W = [Wg; Wu], with the activation in the persistent GEMM's epilogue (prompts) or in
+    the split-K reduction (decode): clipped (``limit``) or gelu_tanh (None); None if the shape takes neither."""
     k = x.shape[-1]
     n = w_gate_up.shape[0]
     m = x.numel() // k
@@ -404,15 +404,28 @@ def linear_clipped_glu(x: torch.Tensor, w_gate_up: torch.Tensor, limit: float) -
         return None
     if not _use_wide(m, n, k, x, w_gate_up) and _use_pp(m, n, k, x, w_gate_up, knobs.K.pp_swiglu_min_m) \
             and knobs.K.pp_persistent and m * (n // 2) * 2 < (1 << 31) and pf_fills(m, n, x.device):
-        return linear_pf(x, w_gate_up, limit=limit)
+        return linear_pf(x, w_gate_up, limit=limit, gelu=limit is None)
     y = linear(x, w_gate_up, defer=True)
     if isinstance(y, SplitKPartial):
         out = torch.empty(*x.shape[:-1], n // 2, dtype=x.dtype, device=x.device)
-        _ext.kernels().splitk_reduce_clipped(out.data_ptr(), y.ws.data_ptr(), y.splits, y.m, y.n, float(limit),
-                                             torch.cuda.current_stream().cuda_stream)
+        st = torch.cuda.current_stream().cuda_stream
+        if limit is None:
+            _ext.kernels().splitk_reduce_gelu(out.data_ptr(), y.ws.data_ptr(), y.splits, y.m, y.n, st)
+        else:
+            _ext.kernels().splitk_reduce_clipped(out.data_ptr(), y.ws.data_ptr(), y.splits, y.m, y.n, float(limit), st)
         return out
-    from .seqmix import clipped_glu
-    return clipped_glu(y, None, limit)
+    from .seqmix import clipped_glu, gelu_glu
+    return gelu_glu(y) if limit is None else clipped_glu(y, None, limit)
+
+
+def linear_clipped_glu(x: torch.Tensor, w_gate_up: torch.Tensor, limit: float) -> Optional[torch.Tensor]:
+    """g sigmoid(1.702 g) (u + 1), g = min(x Wg^T, limit), u = clamp(x Wu^T, -limit, limit), fused (:func:`_linear_glu`)."""
+    return _linear_glu(x, w_gate_up, float(limit))
+
+
+def linear_gelu_glu(x: torch.Tensor, w_gate_up: torch.Tensor) -> Optional[torch.Tensor]:
+    """gelu_tanh(x Wg^T) * (x Wu^T), fused (:func:`_linear_glu`)."""
+    return _linear_glu(x, w_gate_up, None)
 
 
 def linear_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor) -> Optional[torch.Tensor]:

@@ -2,12 +2,13 @@
 pre- and post-sublayer RMS norms (also for sublayers that read the stream unnormed, and for two mixer
 outputs summed with scales), short causal convolutions with a state tail, the real-gated linear
 recurrent unit (RG-LRU), sliding-window and chunked attention over a paged K/V cache whose key and value
-widths differ (optionally with capped scores, per-head sinks and one averaged key / value per block of
-positions older than the window), two attention input stages (convolution + per-head norm + interleaved
+widths differ (optionally with capped scores, per-head sinks, one averaged key / value per block of
+positions older than the window, first tokens that stay visible and a gate per head), two attention input stages (convolution + per-head norm + interleaved
 rotation; whole-projection norm + half-split rotation, also without norms and with the values taken from
 the keys; per-head norm before or after a paired rotation with query temperatures), a learned bias per distance
-bucket, the close of pre-norm sublayers whose outputs are normed apart, a token shift, the entry of a
-looped span of layers, a clipped GLU and the logit soft cap.
+bucket, projection biases and values shared between layers, the close of pre-norm sublayers whose outputs are normed
+apart, sublayers between two layer norms, a token shift, the entry of a looped span of layers, clipped and gelu GLUs
+and the logit soft cap.
 
 Same dispatch as :mod:`distributed_llms_amd.ops`: a CUDA tensor goes to the in-tree HIP kernels
 (csrc/kernels/seqmix.hip, attention_window.hip) and raises if they are not built; CPU tensors run
@@ -74,15 +75,15 @@ def _ptr(t: Optional[torch.Tensor]) -> int:
 
 
 # ------------------------------------------------------------------ embedding / norms
-def embedding_f32(ids: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
-    """Rows of ``table`` as a float32 residual stream [T, W]."""
+def embedding_f32(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+    """Rows of ``table`` times ``scale`` as a float32 residual stream [T, W]."""
     if not table.is_cuda:
-        return table.index_select(0, ids.long()).float()
+        return table.index_select(0, ids.long()).float() * scale
     _ck(ids, "ids", torch.int32)
     _ck(table, "table")
     t, (v, w) = ids.numel(), table.shape
     out = torch.empty(t, w, dtype=torch.float32, device=table.device)
-    _k().sm_embed_f32(out.data_ptr(), ids.data_ptr(), table.data_ptr(), t, w, v, _f32flag(table), _stream())
+    _k().sm_embed_f32(out.data_ptr(), ids.data_ptr(), table.data_ptr(), t, w, v, float(scale), _f32flag(table), _stream())
     return out
 
 
@@ -167,6 +168,61 @@ def post_norm_add(x: torch.Tensor, o: torch.Tensor, w_post: torch.Tensor, eps: f
                           float(eps), float(mult), off, _ptr(o2), float(scales[0]), float(scales[1]), _f32flag(o),
                           _stream())
     return x, (x if (plain_next and w_next is None and h is None) else h)
+
+
+def _ref_layer_norm(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor, eps: float) -> torch.Tensor:
+    x = x.float()
+    c = x - x.mean(-1, keepdim=True)
+    return c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w.float() + b.float()
+
+
+LAYER_NORM_MAX_WIDTH = 16384
+
+
+def layer_norm_f32(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor, eps: float, act_dtype) -> torch.Tensor:
+    """x [T, W] float32 -> (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b in ``act_dtype``."""
+    if not x.is_cuda:
+        return _ref_layer_norm(x, w, b, eps).to(act_dtype)
+    _ck(x, "x", torch.float32)
+    _ck(w, "w", act_dtype)
+    _ck(b, "b", act_dtype)
+    t, width = x.shape
+    if w.numel() != width or b.numel() != width:
+        raise ValueError("layer_norm_f32: weight / bias width")
+    y = torch.empty(t, width, dtype=act_dtype, device=x.device)
+    _k().sm_layer_norm(y.data_ptr(), x.data_ptr(), w.data_ptr(), b.data_ptr(), t, width, float(eps), _f32flag(y), _stream())
+    return y
+
+
+def post_layer_norm_add(x: torch.Tensor, o, w_post: torch.Tensor, b_post: torch.Tensor, eps: float,
+                        bias: Optional[torch.Tensor] = None, w_next: Optional[torch.Tensor] = None,
+                        b_next: Optional[torch.Tensor] = None):
+    """The close of a sublayer between two layer norms, fused: ``x += layer_norm(o + bias) `` (weight ``w_post``, bias
+    ``b_post``) in place on the float32 residual stream; with ``w_next`` / ``b_next`` also returns the next sublayer's input
+    layer_norm(x) in the activation type (None otherwise).  ``o`` may be a :class:`~.gemm.SplitKPartial` (the output of a
+    split-K product that is not reduced yet): its slabs are then summed in the same launch."""
+    from .gemm import SplitKPartial
+    if tuple(o.shape) != tuple(x.shape) or (w_next is None) != (b_next is None):
+        raise ValueError("post_layer_norm_add: o / x shape mismatch, or half a next norm")
+    if not x.is_cuda:
+        ob = o.float() if bias is None else o.float() + bias.float()
+        x.add_(_ref_layer_norm(ob, w_post, b_post, eps))
+        return x, (None if w_next is None else _ref_layer_norm(x, w_next, b_next, eps).to(o.dtype))
+    part = o if isinstance(o, SplitKPartial) else None
+    _ck(x, "x", torch.float32)
+    t, width = x.shape
+    if part is None:
+        _ck(o, "o")
+    for n, w in (("bias", bias), ("w_post", w_post), ("b_post", b_post), ("w_next", w_next), ("b_next", b_next)):
+        if w is not None:
+            _ck(w, n, o.dtype)
+            if w.numel() != width:
+                raise ValueError(f"post_layer_norm_add: {n} width")
+    h = None if w_next is None else torch.empty(t, width, dtype=o.dtype, device=x.device)
+    _k().sm_post_layer_norm_add(x.data_ptr(), (part.ws if part is not None else o).data_ptr(), 0 if part is None else part.splits,
+                                _ptr(bias), w_post.data_ptr(), b_post.data_ptr(), _ptr(w_next), _ptr(b_next), _ptr(h), t,
+                                width, float(eps), 1 if o.dtype == torch.float32 else 0, _stream())
+    return x, h
 
 
 def stream_enter(x: torch.Tensor, x0: Optional[torch.Tensor], vec: Optional[torch.Tensor]) -> torch.Tensor:
@@ -394,6 +450,26 @@ def clipped_glu(gu: torch.Tensor, bias_gu: Optional[torch.Tensor], limit: float,
     return out
 
 
+def gelu_glu(gu: torch.Tensor) -> torch.Tensor:
+    """[T, 2F] = gate | up -> gelu_tanh(gate) * up  [T, F]."""
+    t, two_f = gu.shape
+    f = two_f // 2
+    if not gu.is_cuda:
+        return (gelu_tanh_f32(gu[:, :f].float()) * gu[:, f:].float()).to(gu.dtype)
+    _ck(gu, "gu")
+    out = torch.empty(t, f, dtype=gu.dtype, device=gu.device)
+    _k().sm_gelu_glu(out.data_ptr(), gu.data_ptr(), t, f, _f32flag(gu), _stream())
+    return out
+
+
+def linear_gelu_glu(x: torch.Tensor, w_gate_up: torch.Tensor) -> torch.Tensor:
+    """gelu_tanh(x Wg^T) * (x Wu^T), W = [Wg; Wu]: in a GEMM epilogue or the split-K reduction where the framework's
+    bf16 GEMMs take the shape, else the projection followed by the gate kernel (float32, odd sizes)."""
+    from . import gemm, linear
+    y = gemm.linear_gelu_glu(x, w_gate_up) if x.is_cuda else None
+    return gelu_glu(linear(x, w_gate_up)) if y is None else y
+
+
 def softcap_f32(logits: torch.Tensor, cap: float, scale: float = 1.0) -> torch.Tensor:
     """float32 cap * tanh(z / cap) with z = logits * scale (cap <= 0: z itself)."""
     if not logits.is_cuda:
@@ -497,6 +573,42 @@ def attn_prep(qkv: torch.Tensor, conv_w: torch.Tensor, state: torch.Tensor, q_no
     return q
 
 
+# ------------------------------------------------------------------ values shared between layers
+@dataclass
+class ValueMix:
+    """How a layer's values meet those of an earlier layer: ``first`` [T, kv_heads * vdim] (activation type) holds the
+    earlier layer's values of the step's tokens.  ``lam`` None: this IS the earlier layer, its values (projection bias
+    included) are written there; else v <- (1 - lam) v + lam first, and the mixed v is what the cache keeps."""
+    first: torch.Tensor
+    lam: Optional[float] = None
+
+
+def _ref_values(v: torch.Tensor, v_mix: Optional[ValueMix]) -> torch.Tensor:
+    """v [T, kv_heads * vdim] float32 (bias added)."""
+    if v_mix is None:
+        return v
+    if v_mix.lam is None:
+        v_mix.first.copy_(v.to(v_mix.first.dtype))
+        return v
+    return (1.0 - v_mix.lam) * v + v_mix.lam * v_mix.first.float()
+
+
+def _ck_mix(qkv: torch.Tensor, bias: Optional[torch.Tensor], v_mix: Optional[ValueMix], width: int, nv: int):
+    if bias is not None and (bias.numel() != width or bias.dtype != qkv.dtype or not bias.is_contiguous()):
+        raise ValueError("attention input: one bias per projected row, of the projection's type")
+    if v_mix is not None and (tuple(v_mix.first.shape) != (qkv.shape[0], nv) or v_mix.first.dtype != qkv.dtype
+                              or not v_mix.first.is_contiguous()):
+        raise ValueError("attention input: shared values [T, kv_heads * vdim] of the projection's type")
+
+
+def _mix_args(v_mix: Optional[ValueMix]):
+    """(values read, values written, lam) of the kernels."""
+    if v_mix is None:
+        return 0, 0, 0.0
+    p = v_mix.first.data_ptr()
+    return (0, p, 0.0) if v_mix.lam is None else (p, 0, float(v_mix.lam))
+
+
 # ------------------------------------------------------------------ attention input: row norm + half-split rotation + append
 def rotary_frequencies(dims: int, base: float, factor: float = 1.0) -> torch.Tensor:
     """f_i = base^(-2i / dims) / factor, i < dims / 2, computed in float64 and rounded once to float32."""
@@ -520,7 +632,8 @@ def _ref_rope_half(x: torch.Tensor, pos: torch.Tensor, freqs: torch.Tensor, mag:
 def rownorm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor],
                  freqs: torch.Tensor, eps: float, k_cache: torch.Tensor, v_cache: torch.Tensor, slot_mapping: torch.Tensor,
                  positions: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, mag: float = 1.0,
-                 v_from_k: bool = False) -> torch.Tensor:
+                 v_from_k: bool = False, bias: Optional[torch.Tensor] = None,
+                 v_mix: Optional[ValueMix] = None) -> torch.Tensor:
     """From columns ``col0 ..`` of a fused projection [T, .. | q (heads dim) | k (kv_heads dim) | v (kv_heads
     vdim) | ..]: an RMS norm over the WHOLE q projection and over the whole k projection (all heads at
     once; plain weights ``q_norm`` [heads dim], ``k_norm`` [kv_heads dim]; both None: no norm), then the
@@ -528,10 +641,14 @@ def rownorm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor], k
     with i + len(freqs), angle position * freqs[i], cos and sin times ``mag``), and the append of k and v
     (v unchanged) at ``slot_mapping`` into caches k [NB, kv_heads, BS, dim] / v [NB, kv_heads, vdim, BS].
     ``v_from_k``: the projection has no v columns; the values are the keys as projected, BEFORE norm and
-    rotation (vdim = dim).  Returns q [T, heads, dim]."""
+    rotation (vdim = dim).  ``bias`` [heads dim + kv_heads dim + kv_heads vdim]: added to the projected q | k | v before
+    anything else; ``v_mix``: values shared between layers (both: not with ``v_from_k``).  Returns q [T, heads, dim]."""
     t = qkv.shape[0]
     nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
     normed = q_norm is not None
+    if v_from_k and (bias is not None or v_mix is not None):
+        raise ValueError("rownorm_rope: values from keys exclude biases and shared values")
+    _ck_mix(qkv, bias, v_mix, nq + nk + nv, nv)
     if (k_norm is not None) != normed or (v_from_k and vdim != dim) or 2 * freqs.numel() > dim:
         raise ValueError("rownorm_rope: norm weights for both or neither; values from keys need vdim = dim")
     if qkv.shape[1] < col0 + nq + nk + (0 if v_from_k else nv) or (normed and (q_norm.numel() != nq or k_norm.numel() != nk)):
@@ -541,6 +658,8 @@ def rownorm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor], k
         raise ValueError("rownorm_rope: cache shape")
     if not qkv.is_cuda:
         x = qkv[:, col0:col0 + nq + nk].float()
+        if bias is not None:
+            x = x + bias[:nq + nk].float()
         xq, xk = x[:, :nq], x[:, nq:]
         if normed:
             xq, xk = _ref_rms(xq, q_norm, eps, 0.0), _ref_rms(xk, k_norm, eps, 0.0)
@@ -549,7 +668,9 @@ def rownorm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor], k
         slot = slot_mapping.long()
         k_cache[slot // bs, :, slot % bs] = k.to(k_cache.dtype)
         v0 = col0 + nq if v_from_k else col0 + nq + nk
-        v_cache[slot // bs, :, :, slot % bs] = qkv[:, v0:v0 + nv].reshape(t, kv_heads, vdim).to(v_cache.dtype)
+        v = qkv[:, v0:v0 + nv].float()
+        v = _ref_values(v if bias is None else v + bias[nq + nk:].float(), v_mix)
+        v_cache[slot // bs, :, :, slot % bs] = v.reshape(t, kv_heads, vdim).to(v_cache.dtype)
         return q.to(qkv.dtype)
     _ck(qkv, "qkv")
     if normed:
@@ -562,7 +683,7 @@ def rownorm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor], k
     _k().sm_rownorm_rope(q.data_ptr(), qkv.data_ptr(), qkv.shape[1], int(col0), _ptr(q_norm), _ptr(k_norm),
                          freqs.data_ptr(), freqs.numel(), float(eps), k_cache.data_ptr(), v_cache.data_ptr(),
                          slot_mapping.data_ptr(), positions.data_ptr(), t, heads, kv_heads, dim, vdim, bs, float(mag),
-                         1 if v_from_k else 0, _f32flag(qkv), _stream())
+                         1 if v_from_k else 0, _ptr(bias), *_mix_args(v_mix), _f32flag(qkv), _stream())
     return q
 
 
@@ -571,16 +692,19 @@ def head_norm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor],
                    freqs: Optional[torch.Tensor], eps: float, k_cache: torch.Tensor, v_cache: torch.Tensor,
                    slot_mapping: torch.Tensor, positions: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int,
                    norm_last: bool = False, q_mul: Optional[torch.Tensor] = None,
-                   q_temp: Optional[Tuple[float, int]] = None) -> torch.Tensor:
+                   q_temp: Optional[Tuple[float, int]] = None, bias: Optional[torch.Tensor] = None,
+                   v_mix: Optional[ValueMix] = None) -> torch.Tensor:
     """From columns ``col0 ..`` of a fused projection [T, .. | q (heads dim) | k (kv_heads dim) | v (kv_heads
     vdim) | ..]: an RMS norm of every q and k head over its ``dim`` (plain weights ``q_norm`` / ``k_norm`` [dim] shared
     by the heads; both None: no weight), before or -- ``norm_last`` -- after the rotation of its first 2 len(freqs)
     dimensions, pairs (2i, 2i + 1) turning by position * freqs[i] (None: no rotation).  q is then multiplied by
     ``q_mul`` [heads] float32 and by 1 + coef ln(floor((position + 1) / every) + 1) with ``q_temp`` = (coef, every); k and
     v (unchanged) are appended at ``slot_mapping`` to caches k [NB, kv_heads, BS, dim] / v [NB, kv_heads, vdim, BS].
-    Returns q [T, heads, dim]."""
+    ``bias`` [heads dim + kv_heads dim + kv_heads vdim]: added to the projected q | k | v before anything else; ``v_mix``:
+    values shared between layers.  Returns q [T, heads, dim]."""
     t = qkv.shape[0]
     nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
+    _ck_mix(qkv, bias, v_mix, nq + nk + nv, nv)
     nrot = 0 if freqs is None else freqs.numel()
     if (q_norm is None) != (k_norm is None) or 2 * nrot > dim or (q_norm is not None and (q_norm.numel() != dim or
                                                                                           k_norm.numel() != dim)):
@@ -600,15 +724,19 @@ def head_norm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor],
             x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
             x = x if w is None else x * w.float()
             return x if norm_last else turn(x)
-        q = prep(qkv[:, col0:col0 + nq].float().reshape(t, heads, dim), q_norm)
-        k = prep(qkv[:, col0 + nq:col0 + nq + nk].float().reshape(t, kv_heads, dim), k_norm)
+        x = qkv[:, col0:col0 + nq + nk + nv].float()
+        if bias is not None:
+            x = x + bias.float()
+        q = prep(x[:, :nq].reshape(t, heads, dim), q_norm)
+        k = prep(x[:, nq:nq + nk].reshape(t, kv_heads, dim), k_norm)
         if q_mul is not None:
             q = q * q_mul[None, :, None]
         if every:
             q = q * (1.0 + coef * torch.log(((positions + 1) // every).float() + 1.0))[:, None, None]
         slot = slot_mapping.long()
         k_cache[slot // bs, :, slot % bs] = k.to(k_cache.dtype)
-        v_cache[slot // bs, :, :, slot % bs] = qkv[:, col0 + nq + nk:col0 + nq + nk + nv].reshape(t, kv_heads, vdim).to(v_cache.dtype)
+        v = _ref_values(x[:, nq + nk:], v_mix)
+        v_cache[slot // bs, :, :, slot % bs] = v.reshape(t, kv_heads, vdim).to(v_cache.dtype)
         return q.to(qkv.dtype)
     _ck(qkv, "qkv")
     if q_norm is not None:
@@ -626,7 +754,7 @@ def head_norm_rope(qkv: torch.Tensor, col0: int, q_norm: Optional[torch.Tensor],
     _k().sm_head_norm_rope(q.data_ptr(), qkv.data_ptr(), qkv.shape[1], int(col0), _ptr(q_norm), _ptr(k_norm),
                            _ptr(freqs) if nrot else 0, nrot, 1 if norm_last else 0, float(eps), _ptr(q_mul), coef, every,
                            k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), positions.data_ptr(), t, heads,
-                           kv_heads, dim, vdim, bs, _f32flag(qkv), _stream())
+                           kv_heads, dim, vdim, bs, _ptr(bias), *_mix_args(v_mix), _f32flag(qkv), _stream())
     return q
 
 
@@ -719,7 +847,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                      sb: SeqBatch, window: int, scale: float, num_decode: Optional[int] = None,
                      sinks: Optional[torch.Tensor] = None, max_ctx: Optional[int] = None, chunk: int = 0,
                      softcap: float = 0.0, pooled: Optional[tuple] = None,
-                     bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     bias: Optional[torch.Tensor] = None, keep_first: int = 0, gate: Optional[torch.Tensor] = None,
+                     gate_col: int = 0) -> torch.Tensor:
     """Softmax attention of every query token over the keys j of its own sequence with
     0 <= p - j < window (p the query's position) and, with ``chunk`` > 0, floor(j / chunk) =
     floor(p / chunk) (attention inside fixed chunks of positions counted from position 0, wherever a
@@ -737,7 +866,10 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     b < floor((p - window + 1) / pool) of the averaged caches (:func:`pool_blocks`), scored, capped and
     normalised in the same softmax; tokens that left the window inside a block not yet complete are not
     seen at all.  ``bias`` [H, L] float32 (:func:`distance_bias_table`): bias[h][min(n, L - 1)] is added to the scaled
-    score of a key n positions back (not beside averaged caches).  Returns [T, H, vdim]."""
+    score of a key n positions back (not beside averaged caches).  ``keep_first``: beside its window a query also sees
+    the first that many positions of its sequence, at their true distances (not beside averaged caches).  ``gate`` (a
+    [T, *] tensor of q's type with one logit per head from column ``gate_col``): head h's output is multiplied by
+    sigmoid(gate[t, gate_col + h]).  Returns [T, H, vdim]."""
     t, h, d = q.shape
     g, bs, dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[2]
     kp = vp = None
@@ -749,6 +881,11 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             raise ValueError("window_attention: averaged caches do not fit (and exclude a chunk mask)")
     if bias is not None and (pool or bias.dtype != torch.float32 or bias.dim() != 2 or bias.shape[0] != h):
         raise ValueError("window_attention: bias [H, L] float32 (and no averaged caches)")
+    if keep_first < 0 or (keep_first and pool):
+        raise ValueError("window_attention: keep_first >= 0 (and no averaged caches)")
+    if gate is not None and (gate.dim() != 2 or gate.shape[0] != t or gate_col < 0 or gate_col + h > gate.shape[1]
+                             or gate.dtype != q.dtype):
+        raise ValueError("window_attention: gate [T, *] of q's type with one column per head")
     if not q.is_cuda:
         out = torch.empty(t, h, dv, dtype=torch.float32)
         pos, seq = sb.positions.tolist(), sb.tok_seq.tolist()
@@ -756,7 +893,7 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         for i in range(t):
             p = pos[i]
             lo = max(0, p - window + 1, p - p % chunk if chunk > 0 else 0)
-            idx = torch.arange(lo, p + 1)
+            idx = torch.cat([torch.arange(min(keep_first, lo)), torch.arange(lo, p + 1)])
             blk = block_tables[seq[i]].long()[idx // bs]
             kk = k_cache[blk, :, idx % bs].float().repeat_interleave(rep, 1)     # [n, H, d]
             vv = v_cache[blk, :, :, idx % bs].float().repeat_interleave(rep, 1)
@@ -775,6 +912,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             else:
                 pr = torch.softmax(s, -1)
             out[i] = torch.einsum("hn,nhd->hd", pr, vv)
+            if gate is not None:
+                out[i] *= torch.sigmoid(gate[i, gate_col:gate_col + h].float())[:, None]
         return out.to(q.dtype)
     _ck(q, "q")
     _ck(k_cache, "k_cache", q.dtype)
@@ -793,13 +932,19 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     if bias is not None:
         _ck(bias, "bias", torch.float32)
         nbias = bias.shape[1]
+    gp = gld = 0
+    if gate is not None:
+        _ck(gate, "gate")
+        gp, gld = gate.data_ptr() + gate_col * gate.element_size(), gate.shape[1]
+    keep = min(int(keep_first), 1 << 30)
     out = torch.empty(t, h, dv, dtype=q.dtype, device=q.device)
     nd = sb.num_seqs if num_decode is None else int(num_decode)
     f = _f32flag(q)
     if nd:       # one-token rows are the first nd tokens
         span = min(int(window), int(chunk)) if chunk > 0 else int(window)
         ctx = int(max_ctx or 0)
-        keys = min(span, ctx) + (max(0, ctx - span) // pool if pool else 0)      # window tokens + averaged entries
+        # window tokens + averaged entries / kept first tokens
+        keys = min(span, ctx) + (max(0, ctx - span) // pool if pool else min(keep, max(0, ctx - span)))
         splits, ws = decode_splits(nd, h, g, keys), None
         if splits > 1 and not f:
             ws = torch.empty(nd * h * splits * (dv + 2), dtype=torch.float32, device=q.device)
@@ -807,12 +952,12 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                                    block_tables.data_ptr(), block_tables.shape[1], sb.positions.data_ptr(),
                                    sb.tok_seq.data_ptr(), nd, h, g, d, dv, bs, int(window), int(chunk), float(scale), _ptr(sinks),
                                    splits if ws is not None else 1, _ptr(ws), float(softcap), _ptr(kp), _ptr(vp), int(pool),
-                                   int(pb), _ptr(bias), nbias, f, _stream())
+                                   int(pb), _ptr(bias), nbias, keep, gp, gld, f, _stream())
     if t > nd:
         _k().sm_window_attn_prefill(out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                                     block_tables.data_ptr(), block_tables.shape[1], sb.cu.data_ptr(),
                                     sb.positions.data_ptr(), sb.tok_seq.data_ptr(), nd, sb.num_seqs, t, sb.max_q_len,
                                     h, g, d, dv, bs,
                                     int(window), int(chunk), float(scale), _ptr(sinks), float(softcap), _ptr(kp), _ptr(vp),
-                                    int(pool), int(pb), _ptr(bias), nbias, f, _stream())
+                                    int(pool), int(pb), _ptr(bias), nbias, keep, gp, gld, f, _stream())
     return out
