@@ -95,7 +95,8 @@ def parse(argv=None):
                          "Mixtral), or fekizen,zebutar,mixtral (window attention with averaged blocks beside gated "
                          "linear attention, lightning layers + SwiGLU experts, beside both), or "
                          "kupedra,fekizen,mixtral (hyper-connected streams, distance-biased attention beside a gated "
-                         "matrix memory + clipped-GLU experts, beside both), or one of them")
+                         "matrix memory + clipped-GLU experts, beside both), or basopel,tudilix,llama (biased windows, chunked "
+                         "and latent attention between layer norms + gelu GLUs, beside both), or one of them")
     return ap.parse_args(argv)
 
 

@@ -288,33 +288,56 @@ __global__ void __launch_bounds__(256) sm_post_layer_norm_kernel(
   const size_t row = (size_t)blockIdx.x * width;
   float* xr = x + row;
   float v[NV][V], xv[NV][V], w[NV][V], b[NV][V];
+  // every load of the row off a clamped place, so that none waits behind another's guard; the slabs eight at a time
+  const int top = width - V;
+  if (V == 4 && parts > 0) {
+    const float* P = (const float*)o_;
+    const size_t slab = (size_t)gridDim.x * width;
+    constexpr int CH = NV <= 4 ? 8 : 2;
+    f32x4 a[NV];
+#pragma unroll
+    for (int k = 0; k < NV; ++k) a[k] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int s0 = 0; s0 < parts; s0 += CH) {
+      f32x4 l[CH][NV];
+#pragma unroll
+      for (int u = 0; u < CH; ++u)
+#pragma unroll
+        for (int k = 0; k < NV; ++k)
+          l[u][k] = part_load4(P, min(s0 + u, parts - 1) * slab + row + min((k * 256 + (int)threadIdx.x) * V, top));
+#pragma unroll
+      for (int u = 0; u < CH; ++u)
+        if (s0 + u < parts) {
+#pragma unroll
+          for (int k = 0; k < NV; ++k) a[k] += l[u][k];
+        }
+    }
+#pragma unroll
+    for (int k = 0; k < NV; ++k)
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[k][j] = bf2f(f2bf(a[k][j & 3]));
+  } else {
+#pragma unroll
+    for (int k = 0; k < NV; ++k) ldv<V>((const T*)o_ + row + min((k * 256 + (int)threadIdx.x) * V, top), v[k]);
+  }
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
-    const int i = (k * 256 + threadIdx.x) * V;
+    const int i = min((k * 256 + (int)threadIdx.x) * V, top);
+    ldv<V>(xr + i, xv[k]);
+    ldv<V>((const T*)wp_ + i, w[k]);
+    ldv<V>((const T*)bp_ + i, b[k]);
+    if (bias_) {
+      float c[V];
+      ldv<V>((const T*)bias_ + i, c);
 #pragma unroll
-    for (int j = 0; j < V; ++j) v[k][j] = xv[k][j] = 0.f;
-    if (i < width) {
-      if (V == 4 && parts > 0) {
-        const float* P = (const float*)o_;
-        const size_t slab = (size_t)gridDim.x * width;
-        f32x4 a = {0.f, 0.f, 0.f, 0.f};
-        for (int s = 0; s < parts; ++s) a += part_load4<true>(P, s * slab + row + i);
-#pragma unroll
-        for (int j = 0; j < V; ++j) v[k][j] = bf2f(f2bf(a[j & 3]));
-      } else {
-        ldv<V>((const T*)o_ + row + i, v[k]);
-      }
-      ldv<V>(xr + i, xv[k]);
-      ldv<V>((const T*)wp_ + i, w[k]);
-      ldv<V>((const T*)bp_ + i, b[k]);
-      if (bias_) {
-        float c[V];
-        ldv<V>((const T*)bias_ + i, c);
-#pragma unroll
-        for (int j = 0; j < V; ++j) v[k][j] += c[j];
-      }
+      for (int j = 0; j < V; ++j) v[k][j] += c[j];
     }
   }
+#pragma unroll
+  for (int k = 0; k < NV; ++k)
+    if ((k * 256 + (int)threadIdx.x) * V >= width) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[k][j] = xv[k][j] = 0.f;
+    }
   float mean, inv;
   ln_stats<V, NV>(v, width, eps, red, mean, inv);
 #pragma unroll
@@ -1370,6 +1393,49 @@ __device__ __forceinline__ void append_values(const T* __restrict__ v, const T* 
   }
 }
 
+// The same for `n` (1 .. 8) consecutive tokens of the batch by one workgroup, v of token j at v + j ld.  Eight tokens that
+// fill an aligned eighth of places of one cache block leave as one piece per channel (a token alone touches a cache line
+// per channel for 2 bytes of it).
+template <typename T>
+__device__ __forceinline__ void append_value_rows(const T* __restrict__ v, long ld, const T* __restrict__ vb,
+                                                  const T* __restrict__ v_in, T* __restrict__ v_out, float lam,
+                                                  T* __restrict__ vc, const int32_t* __restrict__ slots, int n, int G, int Dv,
+                                                  int bs) {
+  const int nv = G * Dv, slot0 = slots[0];
+  bool run = n == 8 && slot0 % 8 == 0 && bs % 8 == 0;
+  for (int j = 1; run && j < 8; ++j) run = slots[j] == slot0 + j;
+  for (int e = threadIdx.x; e < nv; e += blockDim.x) {
+    const int g = e / Dv, c = e - g * Dv;
+    const float b = vb ? ldf(vb + e) : 0.f;
+    float x[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = ldf(v + (size_t)min(j, n - 1) * ld + e) + b;
+    if (v_in) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] = (1.0f - lam) * x[j] + lam * ldf(v_in + (size_t)min(j, n - 1) * nv + e);
+    }
+    if (v_out) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        if (j < n) stf(v_out + (size_t)j * nv + e, x[j]);
+    }
+    if (run) {
+      const int blk = slot0 / bs, off = slot0 - blk * bs;
+      stv<8>(vc + (((size_t)blk * G + g) * Dv + c) * bs + off, x);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        if (j >= n) break;
+        const int blk = slots[j] / bs, off = slots[j] - blk * bs;
+        stf(vc + (((size_t)blk * G + g) * Dv + c) * bs + off, x[j]);
+      }
+    }
+  }
+}
+
+// Tokens per workgroup of the value rows: one while all rows' workgroups find a CU at once, else an eighth of a block
+static int value_rows(int tokens) { return tokens <= 1024 ? 1 : 8; }
+
 // --------------------------------------------------------------------------- attention input: row norm + half-split rotation + append
 // From a fused projection row [.. | q (H D) | k (G D) | v (G Dv) | ..] (row stride ld, q at column `col0`):
 // an RMS norm over the WHOLE q projection and over the whole k projection (all heads at once, plain
@@ -1454,9 +1520,19 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
     const void* __restrict__ kw_, const float* __restrict__ freqs, int nrot, float eps, void* __restrict__ k_cache_,
     void* __restrict__ v_cache_, const int32_t* __restrict__ slot_mapping, const int32_t* __restrict__ positions, int H,
     int G, int D, int Dv, int bs, float mag, int v_from_k, const void* __restrict__ pb_, const void* __restrict__ v_in_,
-    void* __restrict__ v_out_, float lam) {
+    void* __restrict__ v_out_, float lam, int tokens, int vt) {
   __shared__ float red[32];
   extern __shared__ float csn[];                   // cos | sin of the token's nrot angles
+  const int nq = H * D, nk = G * D, nv = G * Dv;
+  const T* pb = (const T*)pb_;
+  if ((int)blockIdx.x >= tokens) {                 // value rows: vt tokens of the batch
+    const int t0 = (blockIdx.x - tokens) * vt;
+    append_value_rows<T>((const T*)qkv_ + (size_t)t0 * ld + col0 + nq + (v_from_k ? 0 : nk), ld, pb ? pb + nq + nk : nullptr,
+                         v_in_ ? (const T*)v_in_ + (size_t)t0 * nv : nullptr,
+                         v_out_ ? (T*)v_out_ + (size_t)t0 * nv : nullptr, lam, (T*)v_cache_, slot_mapping + t0,
+                         min(vt, tokens - t0), G, Dv, bs);
+    return;
+  }
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const float fpos = (float)positions[t];
   for (int i = tid; i < nrot; i += 256) {
@@ -1465,9 +1541,6 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
     csn[nrot + i] = sinf(ang) * mag;
   }
   const T* q = (const T*)qkv_ + (size_t)t * ld + col0;
-  const int nq = H * D, nk = G * D, nv = G * Dv;
-  const T* v = v_from_k ? q + nq : q + nq + nk;
-  const T* pb = (const T*)pb_;
   const bool normed = qw_ != nullptr;
   float sq = 0.f, sk = 0.f;
   if (normed) {
@@ -1494,7 +1567,6 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
   const int slot = slot_mapping[t], blk = slot / bs, off = slot - blk * bs;
   T* q_out = (T*)q_out_ + (size_t)t * nq;
   T* kc = (T*)k_cache_;
-  T* vc = (T*)v_cache_;
   for (int e = tid * 8; e < nq + nk; e += 2048) {
     const bool isq = e < nq;
     const int ee = isq ? e : e - nq;
@@ -1529,8 +1601,6 @@ __global__ void __launch_bounds__(256) sm_rownorm_rope_vec_kernel(
     if (isq) stv<8>(q_out + ee, x);
     else stv<8>(kc + (((size_t)blk * G + hd) * bs + off) * D + d, x);
   }
-  append_values<T>(v, pb ? pb + nq + nk : nullptr, v_in_ ? (const T*)v_in_ + (size_t)t * nv : nullptr,
-                   v_out_ ? (T*)v_out_ + (size_t)t * nv : nullptr, lam, vc, blk, off, G, Dv, bs);
 }
 
 void sm_rownorm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_t q_norm, uintptr_t k_norm,
@@ -1545,11 +1615,12 @@ void sm_rownorm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintptr_
   DLLM_HOST_CHECK(q_out && k_cache && v_cache && (!q_norm == !k_norm) && (nrot == 0 || freqs), "rownorm_rope arguments");
   const int esz = f32 ? 4 : 2;
   if (D % 8 == 0 && nrot % 8 == 0 && ld % 8 == 0 && col0 % 8 == 0 && qkv % (8 * esz) == 0 && q_norm % (8 * esz) == 0 &&
-      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0 && bias % (8 * esz) == 0) {
-    SM_DISPATCH(f32, sm_rownorm_rope_vec_kernel, dim3(tokens), dim3(256), 2 * (size_t)nrot * sizeof(float), stream,
+      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0 && v_cache % (8 * esz) == 0 && bias % (8 * esz) == 0) {
+    const int vt = value_rows(tokens);
+    SM_DISPATCH(f32, sm_rownorm_rope_vec_kernel, dim3(tokens + (tokens + vt - 1) / vt), dim3(256), 2 * (size_t)nrot * sizeof(float), stream,
                 (void*)q_out, (const void*)qkv, ld, col0, (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot,
                 eps, (void*)k_cache, (void*)v_cache, (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs,
-                mag, v_from_k, (const void*)bias, (const void*)v_in, (void*)v_out, lam);
+                mag, v_from_k, (const void*)bias, (const void*)v_in, (void*)v_out, lam, tokens, vt);
     return;
   }
   SM_DISPATCH(f32, sm_rownorm_rope_kernel, dim3(tokens), dim3(256), 2 * (size_t)nrot * sizeof(float), stream, (void*)q_out, (const void*)qkv, ld, col0,
@@ -1581,8 +1652,18 @@ __global__ void __launch_bounds__(256) sm_head_norm_rope_vec_kernel(
     const float* __restrict__ q_mul, float temp_coef, int temp_every, void* __restrict__ k_cache_,
     void* __restrict__ v_cache_, const int32_t* __restrict__ slot_mapping, const int32_t* __restrict__ positions, int H,
     int G, int D, int Dv, int bs, int lph, const void* __restrict__ pb_, const void* __restrict__ v_in_,
-    void* __restrict__ v_out_, float lam) {
+    void* __restrict__ v_out_, float lam, int tokens, int vt) {
   extern __shared__ float csn[];                   // cos | sin of the token's nrot angles
+  const int nq = H * D, nk = G * D, nv = G * Dv;
+  const T* pb = (const T*)pb_;
+  if ((int)blockIdx.x >= tokens) {                 // value rows: vt tokens of the batch
+    const int t0 = (blockIdx.x - tokens) * vt;
+    append_value_rows<T>((const T*)qkv_ + (size_t)t0 * ld + col0 + nq + nk, ld, pb ? pb + nq + nk : nullptr,
+                         v_in_ ? (const T*)v_in_ + (size_t)t0 * nv : nullptr,
+                         v_out_ ? (T*)v_out_ + (size_t)t0 * nv : nullptr, lam, (T*)v_cache_, slot_mapping + t0,
+                         min(vt, tokens - t0), G, Dv, bs);
+    return;
+  }
   const int t = blockIdx.x, tid = threadIdx.x, pos = positions[t];
   const float fpos = (float)pos;
   for (int i = tid; i < nrot; i += 256) {
@@ -1591,13 +1672,9 @@ __global__ void __launch_bounds__(256) sm_head_norm_rope_vec_kernel(
     csn[nrot + i] = sinf(ang);
   }
   const T* q = (const T*)qkv_ + (size_t)t * ld + col0;
-  const int nq = H * D, nk = G * D, nv = G * Dv;
-  const T* v = q + nq + nk;
-  const T* pb = (const T*)pb_;
   const int slot = slot_mapping[t], blk = slot / bs, off = slot - blk * bs;
   T* q_out = (T*)q_out_ + (size_t)t * nq;
   T* kc = (T*)k_cache_;
-  T* vc = (T*)v_cache_;
   const float qt = query_temp(pos, temp_coef, temp_every);
   const int sub = tid & (lph - 1), d = sub * 8;
   if (nrot > 0) __syncthreads();                   // uniform: csn is complete
@@ -1651,8 +1728,6 @@ __global__ void __launch_bounds__(256) sm_head_norm_rope_vec_kernel(
       stv<8>(kc + (((size_t)blk * G + (head - H)) * bs + off) * D + d, x);
     }
   }
-  append_values<T>(v, pb ? pb + nq + nk : nullptr, v_in_ ? (const T*)v_in_ + (size_t)t * nv : nullptr,
-                   v_out_ ? (T*)v_out_ + (size_t)t * nv : nullptr, lam, vc, blk, off, G, Dv, bs);
 }
 
 // The same for any head size: a wave per (token, head), the head's values in LDS.
@@ -1722,14 +1797,15 @@ void sm_head_norm_rope(uintptr_t q_out, uintptr_t qkv, long ld, int col0, uintpt
                   "head_norm_rope arguments");
   const int esz = f32 ? 4 : 2;
   if (D % 8 == 0 && D <= 512 && ld % 8 == 0 && col0 % 8 == 0 && qkv % (8 * esz) == 0 && q_norm % (8 * esz) == 0 &&
-      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0 && bias % (8 * esz) == 0) {
+      k_norm % (8 * esz) == 0 && q_out % (8 * esz) == 0 && k_cache % (8 * esz) == 0 && v_cache % (8 * esz) == 0 && bias % (8 * esz) == 0) {
     int lph = 1;
     while (8 * lph < D) lph *= 2;
-    SM_DISPATCH(f32, sm_head_norm_rope_vec_kernel, dim3(tokens), dim3(256), 2 * (size_t)nrot * sizeof(float), stream,
+    const int vt = value_rows(tokens);
+    SM_DISPATCH(f32, sm_head_norm_rope_vec_kernel, dim3(tokens + (tokens + vt - 1) / vt), dim3(256), 2 * (size_t)nrot * sizeof(float), stream,
                 (void*)q_out, (const void*)qkv, ld, col0, (const void*)q_norm, (const void*)k_norm, (const float*)freqs, nrot,
                 norm_last, eps, (const float*)q_mul, temp_coef, temp_every, (void*)k_cache, (void*)v_cache,
                 (const int32_t*)slot_mapping, (const int32_t*)positions, H, G, D, Dv, bs, lph,
-                (const void*)bias, (const void*)v_in, (void*)v_out, lam);
+                (const void*)bias, (const void*)v_in, (void*)v_out, lam, tokens, vt);
     return;
   }
   SM_DISPATCH(f32, sm_head_norm_rope_kernel, dim3(tokens, H + 2 * G), dim3(64), (size_t)D * sizeof(float), stream,

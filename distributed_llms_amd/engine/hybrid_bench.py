@@ -7,7 +7,9 @@ Zebutar (chunked attention beside a gated delta rule, SwiGLU experts) beside the
 Fekizen (window attention with averaged blocks beside gated linear attention, lightning layers, SwiGLU experts)
 beside the same Mixtral model and, for its kernels, beside Zebutar;
 Kupedra (several residual streams, distance-biased attention beside an exponentially gated matrix memory, rotated attention,
-clipped-GLU experts) beside Fekizen and the same Mixtral model.  Every step goes through the engine's StageRunner (the trace
+clipped-GLU experts) beside Fekizen and the same Mixtral model;
+Basopel (layer-normed sublayers, distance-biased windows with kept first tokens, chunked and latent attention, gelu GLUs)
+beside Tudilix and the Llama-architecture model of the same sizes.  Every step goes through the engine's StageRunner (the trace
 replayer builds the batches): one step with ``batch`` prompts of ``prompt_len`` tokens (prefill),
 then ``gen_len`` steps of one token per sequence (decode)."""
 from __future__ import annotations
@@ -160,6 +162,26 @@ def kupedra_config(size: str, vocab: int = 32000) -> ModelConfig:
                                       name=f"kupedra-{size}")
 
 
+def basopel_config(size: str, vocab: int = 32000) -> ModelConfig:
+    """Width, layer count, feed-forward size and heads of the Tudilix / Llama sizes.  Layers in turn: chunked attention
+    (chunks of 2048 positions, half of every head rotated, capped scores, sinks, head gates), distance-biased attention
+    (a window of 1024, 4 kept first tokens, 32 buckets up to 128 positions), latent attention (latents of 192 + 64 rotated
+    key dimensions, a window of 2048, element gates); the softmax layers share values."""
+    w, nl, ff, h, g, d, _nb, win = SIZES[size]
+    mlp = {"kind": "dense", "ff": ff}
+    heads = {"heads": h, "kv_heads": g, "dim": d, "vdim": d, "scale": d ** -0.5, "v_mix": True}
+    kinds = [
+        {"type": "attention_2", "mlp": mlp, "mixer": dict(heads, mask={"size": win}, softcap=30.0, rot={
+            "base": 250000.0, "dims": d // 2, "scaling": {"factor": 4.0}})},
+        {"type": "attention", "mlp": mlp, "mixer": dict(heads, mask={"size": win // 2, "keep_first": 4}, bias_max=128)},
+        {"type": "latent_attention", "mlp": mlp, "mixer": {
+            "heads": h, "dim": d, "rot_dim": d // 2, "vdim": d, "kv_rank": 192, "scale": (d + d // 2) ** -0.5,
+            "mask": {"size": win}, "rot": {"base": 500000.0, "dims": d // 2}}}]
+    return ModelConfig.from_hf_config({"architecture": "Basopel", "vocab": vocab, "width": w, "norm": {"eps": 1e-5},
+                                       "embedding": {"scale": float(w) ** 0.5}, "layers": [kinds[i % 3] for i in range(nl)]},
+                                      name=f"basopel-{size}")
+
+
 def _measure(mcfg: ModelConfig, batch: int, prompt_len: int, gen_len: int, reps: int, tmp: str, graphs: bool):
     import os
     os.makedirs(tmp, exist_ok=True)
@@ -197,14 +219,15 @@ def _measure(mcfg: ModelConfig, batch: int, prompt_len: int, gen_len: int, reps:
 
 
 MAKERS = {"tudilix": hybrid_config, "llama": llama_config, "gikovik": gikovik_config, "mixtral": mixtral_config,
-          "zebutar": zebutar_config, "fekizen": fekizen_config, "kupedra": kupedra_config}
-PAIRS = {"tudilix": "llama", "gikovik": "mixtral", "zebutar": "mixtral", "fekizen": "mixtral", "kupedra": "mixtral"}
+          "zebutar": zebutar_config, "fekizen": fekizen_config, "kupedra": kupedra_config, "basopel": basopel_config}
+PAIRS = {"tudilix": "llama", "gikovik": "mixtral", "zebutar": "mixtral", "fekizen": "mixtral", "kupedra": "mixtral",
+         "basopel": "llama"}
 
 
 def run(size: str = "2b", batch: int = 32, prompt_len: int = 1024, gen_len: int = 32, reps: int = 2,
         tmp: str = "/tmp/dllm_hybrid_bench", models=("tudilix", "llama")) -> dict:
-    """``models``: which to run, of tudilix, llama, gikovik, zebutar, fekizen, kupedra, mixtral; a layer-list model and its
-    flat counterpart (tudilix / llama, gikovik / mixtral, zebutar / mixtral, fekizen / mixtral, kupedra / mixtral) also get the ratio
+    """``models``: which to run, of tudilix, llama, gikovik, zebutar, fekizen, kupedra, basopel, mixtral; a layer-list model and its
+    flat counterpart (tudilix / llama, gikovik / mixtral, zebutar / mixtral, fekizen / mixtral, kupedra / mixtral, basopel / llama) also get the ratio
     of their throughputs (``ratios`` holds every pair that ran; ``prefill_ratio`` / ``decode_ratio`` the first)."""
     out = {"size": size, "batch": batch, "prompt_len": prompt_len, "gen_len": gen_len, "dtype": "bf16",
            "data": "synthetic (random-init weights, random token ids)"}

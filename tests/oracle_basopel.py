@@ -98,8 +98,8 @@ def softmax_attention(q, k, v, scale, keys, cap=0.0, bias=None, sink=None):
 
 
 def mix_values(v, first, lam):
-    """(1 - lam) v + lam first; ``first`` None: this is the first layer that mixes."""
-    return v if first is None else (1.0 - lam) * v + lam * first
+    """(1 - lam) v + lam first, row by row of the value projection; ``first`` None: this is the first layer that mixes."""
+    return v if first is None else (1.0 - lam) * v + lam * first.reshape(v.shape)
 
 
 # ------------------------------------------------------------------------------ mixers
