@@ -1394,7 +1394,7 @@ __device__ __forceinline__ void append_values(const T* __restrict__ v, const T* 
 }
 
 // The same for `n` (1 .. 8) consecutive tokens of the batch by one workgroup, v of token j at v + j ld.  Eight tokens that
-// fill an aligned eighth of places of one cache block leave as one piece per channel (a token alone touches a cache line
+// take eight aligned places of one cache block leave as one piece per channel (a token alone touches a cache line
 // per channel for 2 bytes of it).
 template <typename T>
 __device__ __forceinline__ void append_value_rows(const T* __restrict__ v, long ld, const T* __restrict__ vb,
@@ -1433,7 +1433,7 @@ __device__ __forceinline__ void append_value_rows(const T* __restrict__ v, long 
   }
 }
 
-// Tokens per workgroup of the value rows: one while all rows' workgroups find a CU at once, else an eighth of a block
+// Tokens per workgroup of the value rows: one while all workgroups run at once, else eight
 static int value_rows(int tokens) { return tokens <= 1024 ? 1 : 8; }
 
 // --------------------------------------------------------------------------- attention input: row norm + half-split rotation + append
